@@ -14,6 +14,10 @@ typedef _Float16 gd_half;
 typedef _Float16 gd_half8 __attribute__((ext_vector_type(8)));
 typedef _Float16 gd_half4 __attribute__((ext_vector_type(4)));
 typedef _Float16 gd_half2 __attribute__((ext_vector_type(2)));
+typedef __bf16 gd_bf16;
+typedef __bf16 gd_bf16x8 __attribute__((ext_vector_type(8)));
+typedef __bf16 gd_bf16x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 gd_bf16x2 __attribute__((ext_vector_type(2)));
 typedef float gd_float4 __attribute__((ext_vector_type(4)));
 typedef float gd_float16 __attribute__((ext_vector_type(16)));
 
@@ -48,6 +52,19 @@ __device__ __forceinline__ float gd_block_sum(float v, float *smem)
 #pragma unroll
     for (int w = 0; w < NW; ++w) t += smem[w];
     return t;
+}
+
+/* activation functions in F32 */
+__device__ __forceinline__ float gd_sigmoid_f32(float z)
+{
+    const float e = __expf(-fabsf(z)), inv = 1.0f / (1.0f + e);
+    return z >= 0.0f ? inv : e * inv;
+}
+__device__ __forceinline__ float gd_silu_f32(float z) { return z * gd_sigmoid_f32(z); }
+/* 0.5 z (1 + tanh(u)) = z sigmoid(2 u) with u = sqrt(2/pi) (z + 0.044715 z^3) */
+__device__ __forceinline__ float gd_gelu_tanh_f32(float z)
+{
+    return z * gd_sigmoid_f32(2.0f * 0.7978845608028654f * (z + 0.044715f * z * z * z));
 }
 
 /* IEEE round-to-nearest-even float -> half (v_cvt_f16_f32) */

@@ -11,23 +11,37 @@ int gd_hip_launch_linear(hipStream_t stream, const void *x, const void *w, const
                          int kn_vector_ok, int store_vector_ok, int min_workgroups, const gd_hip_rope_epilogue *rope,
                          int wide_mode, int *family);
 
+int gd_hip_launch_linear_bf16(hipStream_t stream, const void *x, const void *w, const void *bias, const void *residual,
+                              const void *norm_w, void *y, const gd_hip_linear_params *params, int vector_ok,
+                              int kn_vector_ok, int store_vector_ok, int min_workgroups, const gd_hip_rope_epilogue *rope,
+                              int wide_mode, int *family);
+int gd_hip_launch_linear_f32(hipStream_t stream, const void *x, const void *w, const void *bias, void *y,
+                             const gd_hip_linear_params *params);
+
 static gd_status project_full(gd_backend *backend, const gd_backend_matrix_view *x, const gd_backend_matrix_view *w,
                               const gd_backend_vector_view *bias, const gd_backend_matrix_view *residual,
                               const gd_backend_vector_view *norm_w, float eps, const gd_backend_matrix_view *y,
                               uint32_t w_is_nk, uint32_t epilogue, uint32_t prologue, uint32_t gated)
 {
     gd_hip_linear_params p;
-    uint32_t K;
-    int vec, kn_vec, store_vec;
+    uint32_t K, es;
+    int vec, kn_vec, store_vec, f16;
     if (backend == NULL || !gd_hip_matrix_ok(x) || !gd_hip_matrix_ok(w) || !gd_hip_matrix_ok(y) ||
         (bias != NULL && !gd_hip_vector_ok(bias)) || (residual != NULL && !gd_hip_matrix_ok(residual)) ||
         (norm_w != NULL && !gd_hip_vector_ok(norm_w)))
         return GD_ERR_INVALID_ARGUMENT;
-    if (x->dtype != GD_BACKEND_DTYPE_F16 || w->dtype != GD_BACKEND_DTYPE_F16 || y->dtype != GD_BACKEND_DTYPE_F16 ||
-        (bias != NULL && bias->dtype != GD_BACKEND_DTYPE_F16) ||
-        (residual != NULL && residual->dtype != GD_BACKEND_DTYPE_F16) ||
-        (norm_w != NULL && norm_w->dtype != GD_BACKEND_DTYPE_F16))
+    f16 = x->dtype == GD_BACKEND_DTYPE_F16;
+    if ((!f16 && x->dtype != GD_BACKEND_DTYPE_BF16 && x->dtype != GD_BACKEND_DTYPE_F32) || w->dtype != x->dtype ||
+        (y->dtype != x->dtype && !(x->dtype == GD_BACKEND_DTYPE_BF16 && y->dtype == GD_BACKEND_DTYPE_F32 && !gated)) ||
+        (bias != NULL && bias->dtype != x->dtype) || (residual != NULL && residual->dtype != x->dtype) ||
+        (norm_w != NULL && norm_w->dtype != x->dtype))
         return GD_ERR_UNSUPPORTED;
+    /* BF16 and F32 operands: [N,K] weights, bias added in F32, no prologue, no residual (linear_elem.h) */
+    if (!f16 && (!w_is_nk || prologue != GD_HIP_PRO_NONE || residual != NULL ||
+                 (bias != NULL && epilogue != GD_HIP_EPI_BIAS_F32)))
+        return GD_ERR_UNSUPPORTED;
+    if (f16 && gated > 1u) return GD_ERR_UNSUPPORTED;
+    es = (uint32_t)gd_hip_dtype_size(x->dtype);
     if (prologue == GD_HIP_PRO_SWIGLU) {
         if ((x->cols & 1u) != 0u) return GD_ERR_INVALID_ARGUMENT;
         K = x->cols / 2u;
@@ -52,9 +66,9 @@ static gd_status project_full(gd_backend *backend, const gd_backend_matrix_view 
     p.M = y->rows;
     p.N = y->cols;
     p.K = K;
-    p.ldx = (uint32_t)(x->row_bytes / 2u);
-    p.ldw = (uint32_t)(w->row_bytes / 2u);
-    p.ldy = (uint32_t)(y->row_bytes / 2u);
+    p.ldx = (uint32_t)(x->row_bytes / es);
+    p.ldw = (uint32_t)(w->row_bytes / es);
+    p.ldy = (uint32_t)(y->row_bytes / gd_hip_dtype_size(y->dtype));
     p.epilogue = bias != NULL ? epilogue : GD_HIP_EPI_NONE;
     p.w_is_nk = w_is_nk;
     p.prologue = prologue;
@@ -66,15 +80,24 @@ static gd_status project_full(gd_backend *backend, const gd_backend_matrix_view 
     p.rope_freq_scale = 0.0f;
     p.force_tiles = (uint16_t)backend->linear_tiles;
     p.force_waves = (uint16_t)backend->linear_waves;
-    p.no_lds_stream = (uint32_t)backend->linear_no_lds_stream;
+    p.no_lds_stream = (uint16_t)(backend->linear_no_lds_stream != 0);
+    p.flags = 0u;
+    if (gated == 2u) p.flags |= GD_HIP_LINEAR_GELU_GATE;
+    if (y->dtype != x->dtype) p.flags |= GD_HIP_LINEAR_Y_F32;
+    if (x->dtype == GD_BACKEND_DTYPE_F32) {
+        backend->last_linear_family = GD_HIP_LINEAR_FAMILY_F32;
+        return gd_hip_finish_op(backend, gd_hip_launch_linear_f32(
+            backend->stream, gd_hip_matrix_ptr(x), gd_hip_matrix_ptr(w), bias != NULL ? gd_hip_vector_ptr(bias) : NULL,
+            gd_hip_matrix_ptr(y), &p));
+    }
     /* 16-byte fragment loads: x rows always, w rows when K-contiguous, the norm weight */
     vec = (K % 8u) == 0u && ((x->offset | x->row_bytes) & 15u) == 0u &&
           (!w_is_nk || ((w->offset | w->row_bytes) & 15u) == 0u) && (norm_w == NULL || (norm_w->offset & 15u) == 0u);
     kn_vec = !w_is_nk && (p.N % 8u) == 0u && ((w->offset | w->row_bytes) & 15u) == 0u;
     store_vec = ((y->offset | y->row_bytes) & 15u) == 0u &&
                 (residual == NULL || ((residual->offset | residual->row_bytes) & 15u) == 0u);
-    if (gated && !vec) return GD_ERR_UNSUPPORTED;
-    return gd_hip_finish_op(backend, gd_hip_launch_linear(
+    if (f16 && gated && !vec) return GD_ERR_UNSUPPORTED;
+    return gd_hip_finish_op(backend, (f16 ? gd_hip_launch_linear : gd_hip_launch_linear_bf16)(
         backend->stream, gd_hip_matrix_ptr(x), gd_hip_matrix_ptr(w), bias != NULL ? gd_hip_vector_ptr(bias) : NULL,
         residual != NULL ? gd_hip_matrix_ptr(residual) : NULL, norm_w != NULL ? gd_hip_vector_ptr(norm_w) : NULL,
         gd_hip_matrix_ptr(y), &p, vec, kn_vec, store_vec, 2 * backend->compute_units, NULL, backend->linear_wide,
@@ -127,7 +150,7 @@ gd_status gd_backend_fused_linear(gd_backend *backend, const gd_backend_matrix_v
                                   const gd_backend_matrix_view *residual, const gd_backend_vector_view *norm_weight,
                                   const gd_backend_matrix_view *y, const gd_backend_fused_linear_args *args)
 {
-    if (args == NULL || args->bias_mode > 2u || args->prologue > 2u || args->epilogue > 1u ||
+    if (args == NULL || args->bias_mode > 2u || args->prologue > 2u || args->epilogue > 2u ||
         (args->bias_mode != 0u) != (bias != NULL))
         return GD_ERR_INVALID_ARGUMENT;
     return project_full(backend, x, w, bias, residual, norm_weight, args->eps, y, args->w_is_nk != 0u, args->bias_mode,
@@ -203,7 +226,8 @@ gd_status gd_backend_fused_qkv_rope_append(gd_backend *backend, const gd_backend
     p.rope_freq_scale = -2.0f * log2f(rope_args->theta) / (float)head_dim;
     p.force_tiles = (uint16_t)backend->linear_tiles;
     p.force_waves = (uint16_t)backend->linear_waves;
-    p.no_lds_stream = (uint32_t)backend->linear_no_lds_stream;
+    p.no_lds_stream = (uint16_t)(backend->linear_no_lds_stream != 0);
+    p.flags = 0u;
     r.rope_pos = (const int32_t *)gd_hip_view_ptr(pos_ids);
     r.cache_pos = (const int32_t *)gd_hip_view_ptr(cache_pos);
     r.q = gd_hip_view_ptr(q);
@@ -291,7 +315,8 @@ gd_status gd_backend_linear_qkv_rope_packed(gd_backend *backend, const gd_backen
     p.rope_freq_scale = 0.0f;
     p.force_tiles = (uint16_t)backend->linear_tiles;
     p.force_waves = (uint16_t)backend->linear_waves;
-    p.no_lds_stream = (uint32_t)backend->linear_no_lds_stream;
+    p.no_lds_stream = (uint16_t)(backend->linear_no_lds_stream != 0);
+    p.flags = 0u;
     head_rows = gd_hip_linear_tile_rope_head_rows(p.M, p.N, backend->compute_units);
     if (head_rows != 0u) {
         gd_hip_linear_params head = p;
@@ -333,9 +358,9 @@ gd_status gd_backend_linear_qkv_rope_packed(gd_backend *backend, const gd_backen
 /* Which kernel family the last projection call on this backend took: "stream", "wide", "tile" or "scalar". */
 gd_status gd_backend_linear_last_kernel(gd_backend *backend, char *out, size_t capacity)
 {
-    static const char *const names[] = {NULL, "stream", "wide", "tile", "scalar"};
+    static const char *const names[] = {NULL, "stream", "wide", "tile", "scalar", "f32"};
     if (backend == NULL || out == NULL || capacity == 0u) return GD_ERR_INVALID_ARGUMENT;
-    if (backend->last_linear_family < 1 || backend->last_linear_family > 4) return GD_ERR_BAD_STATE;
+    if (backend->last_linear_family < 1 || backend->last_linear_family > 5) return GD_ERR_BAD_STATE;
     snprintf(out, capacity, "%s", names[backend->last_linear_family]);
     return GD_OK;
 }

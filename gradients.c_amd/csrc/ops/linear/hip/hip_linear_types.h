@@ -12,6 +12,10 @@
 #define GD_HIP_PRO_SWIGLU 1u      /* a = half(x[:, k] * silu(x[:, K + k])), x has 2K columns */
 #define GD_HIP_PRO_RMS_NORM 2u    /* a = half(x[:, k] * norm_w[k] * rsqrt(mean(x^2) + eps)) */
 
+/* flags */
+#define GD_HIP_LINEAR_GELU_GATE 1u /* swiglu_cols: the gate function is gelu (tanh form) instead of silu */
+#define GD_HIP_LINEAR_Y_F32 2u     /* y is F32 (BF16 operands) */
+
 typedef struct gd_hip_linear_params {
     uint32_t M, N, K;
     uint32_t ldx, ldw, ldy; /* row pitch in elements */
@@ -31,7 +35,8 @@ typedef struct gd_hip_linear_params {
      * behind it fill exactly one 128-byte line of the argument segment.  Keep the structure at 76 bytes: with the
      * tile count on a second line every projection launch of a decode step took 0.06 us longer. */
     uint16_t force_tiles, force_waves; /* tunables: 0 = automatic */
-    uint32_t no_lds_stream;            /* tunable: 1 = weights always go straight to registers */
+    uint16_t no_lds_stream;            /* tunable: 1 = weights always go straight to registers */
+    uint16_t flags;                    /* GD_HIP_LINEAR_* below; the BF16 and F32 kernels only, 0 for F16 operands */
 } gd_hip_linear_params;
 #ifdef __cplusplus
 static_assert(sizeof(gd_hip_linear_params) == 76, "the few-row kernel's arguments must stay within one 128-byte line");
@@ -44,6 +49,7 @@ _Static_assert(sizeof(gd_hip_linear_params) == 76, "the few-row kernel's argumen
 #define GD_HIP_LINEAR_FAMILY_WIDE 2   /* few rows, whole-line weight stream through an LDS ring (linear_wide_kernel.h) */
 #define GD_HIP_LINEAR_FAMILY_TILE 3   /* 128 rows and more, LDS-tiled MFMA kernel (linear_tile.hip) */
 #define GD_HIP_LINEAR_FAMILY_SCALAR 4 /* unaligned operands */
+#define GD_HIP_LINEAR_FAMILY_F32 5    /* F32 operands (linear_f32.hip) */
 
 /* destinations of the rope + append epilogue: q [M,H,D]; caches [M,Tmax,H,D]; positions I32 [M] */
 typedef struct gd_hip_rope_epilogue {

@@ -31,14 +31,32 @@
 
 /* Any shape or alignment: one thread per output, F32 dot product.  Correctness path only. */
 __global__ void __launch_bounds__(256)
-gd_linear_scalar_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__ w,
-                        const gd_half *__restrict__ bias, const gd_half *__restrict__ residual,
-                        const gd_half *__restrict__ norm_w, gd_half *__restrict__ y, gd_hip_linear_params p)
+gd_linear_scalar_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__ w,
+                        const gd_elem *__restrict__ bias, const gd_elem *__restrict__ residual,
+                        const gd_elem *__restrict__ norm_w, gd_elem *__restrict__ y, gd_hip_linear_params p)
 {
     const uint64_t gid = (uint64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (gid >= (uint64_t)p.M * p.N) return;
+#if GD_LINEAR_IS_BF16
+    {
+        const uint32_t m = (uint32_t)(gid / p.N), n = (uint32_t)(gid % p.N);
+        const gd_elem *xr = x + (size_t)m * p.ldx, *wr = w + (size_t)n * p.ldw;
+        float v = 0.f, g = 0.f;
+        for (uint32_t k = 0; k < p.K; ++k) v = fmaf((float)xr[k], (float)wr[k], v);
+        if (p.epilogue == GD_HIP_EPI_BIAS_F32) v += (float)bias[n];
+        if (p.swiglu_cols != 0u) {
+            const gd_elem *gr = w + (size_t)(p.swiglu_cols + n) * p.ldw;
+            for (uint32_t k = 0; k < p.K; ++k) g = fmaf((float)xr[k], (float)gr[k], g);
+            if (p.epilogue == GD_HIP_EPI_BIAS_F32) g += (float)bias[p.swiglu_cols + n];
+            v = gd_lin_gated(v, g, p.flags);
+        }
+        if (p.flags & GD_HIP_LINEAR_Y_F32) reinterpret_cast<float *>(y)[(size_t)m * p.ldy + n] = v;
+        else y[(size_t)m * p.ldy + n] = (gd_elem)v;
+        return;
+    }
+#endif
     const uint32_t m = (uint32_t)(gid / p.N), n = (uint32_t)(gid % p.N);
-    const gd_half *xr = x + (size_t)m * p.ldx;
+    const gd_elem *xr = x + (size_t)m * p.ldx;
     float inv = 1.f;
     if (p.prologue == GD_HIP_PRO_RMS_NORM) {
         float ss = 0.f;
@@ -47,29 +65,31 @@ gd_linear_scalar_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
     }
     float acc = 0.f;
     for (uint32_t k = 0; k < p.K; ++k) {
-        gd_half a = xr[k];
-        if (p.prologue == GD_HIP_PRO_SWIGLU) a = (gd_half)((float)a * gd_lin_silu((float)xr[p.K + k]));
-        if (p.prologue == GD_HIP_PRO_RMS_NORM) a = (gd_half)((float)a * (float)norm_w[k] * inv);
-        const gd_half b = p.w_is_nk ? w[(size_t)n * p.ldw + k] : w[(size_t)k * p.ldw + n];
+        gd_elem a = xr[k];
+        if (p.prologue == GD_HIP_PRO_SWIGLU) a = (gd_elem)((float)a * gd_lin_silu((float)xr[p.K + k]));
+        if (p.prologue == GD_HIP_PRO_RMS_NORM) a = (gd_elem)((float)a * (float)norm_w[k] * inv);
+        const gd_elem b = p.w_is_nk ? w[(size_t)n * p.ldw + k] : w[(size_t)k * p.ldw + n];
         acc = fmaf((float)a, (float)b, acc);
     }
-    gd_half h;
-    if (p.epilogue == GD_HIP_EPI_BIAS_F32) h = (gd_half)(acc + (float)bias[n]);
-    else if (p.epilogue == GD_HIP_EPI_BIAS_F16) h = (gd_half)acc + bias[n];
-    else h = (gd_half)acc;
+    gd_elem h;
+    if (p.epilogue == GD_HIP_EPI_BIAS_F32) h = (gd_elem)(acc + (float)bias[n]);
+    else if (p.epilogue == GD_HIP_EPI_BIAS_F16) h = (gd_elem)acc + bias[n];
+    else h = (gd_elem)acc;
     if (p.has_residual) h = residual[(size_t)m * p.ldr + n] + h;
     y[(size_t)m * p.ldy + n] = h;
 }
 
+#if !GD_LINEAR_IS_BF16
 /* linear_lds.hip: gd_linear_stream_kernel<4, 8, [N,K], rms_norm, resident, LDS stream> */
 extern "C" void gd_hip_launch_linear_lds(hipStream_t stream, const void *x, const void *w, const void *bias,
                                          const void *residual, const void *norm_w, void *y,
                                          const gd_hip_linear_params *p, uint32_t n_tiles,
                                          const gd_hip_rope_epilogue *rope, uint32_t grid_x, uint32_t grid_y);
+#endif
 
 template <int NT, int WAVES>
-static void launch_stream(hipStream_t stream, const gd_half *x, const gd_half *w, const gd_half *bias,
-                          const gd_half *residual, const gd_half *norm_w, gd_half *y, const gd_hip_linear_params &p,
+static void launch_stream(hipStream_t stream, const gd_elem *x, const gd_elem *w, const gd_elem *bias,
+                          const gd_elem *residual, const gd_elem *norm_w, gd_elem *y, const gd_hip_linear_params &p,
                           const gd_hip_rope_epilogue &rope)
 {
     const bool paired = p.swiglu_cols != 0u || p.rope_head_dim != 0u;
@@ -80,6 +100,10 @@ static void launch_stream(hipStream_t stream, const gd_half *x, const gd_half *w
     /* the whole K slice of a wavefront fits the resident registers (8 steps of 32) */
     const bool res = ((p.K + 31u) / 32u + WAVES - 1u) / WAVES <= 8u;
 #define GD_GO(NK, PRO, RES) gd_linear_stream_kernel<NT, WAVES, NK, PRO, RES, false><<<grid, threads, 0, stream>>>(x, w, bias, residual, norm_w, y, p, n_tiles, rope)
+#if GD_LINEAR_IS_BF16
+    GD_GO(true, GD_HIP_PRO_NONE, false);
+    (void)res;
+#else
     if (p.w_is_nk) {
         if (p.prologue == GD_HIP_PRO_SWIGLU) GD_GO(true, GD_HIP_PRO_SWIGLU, false);
         else if (p.prologue == GD_HIP_PRO_RMS_NORM) {
@@ -96,16 +120,17 @@ static void launch_stream(hipStream_t stream, const gd_half *x, const gd_half *w
         else if (p.prologue == GD_HIP_PRO_RMS_NORM) { if (res) GD_GO(false, GD_HIP_PRO_RMS_NORM, true); else GD_GO(false, GD_HIP_PRO_RMS_NORM, false); }
         else GD_GO(false, GD_HIP_PRO_NONE, false);
     }
+#endif
 #undef GD_GO
 }
 
 /* linear_wide.hip: the projections of the wide decoders (megabytes of [N,K] weights, fewer than 128 rows) */
-extern "C" int gd_hip_try_launch_linear_wide(hipStream_t stream, const void *x, const void *w, const void *bias,
+extern "C" int GD_LINEAR_FN(gd_hip_try_launch_linear_wide)(hipStream_t stream, const void *x, const void *w, const void *bias,
                                              const void *residual, const void *norm_w, void *y,
                                              const gd_hip_linear_params *params, const gd_hip_rope_epilogue *rope_epilogue,
                                              uint64_t min_bytes, uint32_t tiles, uint32_t units);
 
-extern "C" int gd_hip_launch_linear_tile(hipStream_t stream, const void *x, const void *w, const void *bias,
+extern "C" int GD_LINEAR_FN(gd_hip_launch_linear_tile)(hipStream_t stream, const void *x, const void *w, const void *bias,
                                          const void *residual, const void *norm_w, void *y,
                                          const gd_hip_linear_params *params, int big_tiles, int vector_store,
                                          int compute_units);
@@ -113,7 +138,7 @@ extern "C" int gd_hip_launch_linear_tile(hipStream_t stream, const void *x, cons
 /* vector_ok: K % 8 == 0 and every pointer / pitch allows 16-byte fragment loads (for w only when it is [N,K]);
  * kn_vector_ok: w stored [K,N] with N % 8 == 0 and 16-byte aligned rows; store_vector_ok: y (and the residual)
  * rows allow 16-byte accesses.  min_workgroups: about two per compute unit.  wide_mode: see below. */
-extern "C" int gd_hip_launch_linear(hipStream_t stream, const void *x, const void *w, const void *bias,
+extern "C" int GD_LINEAR_FN(gd_hip_launch_linear)(hipStream_t stream, const void *x, const void *w, const void *bias,
                                     const void *residual, const void *norm_w, void *y,
                                     const gd_hip_linear_params *params, int vector_ok, int kn_vector_ok,
                                     int store_vector_ok, int min_workgroups, const gd_hip_rope_epilogue *rope_epilogue,
@@ -124,24 +149,24 @@ extern "C" int gd_hip_launch_linear(hipStream_t stream, const void *x, const voi
     const gd_hip_rope_epilogue no_rope = {nullptr, nullptr, nullptr, nullptr, nullptr};
     const gd_hip_rope_epilogue &rope = rope_epilogue != nullptr ? *rope_epilogue : no_rope;
     const gd_hip_linear_params &p = *params;
-    const gd_half *xp = (const gd_half *)x, *wp = (const gd_half *)w, *bp = (const gd_half *)bias;
-    const gd_half *rp = (const gd_half *)residual, *np = (const gd_half *)norm_w;
-    gd_half *yp = (gd_half *)y;
+    const gd_elem *xp = (const gd_elem *)x, *wp = (const gd_elem *)w, *bp = (const gd_elem *)bias;
+    const gd_elem *rp = (const gd_elem *)residual, *np = (const gd_elem *)norm_w;
+    gd_elem *yp = (gd_elem *)y;
     if (p.M == 0 || p.N == 0) return (int)hipSuccess;
     if (!vector_ok || p.K == 0 || (!p.w_is_nk && !kn_vector_ok)) {
         const uint64_t total = (uint64_t)p.M * p.N;
         gd_linear_scalar_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(xp, wp, bp, rp, np, yp, p);
         *family = GD_HIP_LINEAR_FAMILY_SCALAR;
-    } else if (p.M >= 128u && (p.w_is_nk || kn_vector_ok) && p.rope_head_dim == 0u) {
+    } else if (p.M >= 128u && (p.w_is_nk || kn_vector_ok) && p.rope_head_dim == 0u && !(p.flags & GD_HIP_LINEAR_Y_F32)) {
         /* matrix-core bound: LDS-tiled kernel; the 256 x 256 tile once it still gives every compute unit
          * a workgroup, the 128 x 128 tile below that */
         const uint32_t out_cols = p.swiglu_cols != 0u ? 128u : 256u; /* output columns of a 256-wide weight tile */
         const uint64_t big = (uint64_t)((p.M + 255u) / 256u) * ((p.N + out_cols - 1u) / out_cols);
         const uint32_t units = min_workgroups > 0 ? (uint32_t)min_workgroups / 2u : 256u;
         *family = GD_HIP_LINEAR_FAMILY_TILE;
-        return gd_hip_launch_linear_tile(stream, x, w, bias, residual, norm_w, y, params, big >= units, store_vector_ok, (int)units);
+        return GD_LINEAR_FN(gd_hip_launch_linear_tile)(stream, x, w, bias, residual, norm_w, y, params, big >= units, store_vector_ok, (int)units);
     } else if (wide_mode != 0 && p.w_is_nk &&
-               gd_hip_try_launch_linear_wide(stream, x, w, bias, residual, norm_w, y, params, rope_epilogue,
+               GD_LINEAR_FN(gd_hip_try_launch_linear_wide)(stream, x, w, bias, residual, norm_w, y, params, rope_epilogue,
                                              wide_mode > 0 ? 0u : (4ull << 20), p.force_tiles,
                                              min_workgroups > 0 ? (uint32_t)min_workgroups / 2u : 256u)) {
         /* weight matrices of megabytes: the kernel built around the weight stream (wide_mode: 0 never, 1 whenever it

@@ -13,6 +13,6 @@ extern "C" void gd_hip_launch_linear_lds(hipStream_t stream, const void *x, cons
                                          const gd_hip_rope_epilogue *rope, uint32_t grid_x, uint32_t grid_y)
 {
     gd_linear_stream_kernel<4, 8, true, GD_HIP_PRO_RMS_NORM, true, true><<<dim3(grid_x, grid_y), 8 * 64, 0, stream>>>(
-        (const gd_half *)x, (const gd_half *)w, (const gd_half *)bias, (const gd_half *)residual,
-        (const gd_half *)norm_w, (gd_half *)y, *p, n_tiles, *rope);
+        (const gd_elem *)x, (const gd_elem *)w, (const gd_elem *)bias, (const gd_elem *)residual,
+        (const gd_elem *)norm_w, (gd_elem *)y, *p, n_tiles, *rope);
 }

@@ -9,6 +9,7 @@
 #define GD_LINEAR_STREAM_KERNEL_H
 #include "../../_shared/hip_device.h"
 #include "hip_linear_types.h"
+#include "linear_elem.h"
 #include "../../qkv_split_rope/hip/rope_device.h"
 #include <type_traits>
 
@@ -32,9 +33,9 @@ __device__ __forceinline__ void gd_lin_load_lds16(const unsigned char *uniform_b
 
 template <int NT, int WAVES, bool W_NK, int PRO, bool RES, bool LDS_STREAM>
 __global__ void __launch_bounds__(WAVES * 64)
-gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__ w,
-                        const gd_half *__restrict__ bias, const gd_half *__restrict__ residual,
-                        const gd_half *__restrict__ norm_w, gd_half *__restrict__ y, gd_hip_linear_params p,
+gd_linear_stream_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__ w,
+                        const gd_elem *__restrict__ bias, const gd_elem *__restrict__ residual,
+                        const gd_elem *__restrict__ norm_w, gd_elem *__restrict__ y, gd_hip_linear_params p,
                         uint32_t n_tiles, gd_hip_rope_epilogue rope)
 {
     constexpr int U = NT >= 4 ? 2 : 4;  /* K steps per register set; two sets alternate */
@@ -45,7 +46,7 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
     __shared__ float s_inv[16];
     __shared__ float s_part[WAVES][16];
     /* w stored [K,N]: a 32(k) x COLS(n) tile per wavefront, turned by the transposing LDS read */
-    __shared__ __align__(16) gd_half s_tr[W_NK ? 1 : WAVES][W_NK ? 8 : 32 * COLS];
+    __shared__ __align__(16) gd_elem s_tr[W_NK ? 1 : WAVES][W_NK ? 8 : 32 * COLS];
     /* Weight stream through LDS (long-K [N,K] projections behind an rms_norm whose activation slice is resident:
      * the qkv, up/gate and LM-head projections of the wide decoders).  A load that goes straight to registers must
      * follow the MFMA operand layout, 4 lanes = 64 bytes per weight row and instruction, and such half-line requests
@@ -87,7 +88,7 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
      * more dependent round trip at the end of a kernel that is a chain of round trips. */
     constexpr int NTO_MAX = NT >= 2 ? NT : 1; /* output column tiles of the plain form (the paired forms have NT / 2) */
     constexpr int EPT = (NTO_MAX * 256 + WAVES * 64 - 1) / (WAVES * 64);
-    gd_half pf_b1[EPT], pf_b2[EPT], pf_res[EPT];
+    gd_elem pf_b1[EPT], pf_b2[EPT], pf_res[EPT];
     int32_t pf_pos[EPT], pf_cpos[EPT];
 #pragma unroll
     for (int i = 0; i < EPT; ++i) {
@@ -95,7 +96,7 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
         const int j = idx >> 8, rl = idx & 63, rr = (idx >> 6) & 3;
         const uint32_t col = min(n0 + 16u * j + (rl & 15), p.N - 1u);
         const uint32_t row = min(m0 + 4u * (rl >> 4) + rr, p.M - 1u);
-        pf_b1[i] = pf_b2[i] = pf_res[i] = (gd_half)0.f;
+        pf_b1[i] = pf_b2[i] = pf_res[i] = (gd_elem)0.f;
         pf_pos[i] = pf_cpos[i] = 0;
         if (idx < (gated ? NT / 2 : NT) * 256) {
             if (p.epilogue != GD_HIP_EPI_NONE) {
@@ -115,11 +116,11 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
     const uint32_t per_wave = (ksteps + WAVES - 1u) / WAVES;
     const uint32_t s_begin = wave * per_wave, s_end = min(s_begin + per_wave, ksteps);
 
-    gd_half8 bf[2][U][NT];
-    gd_half8 af[2][RES ? 1 : U], zf[2][PRO == GD_HIP_PRO_SWIGLU ? U : 1], nf[2][(PRO == GD_HIP_PRO_RMS_NORM && !RES) ? U : 1];
-    gd_half8 ar[RES ? RES_STEPS : 1], nr[(RES && PRO == GD_HIP_PRO_RMS_NORM) ? RES_STEPS : 1];
-    const gd_half8 zero8 = (gd_half8)(gd_half)0.f;
-    const gd_half *xrow = x + (size_t)mrow * p.ldx;
+    gd_elem8 bf[2][U][NT];
+    gd_elem8 af[2][RES ? 1 : U], zf[2][PRO == GD_HIP_PRO_SWIGLU ? U : 1], nf[2][(PRO == GD_HIP_PRO_RMS_NORM && !RES) ? U : 1];
+    gd_elem8 ar[RES ? RES_STEPS : 1], nr[(RES && PRO == GD_HIP_PRO_RMS_NORM) ? RES_STEPS : 1];
+    const gd_elem8 zero8 = (gd_elem8)(gd_elem)0.f;
+    const gd_elem *xrow = x + (size_t)mrow * p.ldx;
 
     /* Fast path (whole steps of 32, byte offsets that fit 32 bits, all columns of a [K,N] tile in range): the
      * loads carry no guards and take a scalar base that advances with the step plus one per-lane offset computed
@@ -156,13 +157,13 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
             if (FULL) {
                 const unsigned char *ws = wb + (size_t)(s0 + u) * wstep;
 #pragma unroll
-                for (int j = 0; j < NT; ++j) bf[set][u][j] = *reinterpret_cast<const gd_half8 *>(ws + woff[j]);
+                for (int j = 0; j < NT; ++j) bf[set][u][j] = *reinterpret_cast<const gd_elem8 *>(ws + woff[j]);
                 if (!RES) {
                     const unsigned char *xs = xb + (size_t)(s0 + u) * 64u;
-                    af[set][u] = *reinterpret_cast<const gd_half8 *>(xs + xoff);
-                    if (PRO == GD_HIP_PRO_SWIGLU) zf[set][u] = *reinterpret_cast<const gd_half8 *>(xs + (size_t)p.K * 2u + xoff);
+                    af[set][u] = *reinterpret_cast<const gd_elem8 *>(xs + xoff);
+                    if (PRO == GD_HIP_PRO_SWIGLU) zf[set][u] = *reinterpret_cast<const gd_elem8 *>(xs + (size_t)p.K * 2u + xoff);
                     if (PRO == GD_HIP_PRO_RMS_NORM)
-                        nf[set][u] = *reinterpret_cast<const gd_half8 *>(nb + (size_t)(s0 + u) * 64u + (uint32_t)lg * 16u);
+                        nf[set][u] = *reinterpret_cast<const gd_elem8 *>(nb + (size_t)(s0 + u) * 64u + (uint32_t)lg * 16u);
                 }
                 continue;
             }
@@ -177,19 +178,19 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
                     const uint32_t n = (gated && j >= NT / 2)
                                            ? pair_offset + min(n0 + 16u * (uint32_t)(j - NT / 2) + (uint32_t)li, p.N - 1u)
                                            : min(n0 + 16u * (uint32_t)j + (uint32_t)li, p.N - 1u);
-                    if (kok) bf[set][u][j] = *reinterpret_cast<const gd_half8 *>(w + (size_t)n * p.ldw + k);
+                    if (kok) bf[set][u][j] = *reinterpret_cast<const gd_elem8 *>(w + (size_t)n * p.ldw + k);
                 } else {
                     /* load j fetches k-rows j*32/NT .. of the 32 x COLS tile: 2*NT chunks of 8 columns per row */
                     const uint32_t kr = (s0 + u) * 32u + (uint32_t)j * (32u / NT) + (uint32_t)lane / (2u * NT);
                     const uint32_t nc = n0 + ((uint32_t)lane % (2u * NT)) * 8u;
                     if (sok && kr < p.K && nc < p.N)
-                        bf[set][u][j] = *reinterpret_cast<const gd_half8 *>(w + (size_t)kr * p.ldw + nc);
+                        bf[set][u][j] = *reinterpret_cast<const gd_elem8 *>(w + (size_t)kr * p.ldw + nc);
                 }
             }
             if (!RES) {
-                af[set][u] = kok ? *reinterpret_cast<const gd_half8 *>(xrow + k) : zero8;
-                if (PRO == GD_HIP_PRO_SWIGLU) zf[set][u] = kok ? *reinterpret_cast<const gd_half8 *>(xrow + p.K + k) : zero8;
-                if (PRO == GD_HIP_PRO_RMS_NORM) nf[set][u] = kok ? *reinterpret_cast<const gd_half8 *>(norm_w + k) : zero8;
+                af[set][u] = kok ? *reinterpret_cast<const gd_elem8 *>(xrow + k) : zero8;
+                if (PRO == GD_HIP_PRO_SWIGLU) zf[set][u] = kok ? *reinterpret_cast<const gd_elem8 *>(xrow + p.K + k) : zero8;
+                if (PRO == GD_HIP_PRO_RMS_NORM) nf[set][u] = kok ? *reinterpret_cast<const gd_elem8 *>(norm_w + k) : zero8;
             }
         }
     };
@@ -209,36 +210,36 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
         constexpr int base = decltype(base_tag)::value;
 #pragma unroll
         for (int u = 0; u < U; ++u) {
-            gd_half8 a = RES ? ar[(base + u) < RES_STEPS ? (base + u) : 0] : af[set][u];
+            gd_elem8 a = RES ? ar[(base + u) < RES_STEPS ? (base + u) : 0] : af[set][u];
             if (PRO == GD_HIP_PRO_SWIGLU) {
 #pragma unroll
-                for (int e = 0; e < 8; ++e) a[e] = (gd_half)((float)a[e] * gd_lin_silu((float)zf[set][u][e]));
+                for (int e = 0; e < 8; ++e) a[e] = (gd_elem)((float)a[e] * gd_lin_silu((float)zf[set][u][e]));
             }
             if (PRO == GD_HIP_PRO_RMS_NORM) {
-                const gd_half8 nw = RES ? nr[(base + u) < RES_STEPS ? (base + u) : 0] : nf[set][u];
+                const gd_elem8 nw = RES ? nr[(base + u) < RES_STEPS ? (base + u) : 0] : nf[set][u];
 #pragma unroll
-                for (int e = 0; e < 8; ++e) a[e] = (gd_half)((float)a[e] * (float)nw[e] * minv);
+                for (int e = 0; e < 8; ++e) a[e] = (gd_elem)((float)a[e] * (float)nw[e] * minv);
             }
             if (!W_NK) {
-                gd_half *tr = &s_tr[wave][0];
+                gd_elem *tr = &s_tr[wave][0];
 #pragma unroll
                 for (int j = 0; j < NT; ++j)
-                    *reinterpret_cast<gd_half8 *>(tr + ((uint32_t)j * (32u / NT) + (uint32_t)lane / (2u * NT)) * COLS +
+                    *reinterpret_cast<gd_elem8 *>(tr + ((uint32_t)j * (32u / NT) + (uint32_t)lane / (2u * NT)) * COLS +
                                                   ((uint32_t)lane % (2u * NT)) * 8u) = bf[set][u][j];
             }
 #pragma unroll
             for (int j = 0; j < NT; ++j) {
-                gd_half8 b = bf[set][u][j];
+                gd_elem8 b = bf[set][u][j];
                 if (!W_NK) {
                     /* lane q + 4e of a 16-lane group addresses k-row 8*lg + e (+4), columns 4q .. 4q+3 of column tile j;
                      * lane i then receives column i of four consecutive k-rows */
-                    const gd_half *src = &s_tr[wave][0] + (8 * lg + ((lane >> 2) & 3)) * COLS + 16 * j + (lane & 3) * 4;
-                    union { gd_short4 s[2]; gd_half8 h; } t2;
+                    const gd_elem *src = &s_tr[wave][0] + (8 * lg + ((lane >> 2) & 3)) * COLS + 16 * j + (lane & 3) * 4;
+                    union { gd_short4 s[2]; gd_elem8 h; } t2;
                     t2.s[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) gd_short4 *)src);
                     t2.s[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) gd_short4 *)(src + 4 * COLS));
                     b = t2.h;
                 }
-                acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, acc[j], 0, 0, 0);
+                acc[j] = GD_MFMA_16X16X32(a, b, acc[j]);
             }
         }
     };
@@ -282,17 +283,17 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
         if (fast && s_begin + (uint32_t)RES_STEPS <= s_end) {
 #pragma unroll
             for (int r = 0; r < RES_STEPS; ++r) {
-                ar[r] = *reinterpret_cast<const gd_half8 *>(xb + (size_t)(s_begin + r) * 64u + xoff);
+                ar[r] = *reinterpret_cast<const gd_elem8 *>(xb + (size_t)(s_begin + r) * 64u + xoff);
                 if (PRO == GD_HIP_PRO_RMS_NORM)
-                    nr[r] = *reinterpret_cast<const gd_half8 *>(nb + (size_t)(s_begin + r) * 64u + (uint32_t)lg * 16u);
+                    nr[r] = *reinterpret_cast<const gd_elem8 *>(nb + (size_t)(s_begin + r) * 64u + (uint32_t)lg * 16u);
             }
         } else {
 #pragma unroll
             for (int r = 0; r < RES_STEPS; ++r) {
                 const uint32_t k = (s_begin + r) * 32u + lg * 8u;
                 const bool kok = (s_begin + r) < s_end && k < p.K;
-                ar[r] = kok ? *reinterpret_cast<const gd_half8 *>(xrow + k) : zero8;
-                if (PRO == GD_HIP_PRO_RMS_NORM) nr[r] = kok ? *reinterpret_cast<const gd_half8 *>(norm_w + k) : zero8;
+                ar[r] = kok ? *reinterpret_cast<const gd_elem8 *>(xrow + k) : zero8;
+                if (PRO == GD_HIP_PRO_RMS_NORM) nr[r] = kok ? *reinterpret_cast<const gd_elem8 *>(norm_w + k) : zero8;
             }
         }
         /* the second register set is requested here too: behind the barrier of the row norms its round trip would
@@ -316,10 +317,10 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
         /* row norms by a separate pass over x: one wavefront per row, 8 halfs per lane and trip */
         for (uint32_t r = wave; r < 16u; r += WAVES) {
             const uint32_t row = min(m0 + r, p.M - 1u);
-            const gd_half *xr = x + (size_t)row * p.ldx;
+            const gd_elem *xr = x + (size_t)row * p.ldx;
             float ss = 0.f;
             for (uint32_t k = lane * 8u; k < p.K; k += 512u) {
-                const gd_half8 v = *reinterpret_cast<const gd_half8 *>(xr + k);
+                const gd_elem8 v = *reinterpret_cast<const gd_elem8 *>(xr + k);
 #pragma unroll
                 for (int e = 0; e < 8; ++e) ss = fmaf((float)v[e], (float)v[e], ss);
             }
@@ -341,11 +342,11 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
 #pragma unroll
         for (int r = 0; r < RES_STEPS; ++r) {
 #pragma unroll
-            for (int e = 0; e < 8; ++e) ar[r][e] = (gd_half)((float)ar[r][e] * (float)nr[r][e] * minv);
+            for (int e = 0; e < 8; ++e) ar[r][e] = (gd_elem)((float)ar[r][e] * (float)nr[r][e] * minv);
         }
         /* group g is read from its slot while the MFMAs of group g-1 run; the slot of g-1 is refilled only behind
          * those MFMAs, which could not issue before its reads had returned */
-        gd_half8 f0, f1, pf0 = zero8, pf1 = zero8;
+        gd_elem8 f0, f1, pf0 = zero8, pf1 = zero8;
 #pragma unroll
         for (int g = 0; g <= NG; ++g) {
             if (g < NG) {
@@ -361,13 +362,13 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
                 else if (later == 1) asm volatile("s_waitcnt vmcnt(2)" ::: "memory");
                 else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
                 const unsigned char *slot = ring + (g % RING) * 2048;
-                f0 = *reinterpret_cast<const gd_half8 *>(slot + rd0);
-                f1 = *reinterpret_cast<const gd_half8 *>(slot + rd1);
+                f0 = *reinterpret_cast<const gd_elem8 *>(slot + rd0);
+                f1 = *reinterpret_cast<const gd_elem8 *>(slot + rd1);
             }
             if (g >= 1) {
                 const int q = g - 1, pair = q / NT, j = q % NT;
-                acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(ar[2 * pair], pf0, acc[j], 0, 0, 0);
-                acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(ar[2 * pair + 1], pf1, acc[j], 0, 0, 0);
+                acc[j] = GD_MFMA_16X16X32(ar[2 * pair], pf0, acc[j]);
+                acc[j] = GD_MFMA_16X16X32(ar[2 * pair + 1], pf1, acc[j]);
                 __builtin_amdgcn_sched_barrier(0);
                 if (q + RING < NG) issue_group((uint32_t)(q + RING));
             }
@@ -416,38 +417,46 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
                 v2 += sm[wv][j + NT / 2][rl][rr];
             }
             if (row < p.M && col < p.N) {
-                gd_half h1, h2;
+#if GD_LINEAR_IS_BF16
                 if (p.epilogue == GD_HIP_EPI_BIAS_F32) {
-                    h1 = (gd_half)(v1 + (float)pf_b1[i]);
-                    h2 = (gd_half)(v2 + (float)pf_b2[i]);
+                    v1 += (float)pf_b1[i];
+                    v2 += (float)pf_b2[i];
+                }
+                y[(size_t)row * p.ldy + col] = (gd_elem)gd_lin_gated(v1, v2, p.flags);
+                continue;
+#endif
+                gd_elem h1, h2;
+                if (p.epilogue == GD_HIP_EPI_BIAS_F32) {
+                    h1 = (gd_elem)(v1 + (float)pf_b1[i]);
+                    h2 = (gd_elem)(v2 + (float)pf_b2[i]);
                 } else if (p.epilogue == GD_HIP_EPI_BIAS_F16) {
-                    h1 = (gd_half)v1 + pf_b1[i];
-                    h2 = (gd_half)v2 + pf_b2[i];
+                    h1 = (gd_elem)v1 + pf_b1[i];
+                    h2 = (gd_elem)v2 + pf_b2[i];
                 } else {
-                    h1 = (gd_half)v1;
-                    h2 = (gd_half)v2;
+                    h1 = (gd_elem)v1;
+                    h2 = (gd_elem)v2;
                 }
                 if (!roped) {
-                    y[(size_t)row * p.ldy + col] = (gd_half)((float)h1 * gd_lin_silu((float)h2));
+                    y[(size_t)row * p.ldy + col] = (gd_elem)((float)h1 * gd_lin_silu((float)h2));
                 } else {
                     /* col = (section * heads + head) * head_dim + pair: q is rotated into its own tensor, k rotated and
                      * v copied into row cache_pos of the sequence's caches (skipped when that row does not exist) */
                     const uint32_t D = p.rope_head_dim, area = p.rope_heads * D;
                     const uint32_t section = col / area, within = col % area, pair = within % D;
-                    gd_half o1 = h1, o2 = h2;
+                    gd_elem o1 = h1, o2 = h2;
                     if (section < 2u) {
                         float c, sn;
                         gd_rope_cos_sin((float)pf_pos[i], pair, p.rope_freq_scale, &c, &sn);
                         gd_rope_rotate((float)h1, (float)h2, c, sn, &o1, &o2);
                     }
                     if (section == 0u) {
-                        gd_half *dst = (gd_half *)rope.q + (size_t)row * area + within;
+                        gd_elem *dst = (gd_elem *)rope.q + (size_t)row * area + within;
                         dst[0] = o1;
                         dst[D / 2u] = o2;
                     } else {
                         const int32_t cp = pf_cpos[i];
                         if (cp >= 0 && (uint32_t)cp < p.rope_tmax) {
-                            gd_half *dst = (gd_half *)(section == 1u ? rope.k_cache : rope.v_cache) +
+                            gd_elem *dst = (gd_elem *)(section == 1u ? rope.k_cache : rope.v_cache) +
                                            ((size_t)row * p.rope_tmax + (size_t)cp) * area + within;
                             dst[0] = o1;
                             dst[D / 2u] = o2;
@@ -470,10 +479,17 @@ gd_linear_stream_kernel(const gd_half *__restrict__ x, const gd_half *__restrict
 #pragma unroll
         for (int wv = 0; wv < WAVES; ++wv) v += sm[wv][j][rl][rr];
         if (row < p.M && col < p.N) {
-            gd_half h;
-            if (p.epilogue == GD_HIP_EPI_BIAS_F32) h = (gd_half)(v + (float)pf_b1[i]);
-            else if (p.epilogue == GD_HIP_EPI_BIAS_F16) h = (gd_half)v + pf_b1[i];
-            else h = (gd_half)v;
+#if GD_LINEAR_IS_BF16
+            if (p.flags & GD_HIP_LINEAR_Y_F32) {
+                if (p.epilogue == GD_HIP_EPI_BIAS_F32) v += (float)pf_b1[i];
+                reinterpret_cast<float *>(y)[(size_t)row * p.ldy + col] = v;
+                continue;
+            }
+#endif
+            gd_elem h;
+            if (p.epilogue == GD_HIP_EPI_BIAS_F32) h = (gd_elem)(v + (float)pf_b1[i]);
+            else if (p.epilogue == GD_HIP_EPI_BIAS_F16) h = (gd_elem)v + pf_b1[i];
+            else h = (gd_elem)v;
             if (p.has_residual) h = pf_res[i] + h;
             y[(size_t)row * p.ldy + col] = h;
         }

@@ -45,6 +45,7 @@
  */
 #include "../../_shared/hip_device.h"
 #include "hip_linear_types.h"
+#include "linear_elem.h"
 #include "../../qkv_split_rope/hip/rope_device.h"
 #include <type_traits>
 
@@ -77,7 +78,7 @@ extern "C" __attribute__((visibility("default"))) int gd_hip_linear_tile_timelin
 struct gd_tile_rope {
     const float *cos, *sin;
     const int32_t *cache_row; /* [M]; negative: the row's k and v go nowhere */
-    gd_half *q, *k_cache, *v_cache;
+    gd_elem *q, *k_cache, *v_cache;
     uint32_t hd;     /* heads * head_dim, a multiple of 256 */
     uint32_t half_d; /* 32 or 64 */
 };
@@ -97,10 +98,22 @@ __device__ __forceinline__ float gd_tile_silu(float z)
     return z * (z >= 0.0f ? inv : e * inv);
 }
 
+__device__ __forceinline__ float gd_tile_gated(float value, float gate, uint32_t flags)
+{
+#if GD_LINEAR_IS_BF16
+    if (flags & GD_HIP_LINEAR_GELU_GATE) {
+        const float u = 2.0f * 0.7978845608028654f * (gate + 0.044715f * gate * gate * gate);
+        const float e = __expf(-fabsf(u)), inv = __builtin_amdgcn_rcpf(1.0f + e);
+        return value * gate * (u >= 0.0f ? inv : e * inv);
+    }
+#endif
+    return value * gd_tile_silu(gate);
+}
+
 /* 16 bytes per lane from global memory straight into LDS: lane l's data lands at lds_base + 16*l.
  * Written as assembly because the compiler, not knowing which LDS stage a load fills, would otherwise
  * wait for ALL outstanding loads before every LDS read; the kernel counts them itself (s_waitcnt vmcnt). */
-__device__ __forceinline__ void gd_tile_load_lds16(const gd_half *uniform_base, uint32_t lane_byte_offset,
+__device__ __forceinline__ void gd_tile_load_lds16(const gd_elem *uniform_base, uint32_t lane_byte_offset,
                                                    uint32_t lds_byte_address)
 {
     asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2"
@@ -111,9 +124,9 @@ __device__ __forceinline__ void gd_tile_load_lds16(const gd_half *uniform_base, 
 
 template <int WM, int WN, bool W_NK, int PRO, bool ROPE = false>
 __global__ void __launch_bounds__(256)
-gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__ w, const gd_half *__restrict__ bias,
-                      const gd_half *__restrict__ residual, const gd_half *__restrict__ norm_w,
-                      gd_half *__restrict__ y, gd_hip_linear_params p, uint32_t tiles_m, uint32_t tiles_n,
+gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__ w, const gd_elem *__restrict__ bias,
+                      const gd_elem *__restrict__ residual, const gd_elem *__restrict__ norm_w,
+                      gd_elem *__restrict__ y, gd_hip_linear_params p, uint32_t tiles_m, uint32_t tiles_n,
                       uint32_t vector_store, gd_tile_rope rp)
 {
     constexpr uint32_t BM = 64u * WM, BN = 64u * WN;
@@ -121,8 +134,8 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     constexpr int B_PER = W_NK ? (int)(BN / 32) : 8; /* weight chunks per thread */
     constexpr uint32_t STAGE_BYTES = 2u * (BM + BN) * 8u * 16u; /* both stages of both operands */
     extern __shared__ __align__(16) unsigned char gd_tile_smem[];
-    gd_half8 *sA = reinterpret_cast<gd_half8 *>(gd_tile_smem); /* [2][BM*8] */
-    gd_half8 *sB = sA + 2u * BM * 8u;                          /* [2][BN*8] */
+    gd_elem8 *sA = reinterpret_cast<gd_elem8 *>(gd_tile_smem); /* [2][BM*8] */
+    gd_elem8 *sB = sA + 2u * BM * 8u;                          /* [2][BN*8] */
     unsigned char *epi = gd_tile_smem + STAGE_BYTES;           /* [64][BN] halfs */
     float *s_inv = reinterpret_cast<float *>(epi); /* [BM] row factors of rms_norm; live during the main loop only */
 
@@ -182,8 +195,8 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     constexpr bool KB_ALL = BN >= 256u; /* every thread owns a block */
     const bool kb_active = W_NK ? false : (tid < BN);
 
-    gd_half8 ra[A_PER], rz[PRO == GD_HIP_PRO_SWIGLU ? A_PER : 1], rb[B_PER], rn;
-    const gd_half8 zero8 = (gd_half8)(gd_half)0.f;
+    gd_elem8 ra[A_PER], rz[PRO == GD_HIP_PRO_SWIGLU ? A_PER : 1], rb[B_PER], rn;
+    const gd_elem8 zero8 = (gd_elem8)(gd_elem)0.f;
     const uint32_t ktiles = (p.K + GD_TILE_BK - 1u) / GD_TILE_BK;
 
     /* ---- staging through registers (any prologue, either weight layout, ragged tiles) ---------------- */
@@ -199,19 +212,19 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                 if (PRO == GD_HIP_PRO_SWIGLU) rz[i] = zero8;
             }
             if (!GUARDED || (kok && gm < p.M)) {
-                const gd_half *xr = x + (size_t)gm * p.ldx + k;
-                ra[i] = *reinterpret_cast<const gd_half8 *>(xr);
-                if (PRO == GD_HIP_PRO_SWIGLU) rz[i] = *reinterpret_cast<const gd_half8 *>(xr + p.K);
+                const gd_elem *xr = x + (size_t)gm * p.ldx + k;
+                ra[i] = *reinterpret_cast<const gd_elem8 *>(xr);
+                if (PRO == GD_HIP_PRO_SWIGLU) rz[i] = *reinterpret_cast<const gd_elem8 *>(xr + p.K);
             }
         }
-        if (PRO == GD_HIP_PRO_RMS_NORM) rn = kok ? *reinterpret_cast<const gd_half8 *>(norm_w + k) : zero8;
+        if (PRO == GD_HIP_PRO_RMS_NORM) rn = kok ? *reinterpret_cast<const gd_elem8 *>(norm_w + k) : zero8;
         if (W_NK) {
 #pragma unroll
             for (int i = 0; i < B_PER; ++i) {
                 const uint32_t gn = wrow(n0, a_r + 32u * (uint32_t)i);
                 if (GUARDED) rb[i] = zero8;
                 if (!GUARDED || (kok && wrow_ok(n0, a_r + 32u * (uint32_t)i)))
-                    rb[i] = *reinterpret_cast<const gd_half8 *>(w + (size_t)gn * p.ldw + k);
+                    rb[i] = *reinterpret_cast<const gd_elem8 *>(w + (size_t)gn * p.ldw + k);
             }
         } else {
             const uint32_t gn = n0 + kb_nc * 8u;
@@ -220,31 +233,31 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                 const uint32_t gk = kt * GD_TILE_BK + kb_j * 8u + i;
                 if (GUARDED || !KB_ALL) rb[i] = zero8;
                 if ((KB_ALL || kb_active) && (!GUARDED || (gk < p.K && gn < p.N)))
-                    rb[i] = *reinterpret_cast<const gd_half8 *>(w + (size_t)gk * p.ldw + gn);
+                    rb[i] = *reinterpret_cast<const gd_elem8 *>(w + (size_t)gk * p.ldw + gn);
             }
         }
     };
     auto store_a = [&](uint32_t stage, int i) __attribute__((always_inline)) {
-        gd_half8 *dA = sA + stage * BM * 8u;
+        gd_elem8 *dA = sA + stage * BM * 8u;
         const uint32_t r = a_r + 32u * i;
-        gd_half8 a = ra[i];
+        gd_elem8 a = ra[i];
         if (PRO == GD_HIP_PRO_SWIGLU) {
 #pragma unroll
-            for (int e = 0; e < 8; ++e) a[e] = (gd_half)((float)a[e] * gd_tile_silu((float)rz[i][e]));
+            for (int e = 0; e < 8; ++e) a[e] = (gd_elem)((float)a[e] * gd_tile_silu((float)rz[i][e]));
         }
         if (PRO == GD_HIP_PRO_RMS_NORM) {
             const float inv = s_inv[r];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) a[e] = (gd_half)((float)a[e] * (float)rn[e] * inv);
+            for (int e = 0; e < 8; ++e) a[e] = (gd_elem)((float)a[e] * (float)rn[e] * inv);
         }
         dA[gd_tile_slot(r, a_c)] = a;
     };
     auto store_b = [&](uint32_t stage, int i) __attribute__((always_inline)) {
-        gd_half8 *dB = sB + stage * BN * 8u;
+        gd_elem8 *dB = sB + stage * BN * 8u;
         if (W_NK) {
             dB[gd_tile_slot(a_r + 32u * i, a_c)] = rb[i];
         } else if (KB_ALL || kb_active) {
-            gd_half8 t; /* column i of the 8 x 8 block becomes one k-contiguous chunk */
+            gd_elem8 t; /* column i of the 8 x 8 block becomes one k-contiguous chunk */
 #pragma unroll
             for (int r = 0; r < 8; ++r) t[r] = rb[r][i];
             dB[gd_tile_slot(kb_nc * 8u + i, kb_j)] = t;
@@ -279,8 +292,8 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     constexpr uint32_t CPR = BN / 8u, RPL = 64u / CPR; /* [K,N] stage: chunks per k-row, k-rows per wavefront load */
     const uint32_t d_off_b = W_NK ? ((lane >> 3) * p.ldw + d_lane_chunk * 8u) * 2u : ((lane / CPR) * p.ldw) * 2u;
     const uint32_t d_off_b1 = ((lane >> 3) * p.ldw + (d_lane_chunk ^ 1u) * 8u) * 2u;
-    gd_half8 *dA = reinterpret_cast<gd_half8 *>(gd_tile_smem); /* [2][BM*8] */
-    gd_half8 *dB = dA + 2u * BM * CH;                          /* [2][BN*8] */
+    gd_elem8 *dA = reinterpret_cast<gd_elem8 *>(gd_tile_smem); /* [2][BM*8] */
+    gd_elem8 *dB = dA + 2u * BM * CH;                          /* [2][BN*8] */
     const uint32_t wave_u = __builtin_amdgcn_readfirstlane(wave);
     const uint32_t lds_base = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) unsigned char *)gd_tile_smem;
     /* item t < A_DIRECT: a wavefront load of the activation tile; A_DIRECT <= t: one of the weight tile */
@@ -315,19 +328,19 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     const uint32_t frag_row = lane & 31u, frag_c = lane >> 5;
     const uint32_t a_frag_row = wm * (WM * 32u) + frag_row, b_frag_row = wn * (WN * 32u) + frag_row;
 
-    auto load_frags = [&](const gd_half8 *cA, const gd_half8 *cB, uint32_t ks, gd_half8 (&fa)[WM], gd_half8 (&fb)[WN])
+    auto load_frags = [&](const gd_elem8 *cA, const gd_elem8 *cB, uint32_t ks, gd_elem8 (&fa)[WM], gd_elem8 (&fb)[WN])
         __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < WM; ++i) fa[i] = cA[gd_tile_slot(a_frag_row + i * 32u, ks * 2u + frag_c)];
 #pragma unroll
         for (int j = 0; j < WN; ++j) fb[j] = cB[gd_tile_slot(b_frag_row + j * 32u, ks * 2u + frag_c)];
     };
-    auto multiply = [&](const gd_half8 (&fa)[WM], const gd_half8 (&fb)[WN]) __attribute__((always_inline)) {
+    auto multiply = [&](const gd_elem8 (&fa)[WM], const gd_elem8 (&fb)[WN]) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < WM; ++i)
 #pragma unroll
             for (int j = 0; j < WN; ++j)
-                acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_f16(fb[j], fa[i], acc[i][j], 0, 0, 0);
+                acc[i][j] = GD_MFMA_32X32X16(fb[j], fa[i], acc[i][j]);
     };
 
     constexpr uint32_t STEPS = GD_TILE_BK / 16u;
@@ -337,8 +350,8 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     auto k_tile_regs = [&](uint32_t kt, auto guarded_tag, auto more_tag) __attribute__((always_inline)) {
         constexpr bool MORE = decltype(more_tag)::value;
         const uint32_t stage = kt & 1u;
-        const gd_half8 *cA = sA + stage * BM * 8u, *cB = sB + stage * BN * 8u;
-        gd_half8 fa[2][WM], fb[2][WN];
+        const gd_elem8 *cA = sA + stage * BM * 8u, *cB = sB + stage * BN * 8u;
+        gd_elem8 fa[2][WM], fb[2][WN];
         load_frags(cA, cB, 0u, fa[0], fb[0]);
         if (MORE) load_tile(kt + 1u, guarded_tag);
 #pragma unroll
@@ -356,12 +369,12 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         __syncthreads();
     };
 
-    auto direct_frag_a = [&](const gd_half8 *cA, uint32_t ks, uint32_t i) __attribute__((always_inline)) {
+    auto direct_frag_a = [&](const gd_elem8 *cA, uint32_t ks, uint32_t i) __attribute__((always_inline)) {
         const uint32_t c = ks * 2u + frag_c;
         const uint32_t r = a_frag_row + i * 32u;
         return cA[r * CH + (c ^ (r & 7u) ^ ((r >> 3) & 1u))];
     };
-    auto direct_frag_b = [&](const gd_half8 *cB, uint32_t ks, uint32_t j) __attribute__((always_inline)) {
+    auto direct_frag_b = [&](const gd_elem8 *cB, uint32_t ks, uint32_t j) __attribute__((always_inline)) {
         if (W_NK) {
             const uint32_t c = ks * 2u + frag_c;
             const uint32_t r = b_frag_row + j * 32u;
@@ -379,7 +392,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                 (__attribute__((address_space(3))) gd_short4 *)(base + byte0));
             const gd_short4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                 (__attribute__((address_space(3))) gd_short4 *)(base + byte0 + 4u * (BN * 2u)));
-            union { gd_short4 s[2]; gd_half8 h; } u;
+            union { gd_short4 s[2]; gd_elem8 h; } u;
             u.s[0] = lo;
             u.s[1] = hi;
             return u.h;
@@ -395,7 +408,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
      *           request the first half of tile kt+2 into the freed stage; step 0 of the next tile requests
      *           the second half.
      * TAIL 0: steady state; 1: tile kt+1 exists but not kt+2; 2: last tile. */
-    gd_half8 qa[2][WM], qb[2][WN];
+    gd_elem8 qa[2][WM], qb[2][WN];
     constexpr uint32_t NM = WM * WN, NR = WM + WN, NL = PER_TILE / 2;
     constexpr uint32_t RPM = NM >= 2u * NR ? 1u : (2u * NR + NM - 1u) / NM; /* fragment reads per matrix instruction */
     constexpr uint32_t LPM = NM >= 2u * NL ? 1u : (2u * NL + NM - 1u) / NM; /* loads per matrix instruction */
@@ -406,7 +419,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         constexpr bool READS = KS < 3u || TAIL < 2;
         constexpr bool LOADS = (KS == 3u && TAIL == 0) || (KS == 0u && TAIL < 2);
         const uint32_t rstage = KS < 3u ? (kt & 1u) : ((kt + 1u) & 1u);
-        const gd_half8 *cA = dA + rstage * BM * CH, *cB = dB + rstage * BN * CH;
+        const gd_elem8 *cA = dA + rstage * BM * CH, *cB = dB + rstage * BN * CH;
         const uint32_t rks = KS < 3u ? KS + 1u : 0u;
         const bool loads_on = KS == 3u || kt >= 1u; /* tiles 0 and 1 are requested before the loop */
         if (KS == 3u && TAIL < 2) {
@@ -417,7 +430,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
 #pragma unroll
         for (uint32_t idx = 0; idx < NM; ++idx) {
             const uint32_t i = idx / WN, j = idx % WN;
-            acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_f16(qb[CUR][j], qa[CUR][i], acc[i][j], 0, 0, 0);
+            acc[i][j] = GD_MFMA_32X32X16(qb[CUR][j], qa[CUR][i], acc[i][j]);
             if (READS) {
 #pragma unroll
                 for (uint32_t r = min(idx * RPM, NR); r < min((idx + 1u) * RPM, NR); ++r) {
@@ -452,8 +465,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     /* 8-byte pieces of the epilogue buffer: piece u of row e sits at e*EU + (u ^ (e & 31)), which spreads the
      * 32 rows that one wavefront store touches over all banks; a 16-byte read-back takes pieces 2v, 2v+1 */
     constexpr uint32_t EU = BN / 4u;
-    typedef _Float16 gd_half4 __attribute__((ext_vector_type(4)));
-    gd_half4 bq[WN][4]; /* bias of the 4 columns of every register quad, loaded once per tile */
+    gd_elem4 bq[WN][4]; /* bias of the 4 columns of every register quad, loaded once per tile */
     auto load_bias = [&]() __attribute__((always_inline)) {
         const bool vec = (reinterpret_cast<uintptr_t>(bias) & 7u) == 0u;
 #pragma unroll
@@ -463,11 +475,11 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                 const uint32_t lc = wn * (WN * 32u) + (uint32_t)j * 32u + 8u * (uint32_t)q + 4u * frag_c;
                 const uint32_t gc = wrow(n0, lc); /* the four columns of a quad lie in the same half of a gated tile */
                 if (vec && (gc & 3u) == 0u && wrow_ok(n0, lc + 3u)) {
-                    bq[j][q] = *reinterpret_cast<const gd_half4 *>(bias + gc);
+                    bq[j][q] = *reinterpret_cast<const gd_elem4 *>(bias + gc);
                 } else {
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
-                        bq[j][q][r] = wrow_ok(n0, lc + (uint32_t)r) ? bias[gc + (uint32_t)r] : (gd_half)0.f;
+                        bq[j][q][r] = wrow_ok(n0, lc + (uint32_t)r) ? bias[gc + (uint32_t)r] : (gd_elem)0.f;
                 }
             }
         }
@@ -475,13 +487,13 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     /* the four columns of register quad q of accumulator tile a, rounded to F16 with the bias of the mode */
     auto quad_f16 = [&](auto mode_tag, const gd_float16 &a, int j, int q) __attribute__((always_inline)) {
         constexpr uint32_t MODE = decltype(mode_tag)::value;
-        gd_half4 h;
+        gd_elem4 h;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const float v = a[4 * q + r];
-            if (MODE == GD_HIP_EPI_NONE) h[r] = (gd_half)v;
-            else if (MODE == GD_HIP_EPI_BIAS_F32) h[r] = (gd_half)(v + (float)bq[j][q][r]);
-            else h[r] = (gd_half)v + bq[j][q][r];
+            if (MODE == GD_HIP_EPI_NONE) h[r] = (gd_elem)v;
+            else if (MODE == GD_HIP_EPI_BIAS_F32) h[r] = (gd_elem)(v + (float)bq[j][q][r]);
+            else h[r] = (gd_elem)v + bq[j][q][r];
         }
         return h;
     };
@@ -493,15 +505,15 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
                 const uint32_t lc = wn * (WN * 32u) + (uint32_t)j * 32u + 8u * (uint32_t)q + 4u * frag_c;
-                *reinterpret_cast<gd_half4 *>(epi + (e * EU + ((lc >> 2) ^ (e & 31u))) * 8u) = quad_f16(mode_tag, acc[I][j], j, q);
+                *reinterpret_cast<gd_elem4 *>(epi + (e * EU + ((lc >> 2) ^ (e & 31u))) * 8u) = quad_f16(mode_tag, acc[I][j], j, q);
             }
         }
         __syncthreads();
         constexpr uint32_t CPRW = BN / 8u; /* 16-byte chunks per row */
         auto read_chunk = [&](uint32_t er, uint32_t v) __attribute__((always_inline)) {
             const uint32_t xr = er & 31u;
-            const gd_half8 raw = *reinterpret_cast<const gd_half8 *>(epi + (er * EU + 2u * (v ^ (xr >> 1))) * 8u);
-            gd_half8 h = raw;
+            const gd_elem8 raw = *reinterpret_cast<const gd_elem8 *>(epi + (er * EU + 2u * (v ^ (xr >> 1))) * 8u);
+            gd_elem8 h = raw;
             if (xr & 1u) {
 #pragma unroll
                 for (int t = 0; t < 4; ++t) {
@@ -521,13 +533,13 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                 if (gr >= p.M || gc >= p.N) continue;
                 /* staged columns: wavefront column wc holds its HW value columns, then their gates */
                 const uint32_t cv = (v / (HW / 8u)) * (HW / 4u) + v % (HW / 8u);
-                const gd_half8 hv = read_chunk(er, cv), hg = read_chunk(er, cv + HW / 8u);
-                gd_half8 h;
+                const gd_elem8 hv = read_chunk(er, cv), hg = read_chunk(er, cv + HW / 8u);
+                gd_elem8 h;
 #pragma unroll
-                for (int t = 0; t < 8; ++t) h[t] = (gd_half)((float)hv[t] * gd_tile_silu((float)hg[t]));
-                gd_half *yr = y + (size_t)gr * p.ldy + gc;
+                for (int t = 0; t < 8; ++t) h[t] = (gd_elem)gd_tile_gated((float)hv[t], (float)hg[t], p.flags);
+                gd_elem *yr = y + (size_t)gr * p.ldy + gc;
                 if (vector_store && gc + 8u <= p.N) {
-                    *reinterpret_cast<gd_half8 *>(yr) = h;
+                    *reinterpret_cast<gd_elem8 *>(yr) = h;
                 } else {
                     for (uint32_t t = 0; t < 8u && gc + t < p.N; ++t) yr[t] = h[t];
                 }
@@ -539,20 +551,20 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
             const uint32_t er = idx / CPRW, v = idx % CPRW;
             const uint32_t gr = m0 + (er >> 5) * (WM * 32u) + (uint32_t)I * 32u + (er & 31u), gc = n0 + v * 8u;
             if (gr >= p.M || gc >= p.N) continue;
-            gd_half8 h = read_chunk(er, v);
-            gd_half *yr = y + (size_t)gr * p.ldy + gc;
+            gd_elem8 h = read_chunk(er, v);
+            gd_elem *yr = y + (size_t)gr * p.ldy + gc;
             if (vector_store && gc + 8u <= p.N) {
                 if (p.has_residual) {
-                    const gd_half8 r = *reinterpret_cast<const gd_half8 *>(residual + (size_t)gr * p.ldr + gc);
+                    const gd_elem8 r = *reinterpret_cast<const gd_elem8 *>(residual + (size_t)gr * p.ldr + gc);
 #pragma unroll
                     for (int t = 0; t < 8; ++t) h[t] = r[t] + h[t];
                 }
                 /* long K: the output is not read again soon and would only push operand panels out of L2 */
-                if (p.K >= 1024u) __builtin_nontemporal_store(h, reinterpret_cast<gd_half8 *>(yr));
-                else *reinterpret_cast<gd_half8 *>(yr) = h;
+                if (p.K >= 1024u) __builtin_nontemporal_store(h, reinterpret_cast<gd_elem8 *>(yr));
+                else *reinterpret_cast<gd_elem8 *>(yr) = h;
             } else {
                 for (uint32_t t = 0; t < 8u && gc + t < p.N; ++t) {
-                    gd_half v1 = h[t];
+                    gd_elem v1 = h[t];
                     if (p.has_residual) v1 = residual[(size_t)gr * p.ldr + gc + t] + v1;
                     yr[t] = v1;
                 }
@@ -580,14 +592,14 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
      * one chunk, and the lanes of one read, hit all banks.  The residual rows of a pass are requested before its
      * accumulators are rounded, so that their latency passes behind that work. */
     typedef unsigned gd_uint2v __attribute__((ext_vector_type(2)));
-    auto pair_chunk = [&](gd_half4 a, gd_half4 b) __attribute__((always_inline)) {
-        union { gd_half4 h; uint32_t u[2]; } ua, ub;
+    auto pair_chunk = [&](gd_elem4 a, gd_elem4 b) __attribute__((always_inline)) {
+        union { gd_elem4 h; uint32_t u[2]; } ua, ub;
         ua.h = a;
         ub.h = b;
         /* lanes 32-63 of the first operand change places with lanes 0-31 of the second */
         const gd_uint2v s0 = __builtin_amdgcn_permlane32_swap(ua.u[0], ub.u[0], false, false);
         const gd_uint2v s1 = __builtin_amdgcn_permlane32_swap(ua.u[1], ub.u[1], false, false);
-        union { uint32_t u[4]; gd_half8 h; } c;
+        union { uint32_t u[4]; gd_elem8 h; } c;
         c.u[0] = s0[0];
         c.u[1] = s1[0];
         c.u[2] = s0[1];
@@ -600,32 +612,32 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         const uint32_t rr = lane >> 4, v = lane & 15u;
         /* offsets of this lane's piece from the tile's first element; the pass and the row group add a uniform
          * term */
-        const gd_half *rtile = residual + ((size_t)m0 * p.ldr + n0);
-        gd_half *ytile = y + ((size_t)m0 * p.ldy + n0);
+        const gd_elem *rtile = residual + ((size_t)m0 * p.ldr + n0);
+        gd_elem *ytile = y + ((size_t)m0 * p.ldy + n0);
         const uint32_t y_lane = (wm * (WM * 32u) + rr) * p.ldy + wn * (WN * 32u) + v * 8u;
         const uint32_t r_lane = (wm * (WM * 32u) + rr) * p.ldr + wn * (WN * 32u) + v * 8u;
         auto pass = [&](auto pass_tag) __attribute__((always_inline)) {
             constexpr int I = decltype(pass_tag)::value;
-            gd_half8 res[8];
+            gd_elem8 res[8];
             if (p.has_residual) {
 #pragma unroll
                 for (uint32_t it = 0; it < 8u; ++it)
-                    res[it] = *reinterpret_cast<const gd_half8 *>(rtile + ((uint32_t)I * 32u + it * 4u) * p.ldr + r_lane);
+                    res[it] = *reinterpret_cast<const gd_elem8 *>(rtile + ((uint32_t)I * 32u + it * 4u) * p.ldr + r_lane);
             }
 #pragma unroll
             for (int j = 0; j < WN; ++j) {
 #pragma unroll
                 for (int pr = 0; pr < 2; ++pr) {
                     const uint32_t c = (uint32_t)j * 4u + 2u * (uint32_t)pr + frag_c;
-                    *reinterpret_cast<gd_half8 *>(own + (frag_row * 16u + (c ^ (frag_row & 15u))) * 16u) =
+                    *reinterpret_cast<gd_elem8 *>(own + (frag_row * 16u + (c ^ (frag_row & 15u))) * 16u) =
                         pair_chunk(quad_f16(mode_tag, acc[I][j], j, 2 * pr), quad_f16(mode_tag, acc[I][j], j, 2 * pr + 1));
                 }
             }
-            gd_half8 h[8];
+            gd_elem8 h[8];
 #pragma unroll
             for (uint32_t it = 0; it < 8u; ++it) {
                 const uint32_t e = it * 4u + rr;
-                h[it] = *reinterpret_cast<const gd_half8 *>(own + (e * 16u + (v ^ (e & 15u))) * 16u);
+                h[it] = *reinterpret_cast<const gd_elem8 *>(own + (e * 16u + (v ^ (e & 15u))) * 16u);
             }
 #pragma unroll
             for (uint32_t it = 0; it < 8u; ++it) {
@@ -633,7 +645,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
 #pragma unroll
                     for (int t = 0; t < 8; ++t) h[it][t] = res[it][t] + h[it][t];
                 }
-                *reinterpret_cast<gd_half8 *>(ytile + ((uint32_t)I * 32u + it * 4u) * p.ldy + y_lane) = h[it];
+                *reinterpret_cast<gd_elem8 *>(ytile + ((uint32_t)I * 32u + it * 4u) * p.ldy + y_lane) = h[it];
             }
         };
         pass(std::integral_constant<int, 0>{});
@@ -645,7 +657,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         if (decltype(mode_tag)::value != GD_HIP_EPI_NONE) load_bias();
         unsigned char *own = epi + wave * 8192u;
         const uint32_t rr = lane >> 3, v = lane & 7u;
-        gd_half *ytile = y + ((size_t)m0 * p.ldy + n0);
+        gd_elem *ytile = y + ((size_t)m0 * p.ldy + n0);
         const uint32_t y_lane = (wm * (WM * 32u) + rr) * p.ldy + wn * HW + v * 8u;
         auto pass = [&](auto pass_tag) __attribute__((always_inline)) {
             constexpr int I = decltype(pass_tag)::value;
@@ -653,28 +665,41 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
             for (int j = 0; j < WN / 2; ++j) {
 #pragma unroll
                 for (int pr = 0; pr < 2; ++pr) {
-                    gd_half4 o[2];
+                    gd_elem4 o[2];
 #pragma unroll
                     for (int s2 = 0; s2 < 2; ++s2) {
-                        const gd_half4 hv = quad_f16(mode_tag, acc[I][j], j, 2 * pr + s2);
-                        const gd_half4 hg = quad_f16(mode_tag, acc[I][j + WN / 2], j + WN / 2, 2 * pr + s2);
+#if GD_LINEAR_IS_BF16
 #pragma unroll
-                        for (int t = 0; t < 4; ++t) o[s2][t] = (gd_half)((float)hv[t] * gd_tile_silu((float)hg[t]));
+                        for (int t = 0; t < 4; ++t) {
+                            const int q = 2 * pr + s2;
+                            float fv = acc[I][j][4 * q + t], fg = acc[I][j + WN / 2][4 * q + t];
+                            if (decltype(mode_tag)::value == GD_HIP_EPI_BIAS_F32) {
+                                fv += (float)bq[j][q][t];
+                                fg += (float)bq[j + WN / 2][q][t];
+                            }
+                            o[s2][t] = (gd_elem)gd_tile_gated(fv, fg, p.flags);
+                        }
+#else
+                        const gd_elem4 hv = quad_f16(mode_tag, acc[I][j], j, 2 * pr + s2);
+                        const gd_elem4 hg = quad_f16(mode_tag, acc[I][j + WN / 2], j + WN / 2, 2 * pr + s2);
+#pragma unroll
+                        for (int t = 0; t < 4; ++t) o[s2][t] = (gd_elem)((float)hv[t] * gd_tile_silu((float)hg[t]));
+#endif
                     }
                     const uint32_t c = (uint32_t)j * 4u + 2u * (uint32_t)pr + frag_c;
-                    *reinterpret_cast<gd_half8 *>(own + (frag_row * 8u + (c ^ ((frag_row >> 1) & 7u))) * 16u) =
+                    *reinterpret_cast<gd_elem8 *>(own + (frag_row * 8u + (c ^ ((frag_row >> 1) & 7u))) * 16u) =
                         pair_chunk(o[0], o[1]);
                 }
             }
-            gd_half8 h[4];
+            gd_elem8 h[4];
 #pragma unroll
             for (uint32_t it = 0; it < 4u; ++it) {
                 const uint32_t e = it * 8u + rr;
-                h[it] = *reinterpret_cast<const gd_half8 *>(own + (e * 8u + (v ^ ((e >> 1) & 7u))) * 16u);
+                h[it] = *reinterpret_cast<const gd_elem8 *>(own + (e * 8u + (v ^ ((e >> 1) & 7u))) * 16u);
             }
 #pragma unroll
             for (uint32_t it = 0; it < 4u; ++it)
-                *reinterpret_cast<gd_half8 *>(ytile + ((uint32_t)I * 32u + it * 8u) * p.ldy + y_lane) = h[it];
+                *reinterpret_cast<gd_elem8 *>(ytile + ((uint32_t)I * 32u + it * 8u) * p.ldy + y_lane) = h[it];
         };
         pass(std::integral_constant<int, 0>{});
         pass(std::integral_constant<int, 1>{});
@@ -694,7 +719,7 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         const uint32_t rr = lane >> 4, v = lane & 15u;
         const uint32_t col0 = n0 + wn * (WN * 32u);
         const uint32_t region = col0 >= 2u * rp.hd ? 2u : (col0 >= rp.hd ? 1u : 0u); /* q, k, v */
-        gd_half *dst = rp.q;
+        gd_elem *dst = rp.q;
         if (region == 1u) dst = rp.k_cache;
         if (region == 2u) dst = rp.v_cache;
         dst += col0 - region * rp.hd + v * 8u;
@@ -725,9 +750,9 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
             constexpr int T = decltype(t_tag)::value; /* accumulator tiles per half head */
             constexpr bool MORE = I + 1 < WM;
             if (MORE) request_rows(I + 1, drow_next);
-            auto stage = [&](int j, int pr, gd_half4 a, gd_half4 b) __attribute__((always_inline)) {
+            auto stage = [&](int j, int pr, gd_elem4 a, gd_elem4 b) __attribute__((always_inline)) {
                 const uint32_t c = (uint32_t)j * 4u + 2u * (uint32_t)pr + frag_c;
-                *reinterpret_cast<gd_half8 *>(own + (frag_row * 16u + (c ^ (frag_row & 15u))) * 16u) = pair_chunk(a, b);
+                *reinterpret_cast<gd_elem8 *>(own + (frag_row * 16u + (c ^ (frag_row & 15u))) * 16u) = pair_chunk(a, b);
             };
             if (region < 2u) {
                 const int32_t tnext = table_at(I + 1);
@@ -735,18 +760,18 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                 for (int t = 0; t < T; ++t) {
 #pragma unroll
                     for (int pr = 0; pr < 2; ++pr) {
-                        gd_half4 olo[WN / (2 * T)][2], ohi[WN / (2 * T)][2];
+                        gd_elem4 olo[WN / (2 * T)][2], ohi[WN / (2 * T)][2];
 #pragma unroll
                         for (int s2 = 0; s2 < 2; ++s2) {
                             const int q = 2 * pr + s2;
 #pragma unroll
                             for (int g = 0; g < WN / (2 * T); ++g) {
                                 const int jlo = g * 2 * T + t, jhi = jlo + T;
-                                const gd_half4 lo = quad_f16(mode_tag, acc[I][jlo], jlo, q);
-                                const gd_half4 hi = quad_f16(mode_tag, acc[I][jhi], jhi, q);
+                                const gd_elem4 lo = quad_f16(mode_tag, acc[I][jlo], jlo, q);
+                                const gd_elem4 hi = quad_f16(mode_tag, acc[I][jhi], jhi, q);
 #pragma unroll
                                 for (int r = 0; r < 4; ++r) {
-                                    gd_half a, b;
+                                    gd_elem a, b;
                                     gd_rope_rotate((float)lo[r], (float)hi[r], cs[t * 4 + q][r], sn[t * 4 + q][r], &a, &b);
                                     olo[g][s2][r] = a;
                                     ohi[g][s2][r] = b;
@@ -771,15 +796,15 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                     for (int pr = 0; pr < 2; ++pr)
                         stage(j, pr, quad_f16(mode_tag, acc[I][j], j, 2 * pr), quad_f16(mode_tag, acc[I][j], j, 2 * pr + 1));
             }
-            gd_half8 h[8];
+            gd_elem8 h[8];
 #pragma unroll
             for (uint32_t it = 0; it < 8u; ++it) {
                 const uint32_t e = it * 4u + rr;
-                h[it] = *reinterpret_cast<const gd_half8 *>(own + (e * 16u + (v ^ (e & 15u))) * 16u);
+                h[it] = *reinterpret_cast<const gd_elem8 *>(own + (e * 16u + (v ^ (e & 15u))) * 16u);
             }
 #pragma unroll
             for (uint32_t it = 0; it < 8u; ++it) {
-                if (drow[it] >= 0) *reinterpret_cast<gd_half8 *>(dst + (size_t)(uint32_t)drow[it] * rp.hd) = h[it];
+                if (drow[it] >= 0) *reinterpret_cast<gd_elem8 *>(dst + (size_t)(uint32_t)drow[it] * rp.hd) = h[it];
             }
         };
         auto passes = [&](auto t_tag) __attribute__((always_inline)) {
@@ -811,10 +836,10 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
             __syncthreads(); /* the previous tile's epilogue has left the buffer that holds the row factors */
             for (uint32_t r = wave; r < BM; r += 4u) {
                 const uint32_t row = min(m0 + r, p.M - 1u);
-                const gd_half *xr = x + (size_t)row * p.ldx;
+                const gd_elem *xr = x + (size_t)row * p.ldx;
                 float ss = 0.f;
                 for (uint32_t k = lane * 8u; k < p.K; k += 512u) {
-                    const gd_half8 v = *reinterpret_cast<const gd_half8 *>(xr + k);
+                    const gd_elem8 v = *reinterpret_cast<const gd_elem8 *>(xr + k);
 #pragma unroll
                     for (int e = 0; e < 8; ++e) ss = fmaf((float)v[e], (float)v[e], ss);
                 }
@@ -900,8 +925,8 @@ gd_linear_tile_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
 }
 
 template <int WM, int WN, bool W_NK, int PRO>
-static int launch_tile_one(hipStream_t stream, const gd_half *x, const gd_half *w, const gd_half *bias,
-                           const gd_half *residual, const gd_half *norm_w, gd_half *y, const gd_hip_linear_params &p,
+static int launch_tile_one(hipStream_t stream, const gd_elem *x, const gd_elem *w, const gd_elem *bias,
+                           const gd_elem *residual, const gd_elem *norm_w, gd_elem *y, const gd_hip_linear_params &p,
                            uint32_t vector_store, uint32_t workgroups)
 {
     constexpr uint32_t BM = 64u * WM, BN = 64u * WN;
@@ -924,11 +949,14 @@ static int launch_tile_one(hipStream_t stream, const gd_half *x, const gd_half *
 }
 
 template <int WM, int WN>
-static int launch_tile(hipStream_t stream, const gd_half *x, const gd_half *w, const gd_half *bias,
-                       const gd_half *residual, const gd_half *norm_w, gd_half *y, const gd_hip_linear_params &p,
+static int launch_tile(hipStream_t stream, const gd_elem *x, const gd_elem *w, const gd_elem *bias,
+                       const gd_elem *residual, const gd_elem *norm_w, gd_elem *y, const gd_hip_linear_params &p,
                        uint32_t vector_store, uint32_t workgroups)
 {
 #define GD_GO(NK, PRO) return launch_tile_one<WM, WN, NK, PRO>(stream, x, w, bias, residual, norm_w, y, p, vector_store, workgroups)
+#if GD_LINEAR_IS_BF16
+    GD_GO(true, GD_HIP_PRO_NONE);
+#else
     if (p.w_is_nk) {
         if (p.prologue == GD_HIP_PRO_SWIGLU) GD_GO(true, GD_HIP_PRO_SWIGLU);
         if (p.prologue == GD_HIP_PRO_RMS_NORM) GD_GO(true, GD_HIP_PRO_RMS_NORM);
@@ -937,21 +965,22 @@ static int launch_tile(hipStream_t stream, const gd_half *x, const gd_half *w, c
     if (p.prologue == GD_HIP_PRO_SWIGLU) GD_GO(false, GD_HIP_PRO_SWIGLU);
     if (p.prologue == GD_HIP_PRO_RMS_NORM) GD_GO(false, GD_HIP_PRO_RMS_NORM);
     GD_GO(false, GD_HIP_PRO_NONE);
+#endif
 #undef GD_GO
 }
 
 /* Requires: K % 8 == 0, 16-byte aligned x rows (and gate half), w rows (for [K,N]: N % 8 == 0 too) and
  * norm weight; M >= 1.  big_tiles: use the 256 x 256 tile (one workgroup per compute unit; the 128 x 128 tile
  * fits two). */
-extern "C" int gd_hip_launch_linear_tile(hipStream_t stream, const void *x, const void *w, const void *bias,
+extern "C" int GD_LINEAR_FN(gd_hip_launch_linear_tile)(hipStream_t stream, const void *x, const void *w, const void *bias,
                                          const void *residual, const void *norm_w, void *y,
                                          const gd_hip_linear_params *params, int big_tiles, int vector_store,
                                          int compute_units)
 {
     const gd_hip_linear_params &p = *params;
     const uint32_t units = ((uint32_t)(compute_units > 0 ? compute_units : 256) + 7u) & ~7u;
-    const gd_half *xp = (const gd_half *)x, *rp = (const gd_half *)residual;
-    gd_half *yp = (gd_half *)y;
+    const gd_elem *xp = (const gd_elem *)x, *rp = (const gd_elem *)residual;
+    gd_elem *yp = (gd_elem *)y;
     if (big_tiles) {
         /* The persistent workgroups walk whole rounds of 256 x 256 tiles; a last round that fills only part of the
          * compute units costs a full tile time.  When that costs more than it would with small tiles, the rows of
@@ -987,15 +1016,15 @@ extern "C" int gd_hip_launch_linear_tile(hipStream_t stream, const void *x, cons
                 int e;
                 head.M = head_rows;
                 tail.M = tail_rows;
-                e = launch_tile<4, 4>(stream, xp, (const gd_half *)w, (const gd_half *)bias, rp, (const gd_half *)norm_w,
+                e = launch_tile<4, 4>(stream, xp, (const gd_elem *)w, (const gd_elem *)bias, rp, (const gd_elem *)norm_w,
                                       yp, head, (uint32_t)vector_store, units);
                 if (e != (int)hipSuccess) return e;
                 if (mid_tiles) {
                     const uint32_t first = p.M - mid_rows;
                     tail.M = mid_rows;
                     return launch_tile_one<3, 4, true, GD_HIP_PRO_NONE>(
-                        stream, xp + (size_t)first * p.ldx, (const gd_half *)w, (const gd_half *)bias,
-                        rp != nullptr ? rp + (size_t)first * p.ldr : nullptr, (const gd_half *)norm_w,
+                        stream, xp + (size_t)first * p.ldx, (const gd_elem *)w, (const gd_elem *)bias,
+                        rp != nullptr ? rp + (size_t)first * p.ldr : nullptr, (const gd_elem *)norm_w,
                         yp + (size_t)first * p.ldy, tail, (uint32_t)vector_store, units);
                 }
                 /* small tiles: whole row tiles as well when the output allows it (anchored at the last row) */
@@ -1005,22 +1034,23 @@ extern "C" int gd_hip_launch_linear_tile(hipStream_t stream, const void *x, cons
                     first = p.M - up;
                     tail.M = up;
                 }
-                return launch_tile<2, 2>(stream, xp + (size_t)first * p.ldx, (const gd_half *)w, (const gd_half *)bias,
-                                         rp != nullptr ? rp + (size_t)first * p.ldr : nullptr, (const gd_half *)norm_w,
+                return launch_tile<2, 2>(stream, xp + (size_t)first * p.ldx, (const gd_elem *)w, (const gd_elem *)bias,
+                                         rp != nullptr ? rp + (size_t)first * p.ldr : nullptr, (const gd_elem *)norm_w,
                                          yp + (size_t)first * p.ldy, tail, (uint32_t)vector_store, 2u * units);
             }
         }
-        return launch_tile<4, 4>(stream, xp, (const gd_half *)w, (const gd_half *)bias, rp, (const gd_half *)norm_w, yp, p,
+        return launch_tile<4, 4>(stream, xp, (const gd_elem *)w, (const gd_elem *)bias, rp, (const gd_elem *)norm_w, yp, p,
                                  (uint32_t)vector_store, units);
     }
-    return launch_tile<2, 2>(stream, xp, (const gd_half *)w, (const gd_half *)bias, rp, (const gd_half *)norm_w, yp, p,
+    return launch_tile<2, 2>(stream, xp, (const gd_elem *)w, (const gd_elem *)bias, rp, (const gd_elem *)norm_w, yp, p,
                              (uint32_t)vector_store, 2u * units);
 }
 
+#if !GD_LINEAR_IS_BF16
 /* The qkv projection of a packed prefill with rotation and cache append in the epilogue (gd_tile_rope): x [M,K],
  * w [3*hd, K], whole 256 x 256 tiles only.  Requires: M % 256 == 0, hd % 256 == 0, K % 64 == 0, K >= 128, 16-byte
  * aligned rows of x, w, q and the caches, half_d 32 or 64 (head size 64 or 128). */
-extern "C" int gd_hip_launch_linear_tile_rope(hipStream_t stream, const void *x, const void *w, const void *bias,
+extern "C" int GD_LINEAR_FN(gd_hip_launch_linear_tile_rope)(hipStream_t stream, const void *x, const void *w, const void *bias,
                                               const gd_hip_linear_params *params, const float *cos_rows,
                                               const float *sin_rows, const int32_t *cache_row, void *q, void *k_cache,
                                               void *v_cache, uint32_t hd, uint32_t half_d, int compute_units)
@@ -1042,17 +1072,17 @@ extern "C" int gd_hip_launch_linear_tile_rope(hipStream_t stream, const void *x,
     const uint32_t units = ((uint32_t)(compute_units > 0 ? compute_units : 256) + 7u) & ~7u;
     const uint32_t tiles_m = p.M / 256u, tiles_n = p.N / 256u;
     const uint32_t grid = tiles_m * tiles_n < units ? tiles_m * tiles_n : units;
-    kernel<<<grid, 256, lds, stream>>>((const gd_half *)x, (const gd_half *)w, (const gd_half *)bias, nullptr, nullptr,
+    kernel<<<grid, 256, lds, stream>>>((const gd_elem *)x, (const gd_elem *)w, (const gd_elem *)bias, nullptr, nullptr,
                                        nullptr, p, tiles_m, tiles_n, 1u,
-                                       gd_tile_rope{cos_rows, sin_rows, cache_row, (gd_half *)q, (gd_half *)k_cache,
-                                                    (gd_half *)v_cache, hd, half_d});
+                                       gd_tile_rope{cos_rows, sin_rows, cache_row, (gd_elem *)q, (gd_elem *)k_cache,
+                                                    (gd_elem *)v_cache, hd, half_d});
     return (int)hipGetLastError();
 }
 
 /* Row tiles of 256 that fill whole rounds of `units` workgroups for an [M, N] output in 256-column tiles: the rows
  * the rope form takes; the rest (a partly filled last round, a ragged last row tile) goes through the plain
  * projection and the table-driven rotation kernel. */
-extern "C" uint32_t gd_hip_linear_tile_rope_head_rows(uint32_t M, uint32_t N, int compute_units)
+extern "C" uint32_t GD_LINEAR_FN(gd_hip_linear_tile_rope_head_rows)(uint32_t M, uint32_t N, int compute_units)
 {
     const uint32_t units = ((uint32_t)(compute_units > 0 ? compute_units : 256) + 7u) & ~7u;
     const uint32_t tiles_n = (N + 255u) / 256u, whole_m = M / 256u;
@@ -1064,3 +1094,4 @@ extern "C" uint32_t gd_hip_linear_tile_rope_head_rows(uint32_t M, uint32_t N, in
     if (tiles - (uint64_t)head_m * tiles_n >= (uint64_t)units * 3u / 4u) head_m = whole_m;
     return head_m * 256u;
 }
+#endif

@@ -1,0 +1,3 @@
+/* The many-row projection kernels over BF16 operands: linear_tile.hip compiled with the other element type (linear_elem.h). */
+#define GD_LINEAR_BF16 1
+#include "linear_tile.hip"

@@ -15,8 +15,8 @@ static void launch_wide(hipStream_t stream, const void *x, const void *w, const 
     const uint32_t n_tiles = outs / cols;
     dim3 grid(n_tiles, (p.M + 16u * MT - 1u) / (16u * MT));
     gd_linear_wide_kernel<NT, MT, PMAX, 8, PRO, EPI><<<grid, 512, 0, stream>>>(
-        (const gd_half *)x, (const gd_half *)w, (const gd_half *)bias, (const gd_half *)residual,
-        (const gd_half *)norm_w, (gd_half *)y, p, n_tiles, rope);
+        (const gd_elem *)x, (const gd_elem *)w, (const gd_elem *)bias, (const gd_elem *)residual,
+        (const gd_elem *)norm_w, (gd_elem *)y, p, n_tiles, rope);
 }
 
 /* 8 columns per workgroup (narrow outputs, one row tile): see gd_linear_wide_half_kernel */
@@ -27,7 +27,7 @@ static void launch_wide_half(hipStream_t stream, const void *x, const void *w, c
     const uint32_t n_tiles = p.N / 8u;
     dim3 grid(n_tiles, (p.M + 15u) / 16u);
     gd_linear_wide_half_kernel<QMAX, 8><<<grid, 512, 0, stream>>>(
-        (const gd_half *)x, (const gd_half *)w, (const gd_half *)bias, (const gd_half *)residual, (gd_half *)y, p, n_tiles);
+        (const gd_elem *)x, (const gd_elem *)w, (const gd_elem *)bias, (const gd_elem *)residual, (gd_elem *)y, p, n_tiles);
 }
 
 /* persistent form: K = 2048 behind an rms_norm, at most 8 tiles per workgroup, one workgroup per compute unit */
@@ -56,8 +56,8 @@ static void launch_persistent(hipStream_t stream, const void *x, const void *w, 
     if ((n_tiles + groups - 1u) / groups > 8u) groups = (n_tiles + 7u) / 8u;
     dim3 grid(groups, (p.M + 16u * MT - 1u) / (16u * MT));
     gd_linear_wide_persistent_kernel<NT, MT, 4, RING, EPI, 8><<<grid, 512, 0, stream>>>(
-        (const gd_half *)x, (const gd_half *)w, (const gd_half *)bias, (const gd_half *)residual,
-        (const gd_half *)norm_w, (gd_half *)y, p, n_tiles, tile_w, rope);
+        (const gd_elem *)x, (const gd_elem *)w, (const gd_elem *)bias, (const gd_elem *)residual,
+        (const gd_elem *)norm_w, (gd_elem *)y, p, n_tiles, tile_w, rope);
 }
 
 /* Returns 1 when the launch was taken (hipGetLastError() then tells how it went), 0 when this kernel family does
@@ -68,7 +68,7 @@ static void launch_persistent(hipStream_t stream, const void *x, const void *w, 
  *                     rms_norm prologue, 64 columns per workgroup;
  *   swiglu epilogue:  rms_norm prologue, 32 (tiles == 2) or 64 weight rows per workgroup;
  *   rope epilogue:    rms_norm prologue, 32 weight rows per workgroup (head size a multiple of 32). */
-extern "C" int gd_hip_try_launch_linear_wide(hipStream_t stream, const void *x, const void *w, const void *bias,
+extern "C" int GD_LINEAR_FN(gd_hip_try_launch_linear_wide)(hipStream_t stream, const void *x, const void *w, const void *bias,
                                              const void *residual, const void *norm_w, void *y,
                                              const gd_hip_linear_params *params, const gd_hip_rope_epilogue *rope_epilogue,
                                              uint64_t min_bytes, uint32_t tiles, uint32_t units)
@@ -103,6 +103,10 @@ extern "C" int gd_hip_try_launch_linear_wide(hipStream_t stream, const void *x, 
         if (ppw <= 12u) GD_W(1, 1, 12, GD_HIP_PRO_NONE, GD_WIDE_EPI_PLAIN);
         return 0;
     }
+#if GD_LINEAR_IS_BF16
+    (void)persistent;
+    (void)mt;
+#else
     if (p.prologue != GD_HIP_PRO_RMS_NORM || ppw > 4u) return 0;
     /* K = 2048: the persistent form, where its LDS holds the sums of MT x NT tiles next to the ring */
 #define GD_P(NT, MT, EPI) \
@@ -139,6 +143,7 @@ extern "C" int gd_hip_try_launch_linear_wide(hipStream_t stream, const void *x, 
     }
     if (epi == GD_WIDE_EPI_ROPE && (p.rope_head_dim % 32u) == 0u && p.N == 3u * p.rope_heads * p.rope_head_dim && mt <= 2u)
         GD_W_MT(2, 4, GD_HIP_PRO_RMS_NORM, GD_WIDE_EPI_ROPE);
+#endif
 #undef GD_W_MT
 #undef GD_W
     return 0;

@@ -38,9 +38,9 @@
  * in front of the ring, are waited for with gd_wide_wait_groups (loads return in order: once only the ring's
  * instructions are outstanding, everything older has arrived); gd_wide_arrived then hands the registers to the
  * compiler, which must not touch them before. */
-__device__ __forceinline__ gd_half8 gd_wide_request16(const unsigned char *uniform_base, uint32_t lane_byte_offset)
+__device__ __forceinline__ gd_elem8 gd_wide_request16(const unsigned char *uniform_base, uint32_t lane_byte_offset)
 {
-    gd_half8 v;
+    gd_elem8 v;
     asm volatile("global_load_dwordx4 %0, %1, %2" : "=v"(v) : "v"(lane_byte_offset), "s"(uniform_base) : "memory");
     return v;
 }
@@ -61,9 +61,9 @@ __device__ __forceinline__ void gd_wide_arrived(T &v)
 {
     asm volatile("" : "+v"(v) : : "memory");
 }
-__device__ __forceinline__ gd_half gd_wide_half_of(uint32_t bits)
+__device__ __forceinline__ gd_elem gd_wide_half_of(uint32_t bits)
 {
-    union { unsigned short u; gd_half h; } c;
+    union { unsigned short u; gd_elem h; } c;
     c.u = (unsigned short)bits;
     return c.h;
 }
@@ -90,9 +90,9 @@ __device__ __forceinline__ void gd_wide_wait_groups(int later)
  * pairing for the paired epilogues), 16-byte aligned rows. */
 template <int NT, int MT, int PMAX, int RING, int PRO, int EPI>
 __global__ void __launch_bounds__(512)
-gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__ w, const gd_half *__restrict__ bias,
-                      const gd_half *__restrict__ residual, const gd_half *__restrict__ norm_w,
-                      gd_half *__restrict__ y, gd_hip_linear_params p, uint32_t n_tiles, gd_hip_rope_epilogue rope)
+gd_linear_wide_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__ w, const gd_elem *__restrict__ bias,
+                      const gd_elem *__restrict__ residual, const gd_elem *__restrict__ norm_w,
+                      gd_elem *__restrict__ y, gd_hip_linear_params p, uint32_t n_tiles, gd_hip_rope_epilogue rope)
 {
     constexpr int WAVES = 8;
     constexpr int SMAX = 2 * PMAX;  /* K steps of 32 per wavefront */
@@ -125,7 +125,7 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     const uint32_t m0 = blockIdx.y * (16u * MT);
 
     /* ---- 1. what the epilogue will need, requested first ---- */
-    gd_half pf_b1[EPT], pf_b2[EPT], pf_res[EPT];
+    gd_elem pf_b1[EPT], pf_b2[EPT], pf_res[EPT];
     int32_t pf_pos[EPT], pf_cpos[EPT];
 #pragma unroll
     for (int i = 0; i < EPT; ++i) {
@@ -133,7 +133,7 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         const int jj = idx >> 8, mt = jj / NTO, j = jj % NTO, rl = idx & 63, rr = (idx >> 6) & 3;
         const uint32_t col = min(n0 + 16u * j + (rl & 15), p.N - 1u);
         const uint32_t row = min(m0 + 16u * mt + 4u * (rl >> 4) + rr, p.M - 1u);
-        pf_b1[i] = pf_b2[i] = pf_res[i] = (gd_half)0.f;
+        pf_b1[i] = pf_b2[i] = pf_res[i] = (gd_elem)0.f;
         pf_pos[i] = pf_cpos[i] = 0;
         if (jj < NTO * MT) {
             if (p.epilogue != GD_HIP_EPI_NONE) {
@@ -158,7 +158,7 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
     /* (a wavefront without a K range requests the first step of the row instead of one past its end) */
     const unsigned char *xb = reinterpret_cast<const unsigned char *>(x) + (size_t)(np > 0 ? p_begin : 0u) * 128u;
     const unsigned char *nb = reinterpret_cast<const unsigned char *>(norm_w) + (size_t)(np > 0 ? p_begin : 0u) * 128u;
-    const gd_half8 zero8 = (gd_half8)(gd_half)0.f;
+    const gd_elem8 zero8 = (gd_elem8)(gd_elem)0.f;
     /* ---- 3. the weight stream: group g = pair * NT + j, two instructions of 8 rows x 128 bytes ---- */
     uint32_t goff[NT][2]; /* bytes from the pair's base to the lane's 16 bytes: row 8*half + lane/8, swizzled chunk */
 #pragma unroll
@@ -184,7 +184,7 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
      *          front of the ring and counted by hand, so that it is usable while the ring is still on its way.  Steps
      *          past the wavefront's range re-read its first one (never multiplied with a landed weight group, but the
      *          row sums of the rms_norm must not see them: zeroed after arrival) ---- */
-    gd_half8 ar[MT][SMAX], nr[PRO == GD_HIP_PRO_RMS_NORM ? SMAX : 1];
+    gd_elem8 ar[MT][SMAX], nr[PRO == GD_HIP_PRO_RMS_NORM ? SMAX : 1];
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt) {
         const uint32_t mrow = min(m0 + 16u * mt + (uint32_t)li, p.M - 1u);
@@ -246,7 +246,7 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
             for (int s = 0; s < SMAX; ++s)
 #pragma unroll
                 for (int e = 0; e < 8; ++e)
-                    ar[mt][s][e] = (gd_half)((float)ar[mt][s][e] * (float)nr[s][e] * minv);
+                    ar[mt][s][e] = (gd_elem)((float)ar[mt][s][e] * (float)nr[s][e] * minv);
         }
     }
 
@@ -262,7 +262,7 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         const uint32_t rd0 = half_rows + (li8 * 8u + ((uint32_t)lg ^ li8)) * 16u;
         const uint32_t rd1 = half_rows + (li8 * 8u + ((4u + (uint32_t)lg) ^ li8)) * 16u;
         const unsigned char *ring = &s_mem[0] + (size_t)wave * (RING * 2048);
-        gd_half8 f0 = zero8, f1 = zero8, pf0 = zero8, pf1 = zero8;
+        gd_elem8 f0 = zero8, f1 = zero8, pf0 = zero8, pf1 = zero8;
 #pragma unroll
         for (int g = 0; g <= NGMAX; ++g) {
             if (g < NGMAX && g < ng) {
@@ -272,15 +272,15 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
                 const int last = issued < ng - 1 ? issued : ng - 1;
                 gd_wide_wait_groups(last - g);
                 const unsigned char *slot = ring + (g % RING) * 2048;
-                f0 = *reinterpret_cast<const gd_half8 *>(slot + rd0);
-                f1 = *reinterpret_cast<const gd_half8 *>(slot + rd1);
+                f0 = *reinterpret_cast<const gd_elem8 *>(slot + rd0);
+                f1 = *reinterpret_cast<const gd_elem8 *>(slot + rd1);
             }
             if (g >= 1 && g - 1 < ng) {
                 const int q = g - 1, pair = q / NT, j = q % NT;
 #pragma unroll
                 for (int mt = 0; mt < MT; ++mt) {
-                    acc[mt][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(ar[mt][2 * pair], pf0, acc[mt][j], 0, 0, 0);
-                    acc[mt][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(ar[mt][2 * pair + 1], pf1, acc[mt][j], 0, 0, 0);
+                    acc[mt][j] = GD_MFMA_16X16X32(ar[mt][2 * pair], pf0, acc[mt][j]);
+                    acc[mt][j] = GD_MFMA_16X16X32(ar[mt][2 * pair + 1], pf1, acc[mt][j]);
                 }
                 __builtin_amdgcn_sched_barrier(0);
                 if (q + RING < NGMAX && q + RING < ng) issue_group(q + RING);
@@ -315,41 +315,48 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
         const float v1 = total(mt, j, rl, rr);
         const float v2 = PAIRED ? total(mt, j + NT / 2, rl, rr) : 0.f;
         if (row >= p.M || col >= p.N) continue;
-        gd_half h1, h2 = (gd_half)0.f;
+#if GD_LINEAR_IS_BF16
+        if (p.flags & GD_HIP_LINEAR_Y_F32) {
+            reinterpret_cast<float *>(y)[(size_t)row * p.ldy + col] =
+                p.epilogue == GD_HIP_EPI_BIAS_F32 ? v1 + (float)pf_b1[i] : v1;
+            continue;
+        }
+#endif
+        gd_elem h1, h2 = (gd_elem)0.f;
         if (p.epilogue == GD_HIP_EPI_BIAS_F32) {
-            h1 = (gd_half)(v1 + (float)pf_b1[i]);
-            if (PAIRED) h2 = (gd_half)(v2 + (float)pf_b2[i]);
+            h1 = (gd_elem)(v1 + (float)pf_b1[i]);
+            if (PAIRED) h2 = (gd_elem)(v2 + (float)pf_b2[i]);
         } else if (p.epilogue == GD_HIP_EPI_BIAS_F16) {
-            h1 = (gd_half)v1 + pf_b1[i];
-            if (PAIRED) h2 = (gd_half)v2 + pf_b2[i];
+            h1 = (gd_elem)v1 + pf_b1[i];
+            if (PAIRED) h2 = (gd_elem)v2 + pf_b2[i];
         } else {
-            h1 = (gd_half)v1;
-            if (PAIRED) h2 = (gd_half)v2;
+            h1 = (gd_elem)v1;
+            if (PAIRED) h2 = (gd_elem)v2;
         }
         if (EPI == GD_WIDE_EPI_PLAIN) {
             if (p.has_residual) h1 = pf_res[i] + h1;
             y[(size_t)row * p.ldy + col] = h1;
         } else if (EPI == GD_WIDE_EPI_SWIGLU) {
-            y[(size_t)row * p.ldy + col] = (gd_half)((float)h1 * gd_lin_silu((float)h2));
+            y[(size_t)row * p.ldy + col] = (gd_elem)((float)h1 * gd_lin_silu((float)h2));
         } else {
             /* col = (section * heads + head) * head_dim + pair: q is rotated into its own tensor, k rotated and v
              * copied into row cache_pos of the sequence's caches (skipped when that row does not exist) */
             const uint32_t D = p.rope_head_dim, area = p.rope_heads * D;
             const uint32_t section = col / area, within = col % area, pair = within % D;
-            gd_half o1 = h1, o2 = h2;
+            gd_elem o1 = h1, o2 = h2;
             if (section < 2u) {
                 float c, sn;
                 gd_rope_cos_sin((float)pf_pos[i], pair, p.rope_freq_scale, &c, &sn);
                 gd_rope_rotate((float)h1, (float)h2, c, sn, &o1, &o2);
             }
             if (section == 0u) {
-                gd_half *dst = (gd_half *)rope.q + (size_t)row * area + within;
+                gd_elem *dst = (gd_elem *)rope.q + (size_t)row * area + within;
                 dst[0] = o1;
                 dst[D / 2u] = o2;
             } else {
                 const int32_t cp = pf_cpos[i];
                 if (cp >= 0 && (uint32_t)cp < p.rope_tmax) {
-                    gd_half *dst = (gd_half *)(section == 1u ? rope.k_cache : rope.v_cache) +
+                    gd_elem *dst = (gd_elem *)(section == 1u ? rope.k_cache : rope.v_cache) +
                                    ((size_t)row * p.rope_tmax + (size_t)cp) * area + within;
                     dst[0] = o1;
                     dst[D / 2u] = o2;
@@ -371,8 +378,8 @@ gd_linear_wide_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__
  */
 template <int QMAX, int RING>
 __global__ void __launch_bounds__(512)
-gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__ w, const gd_half *__restrict__ bias,
-                           const gd_half *__restrict__ residual, gd_half *__restrict__ y, gd_hip_linear_params p,
+gd_linear_wide_half_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__ w, const gd_elem *__restrict__ bias,
+                           const gd_elem *__restrict__ residual, gd_elem *__restrict__ y, gd_hip_linear_params p,
                            uint32_t n_tiles)
 {
     constexpr int WAVES = 8;
@@ -391,7 +398,7 @@ gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restr
 
     /* what the epilogue will need, requested first: thread t < 128 owns output (row 4*(t/32) + (t/8)%4, column t%8) */
     const uint32_t e_col = n0 + (threadIdx.x & 7u), e_row = m0 + 4u * (threadIdx.x >> 5) + ((threadIdx.x >> 3) & 3u);
-    gd_half pf_b = (gd_half)0.f, pf_res = (gd_half)0.f;
+    gd_elem pf_b = (gd_elem)0.f, pf_res = (gd_elem)0.f;
     if (threadIdx.x < 128u) {
         if (p.epilogue != GD_HIP_EPI_NONE) pf_b = bias[e_col];
         if (p.has_residual) pf_res = residual[(size_t)min(e_row, p.M - 1u) * p.ldr + e_col];
@@ -404,7 +411,7 @@ gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restr
     const unsigned char *wb = reinterpret_cast<const unsigned char *>(w) + (size_t)q_begin * 256u;
     /* (a wavefront without a K range requests the first piece of the row instead of one past its end) */
     const unsigned char *xb = reinterpret_cast<const unsigned char *>(x) + (size_t)(nq > 0 ? q_begin : 0u) * 256u;
-    const gd_half8 zero8 = (gd_half8)(gd_half)0.f;
+    const gd_elem8 zero8 = (gd_elem8)(gd_elem)0.f;
 
     /* lane's 16 bytes of an instruction: weight row n0 + lane/8, chunk (lane%8 ^ lane/8) of the 128-byte piece */
     const uint32_t goff = ((n0 + (uint32_t)lane / 8u) * p.ldw + ((((uint32_t)lane % 8u) ^ ((uint32_t)lane / 8u)) * 8u)) * 2u;
@@ -421,7 +428,7 @@ gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restr
     };
     /* the activation slice of the wavefront, resident: requested in front of the ring and counted by hand (see
      * gd_wide_request16), so that the first weight group can be multiplied as soon as it lands */
-    gd_half8 ar[SMAX];
+    gd_elem8 ar[SMAX];
     {
         const uint32_t mrow = min(m0 + (uint32_t)li, p.M - 1u);
         const uint32_t xoff = (mrow * p.ldx + (uint32_t)lg * 8u) * 2u;
@@ -448,7 +455,7 @@ gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restr
         const uint32_t rd0 = (li8 * 8u + ((uint32_t)lg ^ li8)) * 16u;
         const uint32_t rd1 = (li8 * 8u + ((4u + (uint32_t)lg) ^ li8)) * 16u;
         const unsigned char *ring = &s_mem[0] + (size_t)wave * (RING * 2048);
-        gd_half8 f[4] = {zero8, zero8, zero8, zero8}, pf[4] = {zero8, zero8, zero8, zero8};
+        gd_elem8 f[4] = {zero8, zero8, zero8, zero8}, pf[4] = {zero8, zero8, zero8, zero8};
 #pragma unroll
         for (int g = 0; g <= QMAX; ++g) {
             if (g < QMAX && g < nq) {
@@ -456,16 +463,16 @@ gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restr
                 const int last = issued < nq - 1 ? issued : nq - 1;
                 gd_wide_wait_groups(last - g);
                 const unsigned char *slot = ring + (g % RING) * 2048;
-                f[0] = *reinterpret_cast<const gd_half8 *>(slot + rd0);
-                f[1] = *reinterpret_cast<const gd_half8 *>(slot + rd1);
-                f[2] = *reinterpret_cast<const gd_half8 *>(slot + 1024 + rd0);
-                f[3] = *reinterpret_cast<const gd_half8 *>(slot + 1024 + rd1);
+                f[0] = *reinterpret_cast<const gd_elem8 *>(slot + rd0);
+                f[1] = *reinterpret_cast<const gd_elem8 *>(slot + rd1);
+                f[2] = *reinterpret_cast<const gd_elem8 *>(slot + 1024 + rd0);
+                f[3] = *reinterpret_cast<const gd_elem8 *>(slot + 1024 + rd1);
             }
             if (g >= 1 && g - 1 < nq) {
                 const int q = g - 1;
 #pragma unroll
                 for (int t = 0; t < 4; ++t)
-                    acc = __builtin_amdgcn_mfma_f32_16x16x32_f16(ar[4 * q + t], pf[t], acc, 0, 0, 0);
+                    acc = GD_MFMA_16X16X32(ar[4 * q + t], pf[t], acc);
                 __builtin_amdgcn_sched_barrier(0);
                 if (q + RING < QMAX && q + RING < nq) issue_group(q + RING);
             }
@@ -486,10 +493,17 @@ gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restr
 #pragma unroll
         for (int wv = 0; wv < WAVES; ++wv) v += sm[((wv * 4 + g4) * 8 + c) * 4 + r];
         if (e_row < p.M) {
-            gd_half h;
-            if (p.epilogue == GD_HIP_EPI_BIAS_F32) h = (gd_half)(v + (float)pf_b);
-            else if (p.epilogue == GD_HIP_EPI_BIAS_F16) h = (gd_half)v + pf_b;
-            else h = (gd_half)v;
+#if GD_LINEAR_IS_BF16
+            if (p.flags & GD_HIP_LINEAR_Y_F32) {
+                reinterpret_cast<float *>(y)[(size_t)e_row * p.ldy + e_col] =
+                    p.epilogue == GD_HIP_EPI_BIAS_F32 ? v + (float)pf_b : v;
+                return;
+            }
+#endif
+            gd_elem h;
+            if (p.epilogue == GD_HIP_EPI_BIAS_F32) h = (gd_elem)(v + (float)pf_b);
+            else if (p.epilogue == GD_HIP_EPI_BIAS_F16) h = (gd_elem)v + pf_b;
+            else h = (gd_elem)v;
             if (p.has_residual) h = pf_res + h;
             y[(size_t)e_row * p.ldy + e_col] = h;
         }
@@ -507,9 +521,9 @@ gd_linear_wide_half_kernel(const gd_half *__restrict__ x, const gd_half *__restr
  */
 template <int NT, int MT, int PMAX, int RING, int EPI, int TPW>
 __global__ void __launch_bounds__(512)
-gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *__restrict__ w,
-                                 const gd_half *__restrict__ bias, const gd_half *__restrict__ residual,
-                                 const gd_half *__restrict__ norm_w, gd_half *__restrict__ y, gd_hip_linear_params p,
+gd_linear_wide_persistent_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__ w,
+                                 const gd_elem *__restrict__ bias, const gd_elem *__restrict__ residual,
+                                 const gd_elem *__restrict__ norm_w, gd_elem *__restrict__ y, gd_hip_linear_params p,
                                  uint32_t n_tiles, uint32_t tile_w, gd_hip_rope_epilogue rope)
 {
     constexpr int WAVES = 8;
@@ -524,7 +538,7 @@ gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *_
     __shared__ __align__(16) unsigned char s_ring[WAVES * RING * 2048];
     __shared__ __align__(16) float s_sum[WAVES * MT * NT * 256];
     __shared__ float s_part[WAVES][MT][16];
-    __shared__ gd_half s_bias[2][TPW * OUT_COLS];
+    __shared__ gd_elem s_bias[2][TPW * OUT_COLS];
     __shared__ int32_t s_pos[2][16 * MT];
 
     asm volatile("" ::"s"(x), "s"(w), "s"(bias), "s"(residual), "s"(norm_w), "s"(y), "s"(p.M), "s"(p.N), "s"(p.K),
@@ -606,9 +620,9 @@ gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *_
     }
     const unsigned char *xb = reinterpret_cast<const unsigned char *>(x) + (size_t)p_begin * 128u;
     const unsigned char *nb = reinterpret_cast<const unsigned char *>(norm_w) + (size_t)p_begin * 128u;
-    gd_half8 ar[MT][SMAX];
+    gd_elem8 ar[MT][SMAX];
     {
-        gd_half8 nr[SMAX];
+        gd_elem8 nr[SMAX];
 #pragma unroll
         for (int mt = 0; mt < MT; ++mt) {
             const uint32_t mrow = min(m0 + 16u * mt + (uint32_t)li, p.M - 1u);
@@ -669,7 +683,7 @@ gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *_
             for (int s = 0; s < SMAX; ++s)
 #pragma unroll
                 for (int e = 0; e < 8; ++e)
-                    ar[mt][s][e] = (gd_half)((float)ar[mt][s][e] * (float)nr[s][e] * minv);
+                    ar[mt][s][e] = (gd_elem)((float)ar[mt][s][e] * (float)nr[s][e] * minv);
         }
     }
 
@@ -677,7 +691,7 @@ gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *_
     const uint32_t rd0 = half_rows + (li8 * 8u + ((uint32_t)lg ^ li8)) * 16u;
     const uint32_t rd1 = half_rows + (li8 * 8u + ((4u + (uint32_t)lg) ^ li8)) * 16u;
     const unsigned char *ring = &s_ring[0] + (size_t)wave * (RING * 2048);
-    const gd_half8 zero8 = (gd_half8)(gd_half)0.f;
+    const gd_elem8 zero8 = (gd_elem8)(gd_elem)0.f;
     int gbase = 0; /* stream index of the tile's first group */
     int slot = 0;  /* ring slot of the group read next */
     for (int ti = 0; ti < tiles; ++ti) {
@@ -686,7 +700,7 @@ gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *_
         for (int mt = 0; mt < MT; ++mt)
 #pragma unroll
             for (int j = 0; j < NT; ++j) acc[mt][j] = (gd_float4){0.f, 0.f, 0.f, 0.f};
-        gd_half8 f0 = zero8, f1 = zero8, pf0 = zero8, pf1 = zero8;
+        gd_elem8 f0 = zero8, f1 = zero8, pf0 = zero8, pf1 = zero8;
         int pslot = 0;
 #pragma unroll
         for (int g = 0; g <= NG; ++g) {
@@ -699,15 +713,15 @@ gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *_
                 const int last = issued < total_groups - 1 ? issued : total_groups - 1;
                 gd_wide_wait_groups(__builtin_amdgcn_readfirstlane(last - gi));
                 const unsigned char *sl = ring + __builtin_amdgcn_readfirstlane(slot) * 2048;
-                f0 = *reinterpret_cast<const gd_half8 *>(sl + rd0);
-                f1 = *reinterpret_cast<const gd_half8 *>(sl + rd1);
+                f0 = *reinterpret_cast<const gd_elem8 *>(sl + rd0);
+                f1 = *reinterpret_cast<const gd_elem8 *>(sl + rd1);
             }
             if (g >= 1) {
                 const int q = g - 1, pair = q / NT, j = q % NT;
 #pragma unroll
                 for (int mt = 0; mt < MT; ++mt) {
-                    acc[mt][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(ar[mt][2 * pair], pf0, acc[mt][j], 0, 0, 0);
-                    acc[mt][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(ar[mt][2 * pair + 1], pf1, acc[mt][j], 0, 0, 0);
+                    acc[mt][j] = GD_MFMA_16X16X32(ar[mt][2 * pair], pf0, acc[mt][j]);
+                    acc[mt][j] = GD_MFMA_16X16X32(ar[mt][2 * pair + 1], pf1, acc[mt][j]);
                 }
                 __builtin_amdgcn_sched_barrier(0);
                 /* the slot just multiplied is free: the group RING further down the stream goes there */
@@ -746,41 +760,41 @@ gd_linear_wide_persistent_kernel(const gd_half *__restrict__ x, const gd_half *_
                 if (PAIRED) v2 += s_sum[(((wv * MT + mt) * NT + j + NT / 2) * 64 + rl) * 4 + rr];
             }
             if (row >= p.M || !col_used) continue;
-            const gd_half b1 = s_bias[0][ti * (int)OUT_COLS + 16 * j + (rl & 15)];
-            const gd_half b2 = s_bias[1][ti * (int)OUT_COLS + 16 * j + (rl & 15)];
-            gd_half h1, h2 = (gd_half)0.f;
+            const gd_elem b1 = s_bias[0][ti * (int)OUT_COLS + 16 * j + (rl & 15)];
+            const gd_elem b2 = s_bias[1][ti * (int)OUT_COLS + 16 * j + (rl & 15)];
+            gd_elem h1, h2 = (gd_elem)0.f;
             if (p.epilogue == GD_HIP_EPI_BIAS_F32) {
-                h1 = (gd_half)(v1 + (float)b1);
-                if (PAIRED) h2 = (gd_half)(v2 + (float)b2);
+                h1 = (gd_elem)(v1 + (float)b1);
+                if (PAIRED) h2 = (gd_elem)(v2 + (float)b2);
             } else if (p.epilogue == GD_HIP_EPI_BIAS_F16) {
-                h1 = (gd_half)v1 + b1;
-                if (PAIRED) h2 = (gd_half)v2 + b2;
+                h1 = (gd_elem)v1 + b1;
+                if (PAIRED) h2 = (gd_elem)v2 + b2;
             } else {
-                h1 = (gd_half)v1;
-                if (PAIRED) h2 = (gd_half)v2;
+                h1 = (gd_elem)v1;
+                if (PAIRED) h2 = (gd_elem)v2;
             }
             if (EPI == GD_WIDE_EPI_PLAIN) {
                 if (p.has_residual) h1 = residual[(size_t)row * p.ldr + col] + h1;
                 y[(size_t)row * p.ldy + col] = h1;
             } else if (EPI == GD_WIDE_EPI_SWIGLU) {
-                y[(size_t)row * p.ldy + col] = (gd_half)((float)h1 * gd_lin_silu((float)h2));
+                y[(size_t)row * p.ldy + col] = (gd_elem)((float)h1 * gd_lin_silu((float)h2));
             } else {
                 const uint32_t D = p.rope_head_dim, area = p.rope_heads * D;
                 const uint32_t section = col / area, within = col % area, pair = within % D;
-                gd_half o1 = h1, o2 = h2;
+                gd_elem o1 = h1, o2 = h2;
                 if (section < 2u) {
                     float c, sn;
                     gd_rope_cos_sin((float)s_pos[0][lrow_i], pair, p.rope_freq_scale, &c, &sn);
                     gd_rope_rotate((float)h1, (float)h2, c, sn, &o1, &o2);
                 }
                 if (section == 0u) {
-                    gd_half *dst = (gd_half *)rope.q + (size_t)row * area + within;
+                    gd_elem *dst = (gd_elem *)rope.q + (size_t)row * area + within;
                     dst[0] = o1;
                     dst[D / 2u] = o2;
                 } else {
                     const int32_t cp = s_pos[1][lrow_i];
                     if (cp >= 0 && (uint32_t)cp < p.rope_tmax) {
-                        gd_half *dst = (gd_half *)(section == 1u ? rope.k_cache : rope.v_cache) +
+                        gd_elem *dst = (gd_elem *)(section == 1u ? rope.k_cache : rope.v_cache) +
                                        ((size_t)row * p.rope_tmax + (size_t)cp) * area + within;
                         dst[0] = o1;
                         dst[D / 2u] = o2;

@@ -13,10 +13,11 @@ __device__ __forceinline__ void gd_rope_cos_sin(float fpos, uint32_t pair, float
     sincosf(__fmul_rn(fpos, exp2f(__fmul_rn((float)pair, freq_scale))), s, c);
 }
 
-__device__ __forceinline__ void gd_rope_rotate(float x0, float x1, float c, float s, gd_half *o0, gd_half *o1)
+template <typename T>
+__device__ __forceinline__ void gd_rope_rotate(float x0, float x1, float c, float s, T *o0, T *o1)
 {
-    *o0 = (gd_half)__fmaf_rn(x0, c, -__fmul_rn(x1, s));
-    *o1 = (gd_half)__fmaf_rn(x0, s, __fmul_rn(x1, c));
+    *o0 = (T)__fmaf_rn(x0, c, -__fmul_rn(x1, s));
+    *o1 = (T)__fmaf_rn(x0, s, __fmul_rn(x1, c));
 }
 
 #endif
