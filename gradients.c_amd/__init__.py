@@ -95,6 +95,19 @@ class SampleTensors(C.Structure):  # gd_backend_sample_tensors
     _fields_ = [(n, C.POINTER(TensorView)) for n in _names]
 
 
+class PackedSeqs(C.Structure):  # gd_backend_packed_seqs
+    _fields_ = [(n, C.POINTER(TensorView)) for n in ("row_seq", "cu", "slot", "start")] + [("max_new", C.c_uint32)]
+
+
+class SsmArgs(C.Structure):  # gd_backend_ssm_args
+    _fields_ = [(n, C.c_uint32) for n in ("heads", "vdim", "state", "groups")]
+
+
+class LatentArgs(C.Structure):  # gd_backend_latent_args
+    _fields_ = [(n, C.c_uint32) for n in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank")] + \
+               [("scale", C.c_float), ("eps", C.c_float)]
+
+
 class ConcatArgs(C.Structure):
     _fields_ = [("count", C.c_uint64), ("inner", C.c_uint64), ("slice_axis", C.c_uint64), ("full_axis", C.c_uint64),
                 ("axis_offset", C.c_uint64)]
@@ -168,6 +181,15 @@ _SIGNATURES = {
     "gd_backend_sample_advance": [_vp, _TV, C.POINTER(SampleTensors), C.POINTER(SampleArgs)],
     "gd_backend_minimax_m3_index_topk": [_vp, _TV, _TV, _TV, _TV, C.POINTER(MinimaxArgs)],
     "gd_backend_minimax_m3_sparse_attention": [_vp, _TV, _TV, _TV, _TV, _TV, _TV, C.POINTER(MinimaxArgs)],
+    "gd_backend_residual_embed": [_vp, _TV, _TV, _TV, _TV, C.c_float],
+    "gd_backend_residual_norm_add": [_vp, _TV, _TV, _TV, _TV, C.c_float, C.c_float],
+    "gd_backend_residual_norm_rows": [_vp, _TV, _TV, _TV, _TV, C.c_float],
+    "gd_backend_causal_conv_silu": [_vp, _MV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs)],
+    "gd_backend_ssm_scan": [_vp, _TV, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(SsmArgs)],
+    "gd_backend_gated_group_norm": [_vp, _TV, _MV, _TV, _TV, C.c_uint32, C.c_float],
+    "gd_backend_latent_prepare": [_vp, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(LatentArgs)],
+    "gd_backend_latent_attend": [_vp, _TV, _TV, _TV, _MV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs),
+                                 C.POINTER(LatentArgs)],
     "gd_backend_copy": [_vp, _vp, C.c_size_t, _vp, C.c_size_t, C.c_size_t],
     "gd_backend_timer_create": [_vp, C.POINTER(_vp)],
     "gd_backend_timer_start": [_vp],
@@ -195,6 +217,8 @@ _OTHER_RESTYPE = {
     "gd_backend_timer_destroy": (None, [_vp]),
     "gd_backend_sample_state_count": (C.c_size_t, [C.c_uint32]),
     "gd_backend_sample_work_count": (C.c_size_t, [C.c_uint32, C.c_uint32]),
+    "gd_backend_latent_pitch": (C.c_uint32, [C.c_uint32, C.c_uint32]),
+    "gd_backend_latent_work_bytes": (C.c_size_t, [_vp, C.POINTER(LatentArgs), C.c_uint32, C.c_uint32, C.c_uint32]),
     "gd_backend_graph_destroy": (None, [_vp]),
 }
 EXPORTED_SYMBOLS = sorted(list(_SIGNATURES) + list(_OTHER_RESTYPE))

@@ -1,0 +1,169 @@
+/*
+ * F32 residual stream with norms on the sublayers' outputs (gfx950).  HBM-bound row kernels, one workgroup per row:
+ *   embed      x = table[id] * scale, and x once more in the type the projections read
+ *   norm_add   x += mult * (u * w / rms(u)) for a sublayer's output u, and the copy
+ *   norm_rows  out = x * w / rms(x) of picked rows (the model's last norm in front of the LM head)
+ * Sums, norms and the residual itself are F32 whatever the element type.  Rows of up to 8 * 256 * 4 elements on
+ * aligned pointers stay in registers between the sum of squares and the update; others are read twice.
+ */
+#include "../../_shared/hip_device.h"
+
+#define GD_RN_THREADS 256
+#define GD_RN_CHUNKS 4 /* 8-element chunks per thread on the register path */
+
+template <typename T>
+struct gd_rn_vec;
+template <>
+struct gd_rn_vec<gd_bf16> {
+    static __device__ __forceinline__ void load(const gd_bf16 *p, float (&v)[8])
+    {
+        const gd_bf16x8 t = *reinterpret_cast<const gd_bf16x8 *>(p);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = (float)t[e];
+    }
+    static __device__ __forceinline__ void store(gd_bf16 *p, const float (&v)[8])
+    {
+        gd_bf16x8 t;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) t[e] = (gd_bf16)v[e];
+        *reinterpret_cast<gd_bf16x8 *>(p) = t;
+    }
+};
+template <>
+struct gd_rn_vec<float> {
+    static __device__ __forceinline__ void load(const float *p, float (&v)[8])
+    {
+        const gd_float4 a = reinterpret_cast<const gd_float4 *>(p)[0], b = reinterpret_cast<const gd_float4 *>(p)[1];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            v[e] = a[e];
+            v[4 + e] = b[e];
+        }
+    }
+    static __device__ __forceinline__ void store(float *p, const float (&v)[8])
+    {
+        gd_float4 a, b;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            a[e] = v[e];
+            b[e] = v[4 + e];
+        }
+        reinterpret_cast<gd_float4 *>(p)[0] = a;
+        reinterpret_cast<gd_float4 *>(p)[1] = b;
+    }
+};
+
+template <typename T>
+__global__ void __launch_bounds__(GD_RN_THREADS)
+gd_residual_embed_kernel(const T *__restrict__ table, const int32_t *__restrict__ ids, float *__restrict__ x,
+                         T *__restrict__ copy, uint32_t vocab, uint32_t cols, float scale)
+{
+    const int32_t id = ids[blockIdx.x];
+    const bool ok = id >= 0 && (uint32_t)id < vocab;
+    const T *row = table + (size_t)(ok ? id : 0) * cols;
+    for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS) {
+        const float v = ok ? (float)row[c] * scale : __builtin_nanf("");
+        x[(size_t)blockIdx.x * cols + c] = v;
+        if (copy != nullptr) copy[(size_t)blockIdx.x * cols + c] = (T)v;
+    }
+}
+
+template <typename T, bool VEC>
+__global__ void __launch_bounds__(GD_RN_THREADS)
+gd_residual_norm_add_kernel(const T *__restrict__ u, const float *__restrict__ w, float *__restrict__ x,
+                            T *__restrict__ copy, uint32_t cols, float eps, float mult)
+{
+    __shared__ float red[GD_RN_THREADS / 64];
+    const size_t base = (size_t)blockIdx.x * cols;
+    float ss = 0.f;
+    if (VEC) {
+        float uv[GD_RN_CHUNKS][8], xv[GD_RN_CHUNKS][8];
+#pragma unroll
+        for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+            const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
+            if (c >= cols) continue;
+            gd_rn_vec<T>::load(u + base + c, uv[i]);
+            gd_rn_vec<float>::load(x + base + c, xv[i]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss = fmaf(uv[i][e], uv[i][e], ss);
+        }
+        ss = gd_block_sum<GD_RN_THREADS / 64>(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)cols + eps);
+#pragma unroll
+        for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+            const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
+            if (c >= cols) continue;
+            float wv[8];
+            gd_rn_vec<float>::load(w + c, wv);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) xv[i][e] += mult * (uv[i][e] * inv * wv[e]);
+            gd_rn_vec<float>::store(x + base + c, xv[i]);
+            if (copy != nullptr) gd_rn_vec<T>::store(copy + base + c, xv[i]);
+        }
+        return;
+    }
+    for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS) {
+        const float v = (float)u[base + c];
+        ss = fmaf(v, v, ss);
+    }
+    ss = gd_block_sum<GD_RN_THREADS / 64>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)cols + eps);
+    for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS) {
+        const float v = x[base + c] + mult * ((float)u[base + c] * inv * w[c]);
+        x[base + c] = v;
+        if (copy != nullptr) copy[base + c] = (T)v;
+    }
+}
+
+template <typename T>
+__global__ void __launch_bounds__(GD_RN_THREADS)
+gd_residual_norm_rows_kernel(const float *__restrict__ x, const int32_t *__restrict__ rows, uint32_t n_rows,
+                             const float *__restrict__ w, T *__restrict__ out, uint32_t cols, float eps)
+{
+    __shared__ float red[GD_RN_THREADS / 64];
+    const int32_t src = rows != nullptr ? rows[blockIdx.x] : (int32_t)blockIdx.x;
+    if (src < 0 || (uint32_t)src >= n_rows) return;
+    const float *xr = x + (size_t)src * cols;
+    float ss = 0.f;
+    for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS) ss = fmaf(xr[c], xr[c], ss);
+    ss = gd_block_sum<GD_RN_THREADS / 64>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)cols + eps);
+    for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS)
+        out[(size_t)blockIdx.x * cols + c] = (T)(xr[c] * inv * w[c]);
+}
+
+extern "C" int gd_hip_launch_residual_embed(hipStream_t stream, const void *table, const int32_t *ids, float *x,
+                                            void *copy, uint32_t n, uint32_t vocab, uint32_t cols, float scale, int is_f32)
+{
+    if (n == 0u) return (int)hipSuccess;
+    if (is_f32)
+        gd_residual_embed_kernel<float><<<n, GD_RN_THREADS, 0, stream>>>((const float *)table, ids, x, (float *)copy, vocab, cols, scale);
+    else
+        gd_residual_embed_kernel<gd_bf16><<<n, GD_RN_THREADS, 0, stream>>>((const gd_bf16 *)table, ids, x, (gd_bf16 *)copy, vocab, cols, scale);
+    return (int)hipGetLastError();
+}
+
+extern "C" int gd_hip_launch_residual_norm_add(hipStream_t stream, const void *u, const float *w, float *x, void *copy,
+                                               uint32_t rows, uint32_t cols, float eps, float mult, int is_f32,
+                                               int aligned16)
+{
+    if (rows == 0u) return (int)hipSuccess;
+    const bool vec = aligned16 && (cols % 8u) == 0u && cols <= 8u * GD_RN_THREADS * GD_RN_CHUNKS;
+#define GD_GO(T, V) gd_residual_norm_add_kernel<T, V><<<rows, GD_RN_THREADS, 0, stream>>>((const T *)u, w, x, (T *)copy, cols, eps, mult)
+    if (is_f32) { if (vec) GD_GO(float, true); else GD_GO(float, false); }
+    else { if (vec) GD_GO(gd_bf16, true); else GD_GO(gd_bf16, false); }
+#undef GD_GO
+    return (int)hipGetLastError();
+}
+
+extern "C" int gd_hip_launch_residual_norm_rows(hipStream_t stream, const float *x, const int32_t *rows, uint32_t n_rows,
+                                                const float *w, void *out, uint32_t n_out, uint32_t cols, float eps,
+                                                int is_f32)
+{
+    if (n_out == 0u) return (int)hipSuccess;
+    if (is_f32)
+        gd_residual_norm_rows_kernel<float><<<n_out, GD_RN_THREADS, 0, stream>>>(x, rows, n_rows, w, (float *)out, cols, eps);
+    else
+        gd_residual_norm_rows_kernel<gd_bf16><<<n_out, GD_RN_THREADS, 0, stream>>>(x, rows, n_rows, w, (gd_bf16 *)out, cols, eps);
+    return (int)hipGetLastError();
+}

@@ -55,6 +55,11 @@ class GptSampling(C.Structure):  # gd_gpt_sampling
                 ("logits_softcap", C.c_float), ("stop_token", C.c_int32), ("rng_state", C.c_uint64)]
 
 
+class ModelOptions(C.Structure):  # gd_model_options
+    _fields_ = [("max_seq", C.c_int32), ("batch", C.c_int32), ("max_step_tokens", C.c_int32), ("compute", C.c_int),
+                ("heads", C.c_int32)]
+
+
 class CheckpointEntry(C.Structure):  # gd_checkpoint_entry
     _fields_ = [("path", C.c_char * 256), ("flags", C.c_uint32), ("dtype", C.c_int), ("rank", C.c_uint32),
                 ("shape", C.c_int64 * 8), ("data_offset", C.c_uint64), ("nbytes", C.c_uint64)]
@@ -147,6 +152,20 @@ def lib():
         l.gd_checkpoint_close.argtypes = [_vp]
         l.gd_checkpoint_close.restype = None
         l.gd_checkpoint_count.argtypes = [_vp]
+        l.gd_gpt_decoder_acquire.argtypes = [_vp, C.POINTER(C.c_int32)]
+        l.gd_gpt_decoder_release.argtypes = [_vp, C.c_int32]
+        l.gd_gpt_decoder_extend.argtypes = [_vp, _vp, C.c_int32, _vp, _vp, _vp, C.c_int32, _vp]
+        l.gd_model_open.argtypes = [C.c_char_p, C.POINTER(_vp), C.c_char_p, C.c_size_t]
+        l.gd_model_open_config.argtypes = [C.c_char_p, C.c_uint64, C.POINTER(_vp), C.c_char_p, C.c_size_t]
+        l.gd_model_close.argtypes = [_vp]
+        l.gd_model_close.restype = None
+        l.gd_model_architecture.argtypes = [_vp]
+        l.gd_model_architecture.restype = C.c_char_p
+        for name in ("gd_model_vocab", "gd_model_layers"):
+            getattr(l, name).argtypes = [_vp]
+            getattr(l, name).restype = C.c_int32
+        l.gd_model_memory.argtypes = [_vp, C.POINTER(ModelOptions), C.POINTER(MemoryConfig)]
+        l.gd_model_create_decoder.argtypes = [_vp, _vp, C.POINTER(ModelOptions), C.POINTER(_vp)]
         l.gd_checkpoint_count.restype = C.c_uint32
         l.gd_checkpoint_entry_at.argtypes = [_vp, C.c_uint32]
         l.gd_checkpoint_entry_at.restype = C.POINTER(CheckpointEntry)
@@ -358,6 +377,78 @@ class GptDecoder:
         self.ctx.check(lib().gd_gpt_decoder_resident_end(self.handle, ids.ctypes.data_as(_vp), gaps.ctypes.data_as(_vp),
                                                          C.byref(done)), "gd_gpt_decoder_resident_end")
         return ids[:done.value], gaps[:done.value]
+
+
+class Model:
+    """A stored model of any architecture the library serves (gd_model.h): a folder with config.json and
+    model.safetensors, a .gdckpt file, or (config_json) a configuration whose weights are drawn from a seed."""
+
+    def __init__(self, path=None, config_json=None, seed=0):
+        h, message = _vp(), C.create_string_buffer(256)
+        if path is not None:
+            st = lib().gd_model_open(os.fsencode(path), C.byref(h), message, 256)
+        else:
+            st = lib().gd_model_open_config(config_json.encode(), seed, C.byref(h), message, 256)
+        if st != GD_OK:
+            raise GdError(st, f"gd_model_open [{message.value.decode()}]")
+        self.handle = h.value
+        self.architecture = lib().gd_model_architecture(self.handle).decode()
+        self.vocab = lib().gd_model_vocab(self.handle)
+        self.n_layers = lib().gd_model_layers(self.handle)
+
+    def close(self):
+        if getattr(self, "handle", None):
+            lib().gd_model_close(self.handle)
+            self.handle = None
+
+    def memory(self, options):
+        mem = MemoryConfig()
+        st = lib().gd_model_memory(self.handle, C.byref(options), C.byref(mem))
+        if st != GD_OK:
+            raise GdError(st, "gd_model_memory")
+        return mem
+
+    def decoder(self, max_seq=0, batch=1, max_step_tokens=0, compute="bfloat16", heads=0):
+        return ModelDecoder(self, ModelOptions(max_seq, batch, max_step_tokens, {"bfloat16": 2, "float32": 3}[compute],
+                                               heads))
+
+
+class ModelDecoder(GptDecoder):
+    """A decoder made from a Model: everything of GptDecoder, and sequences in slots continued by portions."""
+
+    def __init__(self, model, options):
+        mem = model.memory(options)
+        self.cfg = GptConfig(vocab=model.vocab, max_seq=options.max_seq, batch=max(options.batch, 1))
+        self.ctx = Context(mem.params_bytes, mem.state_bytes, mem.scratch_slot_bytes, mem.data_slot_bytes,
+                           mem.scratch_slots, mem.data_slots)
+        h = _vp()
+        st = lib().gd_model_create_decoder(self.ctx.handle, model.handle, C.byref(options), C.byref(h))
+        if st != GD_OK:
+            msg = self.ctx.error()
+            self.ctx.close()
+            raise GdError(st, f"gd_model_create_decoder [{msg}]")
+        self.handle = h.value
+
+    def acquire(self):
+        slot = C.c_int32()
+        self.ctx.check(lib().gd_gpt_decoder_acquire(self.handle, C.byref(slot)), "gd_gpt_decoder_acquire")
+        return slot.value
+
+    def release(self, slot):
+        self.ctx.check(lib().gd_gpt_decoder_release(self.handle, slot), "gd_gpt_decoder_release")
+
+    def extend(self, runs, want=None):
+        """runs: {slot: new tokens}; returns the logits [wanted, vocab] of the packed places in `want` (None: all)."""
+        slots = np.array(list(runs), np.int32)
+        ids = np.concatenate([np.asarray(r, np.int32) for r in runs.values()])
+        cu = np.concatenate([[0], np.cumsum([len(r) for r in runs.values()])]).astype(np.int32)
+        want = np.arange(len(ids), dtype=np.int32) if want is None else np.asarray(want, np.int32)
+        out = np.empty((len(want), self.cfg.vocab), np.float32)
+        st = lib().gd_gpt_decoder_extend(self.handle, slots.ctypes.data_as(_vp), len(slots), ids.ctypes.data_as(_vp),
+                                         cu.ctypes.data_as(_vp), want.ctypes.data_as(_vp), len(want),
+                                         out.ctypes.data_as(_vp))
+        self.ctx.check(st, "gd_gpt_decoder_extend")
+        return out
 
 
 def view_of(t):

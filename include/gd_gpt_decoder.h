@@ -100,6 +100,18 @@ gd_status gd_gpt_decoder_prefill(gd_gpt_decoder *dec, const int32_t *ids, const 
 gd_status gd_gpt_decoder_step(gd_gpt_decoder *dec, const int32_t *ids, int32_t *next_ids, float *gaps,
                               uint16_t *logits);
 
+/* Portions of prompts and single sequences.  The batch rows are slots: acquire hands out a free one at position 0
+ * (GD_ERR_BUSY: none is free), release gives it back.  extend appends n_seqs runs of new tokens, ids [cu[s] ..
+ * cu[s+1]) to the sequence in slots[s], behind what that slot already holds (gd_gpt_decoder_positions), and leaves
+ * the caches and states as a prefill of everything so far would.  want [n_want]: packed places whose logits are
+ * stored in logits F32 [n_want, vocab] (n_want may be 0).  A run of one token goes through the kernels of a decode
+ * step, longer runs through those of a prefill.  GD_ERR_UNSUPPORTED for models that cannot continue a prompt (gpt_lm:
+ * its prefill attends over the new tokens only).  GD_ERR_BUSY while a resident session is open. */
+gd_status gd_gpt_decoder_acquire(gd_gpt_decoder *dec, int32_t *slot);
+gd_status gd_gpt_decoder_release(gd_gpt_decoder *dec, int32_t slot);
+gd_status gd_gpt_decoder_extend(gd_gpt_decoder *dec, const int32_t *slots, int32_t n_seqs, const int32_t *ids,
+                                const int32_t *cu, const int32_t *want, int32_t n_want, float *logits);
+
 /* Device-resident greedy decoding.  A session keeps token ids and cache positions on the device:
  *   begin  uploads first_ids [batch] and the positions, opens one inference step scope, runs the
  *          first step eagerly and captures the step into a graph;

@@ -14,15 +14,19 @@ GD_NULL_OP(gd_backend_add)
 GD_NULL_OP(gd_backend_add_scalar_i32)
 GD_NULL_OP(gd_backend_argmax_advance)
 GD_NULL_OP(gd_backend_argmax_rows)
+GD_NULL_OP(gd_backend_causal_conv_silu)
 GD_NULL_OP(gd_backend_concat_to_full)
 GD_NULL_OP(gd_backend_decode_advance)
 GD_NULL_OP(gd_backend_embedding_forward)
 GD_NULL_OP(gd_backend_fused_linear)
 GD_NULL_OP(gd_backend_fused_qkv_rope_append)
+GD_NULL_OP(gd_backend_gated_group_norm)
 GD_NULL_OP(gd_backend_gather_rows)
 GD_NULL_OP(gd_backend_kv_cache_append_at)
 GD_NULL_OP(gd_backend_kv_cache_append_packed)
 GD_NULL_OP(gd_backend_kv_cache_append_positions)
+GD_NULL_OP(gd_backend_latent_attend)
+GD_NULL_OP(gd_backend_latent_prepare)
 GD_NULL_OP(gd_backend_linear)
 GD_NULL_OP(gd_backend_linear_last_kernel)
 GD_NULL_OP(gd_backend_linear_nt)
@@ -35,6 +39,9 @@ GD_NULL_OP(gd_backend_qkv_rope_append)
 GD_NULL_OP(gd_backend_qkv_rope_append_packed)
 GD_NULL_OP(gd_backend_qkv_split_rope_forward)
 GD_NULL_OP(gd_backend_rand_uniform)
+GD_NULL_OP(gd_backend_residual_embed)
+GD_NULL_OP(gd_backend_residual_norm_add)
+GD_NULL_OP(gd_backend_residual_norm_rows)
 GD_NULL_OP(gd_backend_rms_norm_forward)
 GD_NULL_OP(gd_backend_rope_table_packed)
 GD_NULL_OP(gd_backend_sample_advance)
@@ -45,5 +52,13 @@ GD_NULL_OP(gd_backend_sdpa_decode_positions)
 GD_NULL_OP(gd_backend_sdpa_decode_positions_noalloc)
 GD_NULL_OP(gd_backend_sdpa_varlen)
 GD_NULL_OP(gd_backend_sdpa_varlen_cached)
+GD_NULL_OP(gd_backend_ssm_scan)
 GD_NULL_OP(gd_backend_swiglu_split_forward)
 GD_NULL_OP(gd_backend_swiglu_split_linear)
+
+/* sizes the layer-list decoder asks for: the ones of the header */
+__attribute__((visibility("default"))) uint32_t gd_backend_latent_pitch(uint32_t kv_rank, uint32_t rot_dim)
+{
+    return (kv_rank + rot_dim + 7u) & ~7u;
+}
+__attribute__((visibility("default"))) uint64_t gd_backend_latent_work_bytes() { return 4096u; }
