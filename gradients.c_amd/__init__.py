@@ -96,7 +96,8 @@ class SampleTensors(C.Structure):  # gd_backend_sample_tensors
 
 
 class PackedSeqs(C.Structure):  # gd_backend_packed_seqs
-    _fields_ = [(n, C.POINTER(TensorView)) for n in ("row_seq", "cu", "slot", "start")] + [("max_new", C.c_uint32)]
+    _fields_ = [(n, C.POINTER(TensorView)) for n in ("row_seq", "cu", "slot", "start")] + \
+               [("max_new", C.c_uint32), ("kv_cu", C.POINTER(TensorView)), ("kv_total", C.c_uint32)]
 
 
 class SsmArgs(C.Structure):  # gd_backend_ssm_args
@@ -187,7 +188,7 @@ _SIGNATURES = {
     "gd_backend_causal_conv_silu": [_vp, _MV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs)],
     "gd_backend_ssm_scan": [_vp, _TV, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(SsmArgs)],
     "gd_backend_gated_group_norm": [_vp, _TV, _MV, _TV, _TV, C.c_uint32, C.c_float],
-    "gd_backend_latent_prepare": [_vp, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(LatentArgs)],
+    "gd_backend_latent_prepare": [_vp, _MV, _TV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(LatentArgs)],
     "gd_backend_latent_attend": [_vp, _TV, _TV, _TV, _MV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs),
                                  C.POINTER(LatentArgs)],
     "gd_backend_copy": [_vp, _vp, C.c_size_t, _vp, C.c_size_t, C.c_size_t],
@@ -218,7 +219,7 @@ _OTHER_RESTYPE = {
     "gd_backend_sample_state_count": (C.c_size_t, [C.c_uint32]),
     "gd_backend_sample_work_count": (C.c_size_t, [C.c_uint32, C.c_uint32]),
     "gd_backend_latent_pitch": (C.c_uint32, [C.c_uint32, C.c_uint32]),
-    "gd_backend_latent_work_bytes": (C.c_size_t, [_vp, C.POINTER(LatentArgs), C.c_uint32, C.c_uint32, C.c_uint32]),
+    "gd_backend_latent_work_bytes": (C.c_size_t, [_vp, C.POINTER(LatentArgs)] + [C.c_uint32] * 5),
     "gd_backend_graph_destroy": (None, [_vp]),
 }
 EXPORTED_SYMBOLS = sorted(list(_SIGNATURES) + list(_OTHER_RESTYPE))

@@ -21,7 +21,7 @@
 typedef struct layer_weights {
     gd_tensor norm1, norm2;
     gd_tensor in, conv, conv_b, dt_bias, a_log, d_skip, gnorm; /* mamba2; in: also [dq | dkv | g] of latent attention */
-    gd_tensor dq_norm, dkv_norm, uq, ukv, uk, uv, freq;        /* latent attention; uk, uv: the two parts of ukv */
+    gd_tensor dq_norm, dkv_norm, uq, ukv, ukt, freq; /* latent attention; ukv: [uk | uv]; ukt: uk turned per head */
     gd_tensor out;
     gd_tensor upgate, upgate_b, down, down_b; /* feed-forward; upgate: [up | gate] */
     gd_tensor ring, states, cache;            /* per slot */
@@ -31,6 +31,7 @@ struct layer_list {
     layer_list_config c;
     gd_dtype type; /* of projections and activations */
     int32_t max_step_tokens;
+    int32_t kv_rows; /* tokens whose keys and values a step may expand at once (latent attention) */
     gd_tensor embed, final_norm;
     layer_weights *layers;
     gd_tensor rows_dev, cu_dev; /* 0 .. batch-1 and 0 .. batch: the tables of a decode step over every slot */
@@ -109,6 +110,7 @@ static gd_status each_weight(const layer_list_config *c, gd_dtype type, struct l
             ONE(AT(layers[i].dkv_norm), GD_DTYPE_F32, a->kv_rank, 0, "mix.dkv.norm", 1.0f, 1.0f);
             ONE(AT(layers[i].uq), type, query_size(l), a->q_rank, "mix.uq", -qr, qr);
             TRY(fn(user, &ukv, i));
+            ONE(AT(layers[i].ukt), type, H * a->kv_rank, a->dim, NULL, 0.0f, 0.0f); /* from ukv */
             ONE(AT(layers[i].freq), GD_DTYPE_F32, a->rot_dim / 2, 0, NULL, 0.0f, 0.0f); /* computed, not stored */
         }
         ONE(AT(layers[i].out), type, c->width, mixer_out(l), "mix.o", -wide, wide);
@@ -145,6 +147,7 @@ typedef struct weight_load {
     gd_safetensors *file;
     uint64_t seed;
     unsigned char *raw, *turned; /* host staging of the largest weight */
+    gd_tensor *ukv;              /* the layer's, already filled */
 } weight_load;
 
 static gd_status allocate_weight(void *user, const weight *w, int32_t layer)
@@ -217,6 +220,21 @@ static gd_status fill_weight(void *user, const weight *w, int32_t layer)
     const int64_t n = weight_count(w);
     int64_t done = 0;
     int p;
+    if (w->piece[0] == NULL && w->cols > 0) { /* ukt [heads, kv_rank, dim] from the first part of ukv [heads, dim, kv_rank] */
+        const gd_backend_latent_args *a = &wl->c->layers[layer].latent;
+        const size_t es = gd_dtype_size(w->type);
+        const int64_t D = a->dim, R = a->kv_rank;
+        gd_tensor uk;
+        TRY(gd_tensor_slice(wl->ctx, wl->ukv, 0U, 0, (int64_t)a->heads * D, &uk));
+        TRY(gd_tensor_read(wl->ctx, &uk, wl->raw, (size_t)n * es));
+#pragma omp parallel for schedule(static)
+        for (done = 0; done < n; ++done) {
+            const int64_t h = done / (R * D), r = done / D % R, d = done % D;
+            memcpy(wl->turned + (size_t)done * es, wl->raw + (size_t)((h * D + d) * R + r) * es, es);
+        }
+        return gd_tensor_write(wl->ctx, w->dst, wl->turned, (size_t)n * es);
+    }
+    if (w->piece[0] != NULL && !strcmp(w->piece[0], "mix.uk")) wl->ukv = w->dst;
     if (w->piece[0] == NULL) { /* rotation frequencies: base^(-2i/dims), in double, rounded once */
         const layer_config *l = &wl->c->layers[layer];
         float *f = (float *)wl->turned;
@@ -252,7 +270,7 @@ static gd_status largest_weight(void *user, const weight *w, int32_t layer)
 
 static gd_status load_weights(gd_context *ctx, struct layer_list *ll, gd_safetensors *file, uint64_t seed)
 {
-    weight_load wl = {ctx, &ll->c, file, seed, NULL, NULL};
+    weight_load wl = {ctx, &ll->c, file, seed, NULL, NULL, NULL};
     int64_t most = 0;
     gd_status st;
     if (file != NULL) TRY(each_weight(&ll->c, ll->type, ll, check_weight, &wl)); /* before the first byte is written */
@@ -330,14 +348,16 @@ static gd_status allocate_states(gd_context *ctx, struct layer_list *ll, int64_t
  * buffers whose largest use decides their size. */
 typedef struct scratch_sizes {
     int64_t proj, a, b, branch; /* elements per row */
-    size_t work;                /* bytes for a step of `rows` rows */
+    int64_t angles;             /* F32 values per row */
+    size_t work;                /* bytes for the whole step */
 } scratch_sizes;
 
 static int64_t max64(int64_t a, int64_t b) { return a > b ? a : b; }
 
-static scratch_sizes sizes_of(const layer_list_config *c, gd_dtype type, int64_t rows, int64_t max_seq)
+static scratch_sizes sizes_of(const layer_list_config *c, gd_dtype type, int64_t rows, int64_t max_new, int64_t kv_total,
+                              int64_t max_seq)
 {
-    scratch_sizes s = {0, c->width, 0, c->width, 256U};
+    scratch_sizes s = {0, c->width, 1, c->width, 1, 256U};
     int32_t i;
     for (i = 0; i < c->n_layers; ++i) {
         const layer_config *l = &c->layers[i];
@@ -346,7 +366,9 @@ static scratch_sizes sizes_of(const layer_list_config *c, gd_dtype type, int64_t
             s.a = max64(s.a, max64(conv_channels(l), inner_size(l)));
             s.b = max64(s.b, inner_size(l));
         } else {
-            const size_t w = gd_backend_latent_work_bytes(NULL, &l->latent, (uint32_t)rows, (uint32_t)max_seq, (uint32_t)type);
+            const size_t w = gd_backend_latent_work_bytes(NULL, &l->latent, (uint32_t)rows, (uint32_t)max_new, (uint32_t)kv_total,
+                                                          (uint32_t)max_seq, (uint32_t)type);
+            s.angles = max64(s.angles, l->latent.rot_dim);
             s.a = max64(s.a, max64(l->latent.q_rank, mixer_out(l)));
             s.b = max64(s.b, query_size(l));
             if (w > s.work) s.work = w;
@@ -356,13 +378,12 @@ static scratch_sizes sizes_of(const layer_list_config *c, gd_dtype type, int64_t
     return s;
 }
 
-static size_t forward_bytes(const layer_list_config *c, gd_dtype type, int64_t rows, int64_t max_seq)
+static size_t forward_bytes(const layer_list_config *c, const scratch_sizes *s, gd_dtype type, int64_t rows)
 {
-    const scratch_sizes s = sizes_of(c, type, rows, max_seq);
     const size_t es = gd_dtype_size(type), R = (size_t)rows;
-    return gd_pad256(R * (size_t)c->width * 4U) + gd_pad256(R * (size_t)c->width * es) + gd_pad256(R * (size_t)s.proj * es) +
-           gd_pad256(R * (size_t)s.a * es) + gd_pad256(R * (size_t)s.b * es) + gd_pad256(R * (size_t)s.branch * es) +
-           gd_pad256(s.work);
+    return gd_pad256(R * (size_t)c->width * 4U) + gd_pad256(R * (size_t)c->width * es) + gd_pad256(R * (size_t)s->proj * es) +
+           gd_pad256(R * (size_t)s->a * es) + gd_pad256(R * (size_t)s->b * es) + gd_pad256(R * (size_t)s->branch * es) +
+           gd_pad256(R * (size_t)s->angles * 4U) + gd_pad256(s->work);
 }
 
 typedef struct forward {
@@ -372,8 +393,8 @@ typedef struct forward {
     uint32_t type;
     int64_t rows;
     gd_backend_packed_seqs seqs;
-    gd_backend_tensor_view row_seq, cu, slot, start, ids;
-    gd_tensor x, h, proj, a, b, branch, work; /* h: the copy of x, or x itself when the projections are F32 */
+    gd_backend_tensor_view row_seq, cu, slot, start, kv_cu, ids;
+    gd_tensor x, h, proj, a, b, branch, angles, work; /* h: the copy of x, or x itself when the projections are F32 */
 } forward;
 
 static void view2(const gd_tensor *t, uint32_t dtype, int64_t d0, int64_t d1, gd_backend_tensor_view *v)
@@ -409,22 +430,31 @@ static gd_status scratch(gd_context *ctx, gd_dtype type, int64_t rows, int64_t c
     return gd_tensor_empty(ctx, GD_ARENA_SCRATCH, type, gd_shape_make(2U, dims), 256U, out);
 }
 
-static gd_status forward_begin(forward *f, gd_gpt_decoder *d, int64_t rows)
+/* kv_total 0: the tokens the sequences hold are not expanded */
+static gd_status forward_begin(forward *f, gd_gpt_decoder *d, int64_t rows, int64_t max_new, int64_t kv_total)
 {
     struct layer_list *ll = d->layers;
-    const scratch_sizes s = sizes_of(&ll->c, ll->type, rows, d->cfg.max_seq);
+    const scratch_sizes s = sizes_of(&ll->c, ll->type, rows, max_new, kv_total, d->cfg.max_seq);
     int64_t wdim[1] = {(int64_t)s.work};
     f->d = d;
     f->be = gd_context_backend(d->ctx);
     f->ll = ll;
     f->type = (uint32_t)ll->type;
     f->rows = rows;
+    f->seqs.row_seq = &f->row_seq;
+    f->seqs.cu = &f->cu;
+    f->seqs.slot = &f->slot;
+    f->seqs.start = &f->start;
+    f->seqs.max_new = (uint32_t)max_new;
+    f->seqs.kv_cu = kv_total > 0 ? &f->kv_cu : NULL;
+    f->seqs.kv_total = (uint32_t)kv_total;
     TRY(scratch(d->ctx, GD_DTYPE_F32, rows, ll->c.width, &f->x));
     if (ll->type == GD_DTYPE_F32) f->h = f->x;
     else TRY(scratch(d->ctx, ll->type, rows, ll->c.width, &f->h));
     TRY(scratch(d->ctx, ll->type, rows, s.proj, &f->proj));
     TRY(scratch(d->ctx, ll->type, rows, s.a, &f->a));
-    TRY(scratch(d->ctx, ll->type, rows, s.b > 0 ? s.b : 1, &f->b));
+    TRY(scratch(d->ctx, ll->type, rows, s.b, &f->b));
+    TRY(scratch(d->ctx, GD_DTYPE_F32, rows, s.angles, &f->angles));
     TRY(scratch(d->ctx, ll->type, rows, s.branch, &f->branch));
     return gd_tensor_empty(d->ctx, GD_ARENA_SCRATCH, GD_DTYPE_U8, gd_shape_make(1U, wdim), 256U, &f->work);
 }
@@ -488,7 +518,7 @@ static gd_status latent_attention(forward *f, const layer_config *l, layer_weigh
     const gd_backend_latent_args *a = &l->latent;
     const int64_t P = mixer_in(l), gate_col = P - mixer_out(l);
     gd_backend_matrix_view pm, gate;
-    gd_backend_tensor_view qn, kn, freq, cq, cache, q, uk, uv, work, out;
+    gd_backend_tensor_view qn, kn, freq, ang, cq, cache, q, ukt, ukv, work, out;
     TRY(project(f, &f->h, &w->in, NULL, 0U, &f->proj));
     columns(&f->proj, f->type, f->rows, P, 0, gate_col, &pm);
     columns(&f->proj, f->type, f->rows, P, gate_col, mixer_out(l), &gate);
@@ -497,14 +527,15 @@ static gd_status latent_attention(forward *f, const layer_config *l, layer_weigh
     tview(&w->freq, &freq);
     tview(&w->cache, &cache);
     view2(&f->a, f->type, f->rows, a->q_rank, &cq);
-    TRY(gd_backend_latent_prepare(f->be, &pm, &qn, &kn, &freq, &cq, &cache, &f->seqs, a));
+    view2(&f->angles, GD_BACKEND_DTYPE_F32, f->rows, a->rot_dim, &ang);
+    TRY(gd_backend_latent_prepare(f->be, &pm, &qn, &kn, &freq, &ang, &cq, &cache, &f->seqs, a));
     TRY(project(f, &f->a, &w->uq, NULL, 0U, &f->b));
     view2(&f->b, f->type, f->rows, query_size(l), &q);
-    tview(&w->uk, &uk);
-    tview(&w->uv, &uv);
+    tview(&w->ukt, &ukt);
+    tview(&w->ukv, &ukv);
     tview(&f->work, &work);
     view2(&f->a, f->type, f->rows, mixer_out(l), &out);
-    TRY(gd_backend_latent_attend(f->be, &q, &uk, &uv, &gate, &freq, &cache, &work, &out, &f->seqs, a));
+    TRY(gd_backend_latent_attend(f->be, &q, &ukt, &ukv, &gate, &ang, &cache, &work, &out, &f->seqs, a));
     return project(f, &f->a, &w->out, NULL, 0U, &f->branch);
 }
 
@@ -558,63 +589,62 @@ static gd_status layer_list_step(gd_gpt_decoder *d, const gd_tensor *ids, const 
 {
     forward f;
     (void)fused; /* one form: its launches are fused as far as they go */
-    TRY(forward_begin(&f, d, d->cfg.batch));
+    TRY(forward_begin(&f, d, d->cfg.batch, 1, 0));
     view1(ids, &f.ids);
     view1(&d->layers->rows_dev, &f.row_seq);
     view1(&d->layers->rows_dev, &f.slot);
     view1(&d->layers->cu_dev, &f.cu);
     view1(positions, &f.start);
-    f.seqs.row_seq = &f.row_seq;
-    f.seqs.cu = &f.cu;
-    f.seqs.slot = &f.slot;
-    f.seqs.start = &f.start;
-    f.seqs.max_new = 1U;
     TRY(run_layers(&f));
     return head(&f, NULL, f.rows, logits);
 }
 
 static gd_status layer_list_extend(gd_gpt_decoder *d, const gd_extend_rows *e, gd_tensor *logits)
 {
-    const int64_t N = e->rows, S = e->n_seqs, total = 2 * N + 3 * S + 1 + e->n_want;
+    enum { IDS, ROW_SEQ, CU, SLOT, START, KV_CU, WANT, PARTS };
+    const int64_t N = e->rows, S = e->n_seqs;
+    const int64_t len[PARTS] = {N, N, S + 1, S, S, S + 1, e->n_want};
+    int64_t at[PARTS + 1], kv_total = 0;
     forward f;
-    gd_tensor tables, part[6];
-    const int64_t at[7] = {0, N, 2 * N, 2 * N + S + 1, 2 * N + 2 * S + 1, 2 * N + 3 * S + 1, total};
+    gd_tensor tables, part[PARTS];
     gd_backend_tensor_view want;
     int32_t *host;
     int32_t s, r;
     gd_status st;
     if (N > d->layers->max_step_tokens) return GD_ERR_INVALID_ARGUMENT;
-    host = (int32_t *)malloc((size_t)total * sizeof(int32_t));
+    at[0] = 0;
+    for (r = 0; r < PARTS; ++r) at[r + 1] = at[r] + len[r];
+    host = (int32_t *)malloc((size_t)at[PARTS] * sizeof(int32_t));
     if (host == NULL) return GD_ERR_OUT_OF_MEMORY;
-    /* one upload: ids, row -> sequence, cu, slots, starts, wanted rows */
-    memcpy(host + at[0], e->ids, (size_t)N * sizeof(int32_t));
+    /* one upload for all tables of the step */
+    memcpy(host + at[IDS], e->ids, (size_t)N * sizeof(int32_t));
+    memcpy(host + at[CU], e->cu, (size_t)(S + 1) * sizeof(int32_t));
+    memcpy(host + at[SLOT], e->slots, (size_t)S * sizeof(int32_t));
+    memcpy(host + at[START], e->start, (size_t)S * sizeof(int32_t));
+    if (e->n_want > 0) memcpy(host + at[WANT], e->want, (size_t)e->n_want * sizeof(int32_t));
+    host[at[KV_CU]] = 0;
     for (s = 0; s < S; ++s) {
-        for (r = e->cu[s]; r < e->cu[s + 1]; ++r) host[at[1] + r] = s;
+        for (r = e->cu[s]; r < e->cu[s + 1]; ++r) host[at[ROW_SEQ] + r] = s;
+        kv_total += e->start[s] + (e->cu[s + 1] - e->cu[s]);
+        host[at[KV_CU] + s + 1] = kv_total <= INT32_MAX ? (int32_t)kv_total : INT32_MAX;
     }
-    memcpy(host + at[2], e->cu, (size_t)(S + 1) * sizeof(int32_t));
-    memcpy(host + at[3], e->slots, (size_t)S * sizeof(int32_t));
-    memcpy(host + at[4], e->start, (size_t)S * sizeof(int32_t));
-    if (e->n_want > 0) memcpy(host + at[5], e->want, (size_t)e->n_want * sizeof(int32_t));
-    st = data_i32(d->ctx, host, total, &tables);
+    if (kv_total > d->layers->kv_rows) kv_total = 0; /* too many tokens to expand at once: the absorbed form */
+    st = data_i32(d->ctx, host, at[PARTS], &tables);
     free(host);
-    for (r = 0; r < 6 && st == GD_OK; ++r) {
-        if (at[r + 1] > at[r]) st = gd_tensor_slice(d->ctx, &tables, 0U, at[r], at[r + 1] - at[r], &part[r]);
+    for (r = 0; r < PARTS && st == GD_OK; ++r) {
+        if (len[r] > 0) st = gd_tensor_slice(d->ctx, &tables, 0U, at[r], len[r], &part[r]);
     }
     if (st != GD_OK) return st;
-    TRY(forward_begin(&f, d, N));
-    view1(&part[0], &f.ids);
-    view1(&part[1], &f.row_seq);
-    view1(&part[2], &f.cu);
-    view1(&part[3], &f.slot);
-    view1(&part[4], &f.start);
-    f.seqs.row_seq = &f.row_seq;
-    f.seqs.cu = &f.cu;
-    f.seqs.slot = &f.slot;
-    f.seqs.start = &f.start;
-    f.seqs.max_new = (uint32_t)e->max_new;
+    TRY(forward_begin(&f, d, N, e->max_new, kv_total));
+    view1(&part[IDS], &f.ids);
+    view1(&part[ROW_SEQ], &f.row_seq);
+    view1(&part[CU], &f.cu);
+    view1(&part[SLOT], &f.slot);
+    view1(&part[START], &f.start);
+    view1(&part[KV_CU], &f.kv_cu);
     TRY(run_layers(&f));
     if (e->n_want == 0) return GD_OK;
-    view1(&part[5], &want);
+    view1(&part[WANT], &want);
     return head(&f, &want, e->n_want, logits);
 }
 
@@ -708,11 +738,19 @@ static gd_status settle(const layer_list_config *c, const gd_model_options *in, 
     return GD_OK;
 }
 
+/* tokens whose keys and values a step may expand: a step of new prompts, and one long sequence continued */
+static int32_t kv_rows(const gd_model_options *o)
+{
+    const int64_t n = (int64_t)o->max_step_tokens + o->max_seq;
+    return n > INT32_MAX ? INT32_MAX : (int32_t)n;
+}
+
 gd_status gd_layer_list_memory(const layer_list_config *c, const gd_model_options *in, gd_memory_config *out)
 {
     gd_model_options o;
     gd_gpt_config g;
-    size_t params = 0U, rows, logit_rows;
+    size_t params = 0U, rows, logit_rows, step;
+    scratch_sizes s;
     TRY(settle(c, in, &o, &g));
     TRY(each_weight(c, o.compute, NULL, add_bytes, &params));
     rows = (size_t)o.max_step_tokens;
@@ -723,12 +761,20 @@ gd_status gd_layer_list_memory(const layer_list_config *c, const gd_model_option
     out->state_bytes = state_bytes(c, o.compute, o.batch, o.max_seq) + gd_decoder_session_bytes(&g, GD_DTYPE_F32, false) + 4096U;
     /* a resident session holds an eager step and a captured one, its records besides; logits of every row of a step,
      * up to 1 GiB of them */
-    out->scratch_slot_bytes = forward_bytes(c, o.compute, (int64_t)rows, o.max_seq) +
-                              2U * forward_bytes(c, o.compute, o.batch, o.max_seq) +
+    /* the largest step: every form attention may take with that many rows */
+    s = sizes_of(c, o.compute, (int64_t)rows, 1, 0, o.max_seq);
+    step = forward_bytes(c, &s, o.compute, (int64_t)rows);
+    s = sizes_of(c, o.compute, (int64_t)rows, (int64_t)rows, kv_rows(&o), o.max_seq);
+    step = step > forward_bytes(c, &s, o.compute, (int64_t)rows) ? step : forward_bytes(c, &s, o.compute, (int64_t)rows);
+    /* few rows are cut into more pieces per row; a resident session has an eager and a captured step */
+    s = sizes_of(c, o.compute, 512, 1, 0, o.max_seq);
+    step += 2U * s.work;
+    s = sizes_of(c, o.compute, o.batch, 1, 0, o.max_seq);
+    out->scratch_slot_bytes = step + 2U * forward_bytes(c, &s, o.compute, o.batch) +
                               logit_rows * (size_t)c->vocab * 4U + rows * (size_t)c->width * 4U +
                               2U * gd_pad256((size_t)o.batch * (size_t)c->vocab * 4U) +
                               (size_t)o.batch * (size_t)o.max_seq * 8U + ((size_t)16 << 20);
-    out->data_slot_bytes = rows * 12U + (size_t)o.batch * 64U + ((size_t)1 << 20);
+    out->data_slot_bytes = rows * 16U + (size_t)o.batch * 64U + ((size_t)1 << 20);
     out->scratch_slots = 2U;
     out->data_slots = 2U;
     return GD_OK;
@@ -751,7 +797,6 @@ gd_status gd_layer_list_create(gd_context *ctx, const layer_list_config *c, cons
     gd_gpt_decoder *d;
     struct layer_list *ll;
     gd_status st;
-    int32_t i;
     *out = NULL;
     TRY(settle(c, in, &o, &g));
     TRY(gd_decoder_session_create(ctx, &layer_list_model, &g, &d));
@@ -760,19 +805,11 @@ gd_status gd_layer_list_create(gd_context *ctx, const layer_list_config *c, cons
     if (st == GD_OK) {
         ll->type = o.compute;
         ll->max_step_tokens = o.max_step_tokens;
+        ll->kv_rows = kv_rows(&o);
         ll->layers = (layer_weights *)calloc((size_t)c->n_layers, sizeof(layer_weights));
         if (ll->layers == NULL) st = GD_ERR_OUT_OF_MEMORY;
     }
     if (st == GD_OK) st = load_weights(ctx, ll, weights, seed);
-    for (i = 0; i < c->n_layers && st == GD_OK; ++i) {
-        const layer_config *l = &c->layers[i];
-        const int64_t keys = (int64_t)l->latent.heads * l->latent.dim;
-        if (l->mixer != MIXER_LATENT_ATTENTION) continue;
-        st = gd_tensor_slice(ctx, &ll->layers[i].ukv, 0U, 0, keys, &ll->layers[i].uk);
-        if (st == GD_OK)
-            st = gd_tensor_slice(ctx, &ll->layers[i].ukv, 0U, keys, (int64_t)l->latent.heads * l->latent.vdim,
-                                 &ll->layers[i].uv);
-    }
     if (st == GD_OK) st = allocate_states(ctx, ll, o.batch, o.max_seq);
     if (st == GD_OK) st = gd_decoder_session_allocate(d, GD_DTYPE_F32, false);
     if (st != GD_OK) {

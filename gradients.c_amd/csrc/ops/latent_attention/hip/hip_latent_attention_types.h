@@ -8,5 +8,7 @@ typedef struct gd_hip_latent_params {
     uint32_t pitch; /* elements per cache row and per absorbed query row: kv_rank + rot_dim rounded up to 8 */
     uint32_t tmax;  /* cache rows per slot */
     float scale, eps;
+    /* matrix-core decode form: keys per piece and pieces per row (piece results [rows, pieces, heads]) */
+    uint32_t piece_keys, pieces;
 } gd_hip_latent_params;
 #endif

@@ -1,7 +1,7 @@
 /*
  * Row kernels of latent attention (gfx950), any sizes, BF16 and F32:
- *   prepare  per new token: RMS norm of the query latent; RMS norm of the key/value latent and rotation of the shared
- *            key part, both into the token's cache row
+ *   prepare  per new token: cosines and sines of its position; RMS norm of the query latent; RMS norm of the key/value
+ *            latent and rotation of the shared key part, both into the token's cache row
  *   query    per token and head: the unrotated query taken through the key up-projection, so that its product with a
  *            latent is its product with the key (q . (W_uk c) = (W_uk^T q) . c), and the rotated part turned to its
  *            position: one absorbed query row of a cache row's layout
@@ -13,20 +13,11 @@
 #include "../../_shared/hip_device.h"
 #include "hip_latent_attention_types.h"
 
-/* (u, v) turned by angle position * freq */
-__device__ __forceinline__ void gd_latent_turn(float u, float v, int32_t pos, float freq, float *a, float *b)
-{
-    float s, c;
-    sincosf((float)pos * freq, &s, &c);
-    *a = u * c - v * s;
-    *b = v * c + u * s;
-}
-
 template <typename T>
 __global__ void __launch_bounds__(256)
 gd_latent_prepare_kernel(const T *__restrict__ proj, uint32_t ld, const float *__restrict__ q_norm,
-                         const float *__restrict__ kv_norm, const float *__restrict__ freq, T *__restrict__ cq,
-                         T *__restrict__ cache, gd_hip_latent_params m, gd_hip_seqs q)
+                         const float *__restrict__ kv_norm, const float *__restrict__ freq, float *__restrict__ angles,
+                         T *__restrict__ cq, T *__restrict__ cache, gd_hip_latent_params m, gd_hip_seqs q)
 {
     __shared__ float red[2][4];
     const uint32_t row = blockIdx.x;
@@ -45,40 +36,40 @@ gd_latent_prepare_kernel(const T *__restrict__ proj, uint32_t ld, const float *_
     for (uint32_t c = threadIdx.x; c < m.kv_rank; c += 256u) dst[c] = (T)((float)pc[c] * ic * kv_norm[c]);
     const uint32_t half = m.rot_dim / 2u;
     for (uint32_t i = threadIdx.x; i < half; i += 256u) {
-        float a, b;
-        gd_latent_turn((float)pr[i], (float)pr[half + i], pos, freq[i], &a, &b);
-        dst[m.kv_rank + i] = (T)a;
-        dst[m.kv_rank + half + i] = (T)b;
+        const float u = (float)pr[i], v = (float)pr[half + i];
+        float s1, c1;
+        sincosf((float)pos * freq[i], &s1, &c1);
+        angles[(size_t)row * m.rot_dim + i] = c1;
+        angles[(size_t)row * m.rot_dim + half + i] = s1;
+        dst[m.kv_rank + i] = (T)(u * c1 - v * s1);
+        dst[m.kv_rank + half + i] = (T)(v * c1 + u * s1);
     }
     for (uint32_t c = m.kv_rank + m.rot_dim + threadIdx.x; c < m.pitch; c += 256u) dst[c] = (T)0.f;
 }
 
-/* grid (rows, heads); ql [rows, heads, pitch] */
+/* grid (rows, heads); w_ukt [heads, kv_rank, dim]; ql [rows, heads, pitch] */
 template <typename T>
 __global__ void __launch_bounds__(256)
-gd_latent_query_kernel(const T *__restrict__ qv, const T *__restrict__ w_uk, const float *__restrict__ freq,
-                       T *__restrict__ ql, gd_hip_latent_params m, gd_hip_seqs q)
+gd_latent_query_kernel(const T *__restrict__ qv, const T *__restrict__ w_ukt, const float *__restrict__ angles,
+                       T *__restrict__ ql, gd_hip_latent_params m)
 {
     extern __shared__ float sq[]; /* dim */
-    const uint32_t row = blockIdx.x, h = blockIdx.y;
-    int32_t s, pos, slot;
-    if (!gd_seq_of_row(q, row, &s, &pos, &slot)) return;
-    const T *src = qv + (size_t)row * m.heads * (m.dim + m.rot_dim) + h * (m.dim + m.rot_dim);
+    const uint32_t row = blockIdx.x, h = blockIdx.y, half = m.rot_dim / 2u;
+    const T *src = qv + ((size_t)row * m.heads + h) * (m.dim + m.rot_dim);
     for (uint32_t d = threadIdx.x; d < m.dim; d += 256u) sq[d] = (float)src[d];
     __syncthreads();
     T *dst = ql + ((size_t)row * m.heads + h) * m.pitch;
-    const T *w = w_uk + (size_t)h * m.dim * m.kv_rank;
     for (uint32_t c = threadIdx.x; c < m.kv_rank; c += 256u) {
+        const T *w = w_ukt + ((size_t)h * m.kv_rank + c) * m.dim;
         float a = 0.f;
-        for (uint32_t d = 0; d < m.dim; ++d) a = fmaf(sq[d], (float)w[(size_t)d * m.kv_rank + c], a);
+        for (uint32_t d = 0; d < m.dim; ++d) a = fmaf(sq[d], (float)w[d], a);
         dst[c] = (T)a;
     }
-    const uint32_t half = m.rot_dim / 2u;
     for (uint32_t i = threadIdx.x; i < half; i += 256u) {
-        float a, b;
-        gd_latent_turn((float)src[m.dim + i], (float)src[m.dim + half + i], pos, freq[i], &a, &b);
-        dst[m.kv_rank + i] = (T)a;
-        dst[m.kv_rank + half + i] = (T)b;
+        const float u = (float)src[m.dim + i], v = (float)src[m.dim + half + i];
+        const float c1 = angles[(size_t)row * m.rot_dim + i], s1 = angles[(size_t)row * m.rot_dim + half + i];
+        dst[m.kv_rank + i] = (T)(u * c1 - v * s1);
+        dst[m.kv_rank + half + i] = (T)(v * c1 + u * s1);
     }
     for (uint32_t c = m.kv_rank + m.rot_dim + threadIdx.x; c < m.pitch; c += 256u) dst[c] = (T)0.f;
 }
@@ -156,22 +147,20 @@ gd_latent_value_kernel(const float *__restrict__ o_lat, const T *__restrict__ w_
 }
 
 extern "C" int gd_hip_launch_latent_prepare(hipStream_t stream, const void *proj, uint32_t ld, const float *q_norm,
-                                            const float *kv_norm, const float *freq, void *cq, void *cache,
+                                            const float *kv_norm, const float *freq, float *angles, void *cq, void *cache,
                                             const gd_hip_latent_params *m, const gd_hip_seqs *q, int is_f32)
 {
-    if (q->rows == 0u) return (int)hipSuccess;
-#define GD_GO(T) gd_latent_prepare_kernel<T><<<q->rows, 256, 0, stream>>>((const T *)proj, ld, q_norm, kv_norm, freq, (T *)cq, (T *)cache, *m, *q)
+#define GD_GO(T) gd_latent_prepare_kernel<T><<<q->rows, 256, 0, stream>>>((const T *)proj, ld, q_norm, kv_norm, freq, angles, (T *)cq, (T *)cache, *m, *q)
     if (is_f32) GD_GO(float); else GD_GO(gd_bf16);
 #undef GD_GO
     return (int)hipGetLastError();
 }
 
-extern "C" int gd_hip_launch_latent_query(hipStream_t stream, const void *qv, const void *w_uk, const float *freq,
+extern "C" int gd_hip_launch_latent_query(hipStream_t stream, const void *qv, const void *w_ukt, const float *angles,
                                           void *ql, const gd_hip_latent_params *m, const gd_hip_seqs *q, int is_f32)
 {
     const dim3 grid(q->rows, m->heads);
-    if (q->rows == 0u) return (int)hipSuccess;
-#define GD_GO(T) gd_latent_query_kernel<T><<<grid, 256, m->dim * sizeof(float), stream>>>((const T *)qv, (const T *)w_uk, freq, (T *)ql, *m, *q)
+#define GD_GO(T) gd_latent_query_kernel<T><<<grid, 256, m->dim * sizeof(float), stream>>>((const T *)qv, (const T *)w_ukt, angles, (T *)ql, *m)
     if (is_f32) GD_GO(float); else GD_GO(gd_bf16);
 #undef GD_GO
     return (int)hipGetLastError();
