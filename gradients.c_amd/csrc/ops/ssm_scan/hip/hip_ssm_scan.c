@@ -5,8 +5,14 @@
 int gd_hip_launch_ssm_scan(hipStream_t stream, const void *xbc, const void *dt_raw, const float *dt_bias,
                            const float *a_log, const float *d_skip, float *states, void *y, const gd_hip_ssm_params *m,
                            const gd_hip_seqs *q, int is_f32);
+int gd_hip_launch_ssm_scan_chunk(hipStream_t stream, const void *xbc, const void *dt_raw, const float *dt_bias,
+                                 const float *a_log, const float *d_skip, float *states, void *y,
+                                 const gd_hip_ssm_params *m, const gd_hip_seqs *q);
 int gd_hip_launch_gated_group_norm(hipStream_t stream, const void *y, const void *z, uint32_t ldz, const float *w,
                                    void *out, uint32_t rows, uint32_t inner, uint32_t groups, float eps, int is_f32);
+
+/* new rows of a sequence from which the chunked matrix-core form is taken */
+#define GD_HIP_SSM_CHUNK_FROM 17u
 
 gd_status gd_backend_ssm_scan(gd_backend *backend, const gd_backend_tensor_view *xbc, const gd_backend_matrix_view *dt,
                               const gd_backend_tensor_view *dt_bias, const gd_backend_tensor_view *a_log,
@@ -39,6 +45,12 @@ gd_status gd_backend_ssm_scan(gd_backend *backend, const gd_backend_tensor_view 
     m.groups = args->groups;
     m.ld_xbc = (uint32_t)cols;
     m.ld_dt = (uint32_t)(dt->row_bytes / gd_hip_dtype_size(dt->dtype));
+    if (xbc->dtype == GD_BACKEND_DTYPE_BF16 && q.max_new >= GD_HIP_SSM_CHUNK_FROM && (m.state % 8u) == 0u &&
+        m.state <= 256u && (m.vdim % 8u) == 0u && ((xbc->offset | y->offset) & 15u) == 0u)
+        return gd_hip_finish_op(backend, gd_hip_launch_ssm_scan_chunk(
+            backend->stream, gd_hip_view_ptr(xbc), gd_hip_matrix_ptr(dt), (const float *)gd_hip_view_ptr(dt_bias),
+            (const float *)gd_hip_view_ptr(a_log), (const float *)gd_hip_view_ptr(d_skip), (float *)gd_hip_view_ptr(states),
+            gd_hip_view_ptr(y), &m, &q));
     return gd_hip_finish_op(backend, gd_hip_launch_ssm_scan(
         backend->stream, gd_hip_view_ptr(xbc), gd_hip_matrix_ptr(dt), (const float *)gd_hip_view_ptr(dt_bias),
         (const float *)gd_hip_view_ptr(a_log), (const float *)gd_hip_view_ptr(d_skip), (float *)gd_hip_view_ptr(states),
