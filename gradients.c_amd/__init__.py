@@ -25,9 +25,19 @@ INVALID_ARGUMENT, BAD_STATE, UNSUPPORTED = -1, -5, -6
 
 # dtype codes (reference include/gradients/tensor.h:49-57)
 F16, BF16, F32, I32, U8, U16 = 1, 2, 3, 4, 5, 6
-_NP_DTYPE = {F16: np.float16, F32: np.float32, I32: np.int32, U8: np.uint8, U16: np.uint16}
+_NP_DTYPE = {F16: np.float16, BF16: np.uint16, F32: np.float32, I32: np.int32, U8: np.uint8, U16: np.uint16}
 _CODE_OF = {np.dtype(np.float16): F16, np.dtype(np.float32): F32, np.dtype(np.int32): I32,
             np.dtype(np.uint8): U8, np.dtype(np.uint16): U16}
+
+
+def bf16_bits(values):
+    """float -> BF16 bits, to nearest, ties to even (finite values)."""
+    u = np.ascontiguousarray(values, np.float32).view(np.uint32)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def bf16_values(bits):
+    return (np.ascontiguousarray(bits, np.uint16).astype(np.uint32) << 16).view(np.float32)
 
 
 class GdError(RuntimeError):
@@ -298,6 +308,14 @@ class Tensor:
         assert a.size == self.count, (a.shape, self.shape)
         self.buffer.upload(self.offset, a)
         return self
+
+    def write_float(self, array):
+        """Real values into a tensor of any floating type (BF16: rounded to nearest even)."""
+        return self.write(bf16_bits(array) if self.dtype == BF16 else array)
+
+    def read_float(self):
+        a = self.read()
+        return bf16_values(a) if self.dtype == BF16 else a.astype(np.float32)
 
     def read(self):
         out = np.empty(self.shape, _NP_DTYPE[self.dtype])
