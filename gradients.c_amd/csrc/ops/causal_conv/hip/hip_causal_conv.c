@@ -2,7 +2,8 @@
 #include "../../_shared/packed_seqs_host.h"
 
 int gd_hip_launch_causal_conv_silu(hipStream_t stream, const void *u, uint32_t ldu, const float *w, const float *bias,
-                                   void *ring, void *out, uint32_t C, uint32_t K, const gd_hip_seqs *q, int is_f32);
+                                   void *ring, void *out, uint32_t C, uint32_t K, const gd_hip_seqs *q, int is_f32,
+                                   int aligned16);
 
 gd_status gd_backend_causal_conv_silu(gd_backend *backend, const gd_backend_matrix_view *x,
                                       const gd_backend_tensor_view *taps, const gd_backend_tensor_view *bias,
@@ -21,5 +22,6 @@ gd_status gd_backend_causal_conv_silu(gd_backend *backend, const gd_backend_matr
     return gd_hip_finish_op(backend, gd_hip_launch_causal_conv_silu(
         backend->stream, gd_hip_matrix_ptr(x), (uint32_t)(x->row_bytes / gd_hip_dtype_size(x->dtype)),
         (const float *)gd_hip_view_ptr(taps), (const float *)gd_hip_view_ptr(bias), gd_hip_view_ptr(ring),
-        gd_hip_view_ptr(out), x->cols, (uint32_t)taps->shape[1], &q, x->dtype == GD_BACKEND_DTYPE_F32));
+        gd_hip_view_ptr(out), x->cols, (uint32_t)taps->shape[1], &q, x->dtype == GD_BACKEND_DTYPE_F32,
+        ((x->offset | x->row_bytes | ring->offset | out->offset) & 15u) == 0u));
 }

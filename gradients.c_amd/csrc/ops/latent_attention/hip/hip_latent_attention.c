@@ -4,7 +4,7 @@
 
 int gd_hip_launch_latent_prepare(hipStream_t stream, const void *proj, uint32_t ld, const float *q_norm,
                                  const float *kv_norm, const float *freq, float *angles, void *cq, void *cache,
-                                 const gd_hip_latent_params *m, const gd_hip_seqs *q, int is_f32);
+                                 const gd_hip_latent_params *m, const gd_hip_seqs *q, int is_f32, int aligned16);
 int gd_hip_launch_latent_query(hipStream_t stream, const void *qv, const void *w_ukt, const float *angles, void *ql,
                                const gd_hip_latent_params *m, const gd_hip_seqs *q, int is_f32);
 int gd_hip_launch_latent_attend(hipStream_t stream, const void *ql, const void *cache, float *o_lat,
@@ -141,7 +141,8 @@ gd_status gd_backend_latent_prepare(gd_backend *backend, const gd_backend_matrix
     return gd_hip_finish_op(backend, gd_hip_launch_latent_prepare(
         backend->stream, gd_hip_matrix_ptr(proj), (uint32_t)(proj->row_bytes / gd_hip_dtype_size(proj->dtype)),
         (const float *)gd_hip_view_ptr(q_norm), (const float *)gd_hip_view_ptr(kv_norm), (const float *)gd_hip_view_ptr(freq),
-        (float *)gd_hip_view_ptr(angles), gd_hip_view_ptr(cq), gd_hip_view_ptr(cache), &m, &q, proj->dtype == GD_BACKEND_DTYPE_F32));
+        (float *)gd_hip_view_ptr(angles), gd_hip_view_ptr(cq), gd_hip_view_ptr(cache), &m, &q, proj->dtype == GD_BACKEND_DTYPE_F32,
+        ((proj->offset | proj->row_bytes | cq->offset | cache->offset) & 15u) == 0u));
 }
 
 static bool aligned16(const gd_backend_tensor_view *a, const gd_backend_tensor_view *b, const gd_backend_tensor_view *c)

@@ -47,6 +47,66 @@ gd_latent_prepare_kernel(const T *__restrict__ proj, uint32_t ld, const float *_
     for (uint32_t c = m.kv_rank + m.rot_dim + threadIdx.x; c < m.pitch; c += 256u) dst[c] = (T)0.f;
 }
 
+/* prepare for BF16 rows of q_rank + kv_rank <= 4096 in 16-byte pieces: a wavefront per row, the row in registers */
+__global__ void __launch_bounds__(256)
+gd_latent_prepare_vec_kernel(const gd_bf16 *__restrict__ proj, uint32_t ld, const float *__restrict__ q_norm,
+                             const float *__restrict__ kv_norm, const float *__restrict__ freq, float *__restrict__ angles,
+                             gd_bf16 *__restrict__ cq, gd_bf16 *__restrict__ cache, gd_hip_latent_params m, gd_hip_seqs q)
+{
+    constexpr int KEEP = 8;
+    const uint32_t row = blockIdx.x * 4u + (threadIdx.x >> 6), lane = threadIdx.x & 63u;
+    if (row >= q.rows) return;
+    const gd_bf16 *pr = proj + (size_t)row * ld;
+    const uint32_t qc = m.q_rank / 8u, all = qc + m.kv_rank / 8u, half = m.rot_dim / 2u;
+    int32_t s, pos, slot;
+    const bool live = gd_seq_of_row(q, row, &s, &pos, &slot) && (uint32_t)pos < m.tmax;
+    gd_bf16x8 v[KEEP];
+    float sq = 0.f, sc = 0.f;
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        const uint32_t c = lane + 64u * i;
+        if (c < all) v[i] = *reinterpret_cast<const gd_bf16x8 *>(pr + c * 8u);
+    }
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        const uint32_t c = lane + 64u * i;
+        if (c >= all) continue;
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss = fmaf((float)v[i][e], (float)v[i][e], ss);
+        if (c < qc) sq += ss;
+        else sc += ss;
+    }
+    sq = gd_wave_sum(sq);
+    sc = gd_wave_sum(sc);
+    const float iq = 1.0f / sqrtf(sq / (float)m.q_rank + m.eps), ic = 1.0f / sqrtf(sc / (float)m.kv_rank + m.eps);
+    gd_bf16 *dst = cache + ((size_t)(live ? slot : 0) * m.tmax + (uint32_t)(live ? pos : 0)) * m.pitch;
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        const uint32_t c = lane + 64u * i;
+        if (c >= all) continue;
+        const bool is_q = c < qc;
+        const float inv = is_q ? iq : ic, *w = is_q ? q_norm + c * 8u : kv_norm + (c - qc) * 8u;
+        gd_bf16x8 o;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = (gd_bf16)((float)v[i][e] * inv * w[e]);
+        if (is_q) *reinterpret_cast<gd_bf16x8 *>(cq + (size_t)row * m.q_rank + c * 8u) = o;
+        else if (live) *reinterpret_cast<gd_bf16x8 *>(dst + (c - qc) * 8u) = o;
+    }
+    if (!live) return;
+    const gd_bf16 *rot = pr + m.q_rank + m.kv_rank;
+    for (uint32_t i = lane; i < half; i += 64u) {
+        const float a = (float)rot[i], b = (float)rot[half + i];
+        float s1, c1;
+        sincosf((float)pos * freq[i], &s1, &c1);
+        angles[(size_t)row * m.rot_dim + i] = c1;
+        angles[(size_t)row * m.rot_dim + half + i] = s1;
+        dst[m.kv_rank + i] = (gd_bf16)(a * c1 - b * s1);
+        dst[m.kv_rank + half + i] = (gd_bf16)(b * c1 + a * s1);
+    }
+    for (uint32_t c = m.kv_rank + m.rot_dim + lane; c < m.pitch; c += 64u) dst[c] = (gd_bf16)0.f;
+}
+
 /* grid (rows, heads); w_ukt [heads, kv_rank, dim]; ql [rows, heads, pitch] */
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -148,8 +208,13 @@ gd_latent_value_kernel(const float *__restrict__ o_lat, const T *__restrict__ w_
 
 extern "C" int gd_hip_launch_latent_prepare(hipStream_t stream, const void *proj, uint32_t ld, const float *q_norm,
                                             const float *kv_norm, const float *freq, float *angles, void *cq, void *cache,
-                                            const gd_hip_latent_params *m, const gd_hip_seqs *q, int is_f32)
+                                            const gd_hip_latent_params *m, const gd_hip_seqs *q, int is_f32, int aligned16)
 {
+    if (!is_f32 && aligned16 && (m->q_rank % 8u) == 0u && (m->kv_rank % 8u) == 0u && m->q_rank + m->kv_rank <= 4096u) {
+        gd_latent_prepare_vec_kernel<<<(q->rows + 3u) / 4u, 256, 0, stream>>>(
+            (const gd_bf16 *)proj, ld, q_norm, kv_norm, freq, angles, (gd_bf16 *)cq, (gd_bf16 *)cache, *m, *q);
+        return (int)hipGetLastError();
+    }
 #define GD_GO(T) gd_latent_prepare_kernel<T><<<q->rows, 256, 0, stream>>>((const T *)proj, ld, q_norm, kv_norm, freq, angles, (T *)cq, (T *)cache, *m, *q)
     if (is_f32) GD_GO(float); else GD_GO(gd_bf16);
 #undef GD_GO

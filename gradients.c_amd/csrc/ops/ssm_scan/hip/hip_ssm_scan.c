@@ -9,7 +9,8 @@ int gd_hip_launch_ssm_scan_chunk(hipStream_t stream, const void *xbc, const void
                                  const float *a_log, const float *d_skip, float *states, void *y,
                                  const gd_hip_ssm_params *m, const gd_hip_seqs *q);
 int gd_hip_launch_gated_group_norm(hipStream_t stream, const void *y, const void *z, uint32_t ldz, const float *w,
-                                   void *out, uint32_t rows, uint32_t inner, uint32_t groups, float eps, int is_f32);
+                                   void *out, uint32_t rows, uint32_t inner, uint32_t groups, float eps, int is_f32,
+                                   int aligned16);
 
 /* new rows of a sequence from which the chunked matrix-core form is taken */
 #define GD_HIP_SSM_CHUNK_FROM 17u
@@ -70,5 +71,5 @@ gd_status gd_backend_gated_group_norm(gd_backend *backend, const gd_backend_tens
     return gd_hip_finish_op(backend, gd_hip_launch_gated_group_norm(
         backend->stream, gd_hip_view_ptr(y), gd_hip_matrix_ptr(z), (uint32_t)(z->row_bytes / gd_hip_dtype_size(z->dtype)),
         (const float *)gd_hip_view_ptr(weight), gd_hip_view_ptr(out), z->rows, z->cols, parts, eps,
-        y->dtype == GD_BACKEND_DTYPE_F32));
+        y->dtype == GD_BACKEND_DTYPE_F32, ((y->offset | z->offset | z->row_bytes | out->offset) & 15u) == 0u));
 }

@@ -163,12 +163,57 @@ gd_gated_group_norm_kernel(const T *__restrict__ y, const T *__restrict__ z, uin
         o[c] = (T)((float)yr[c] * gd_silu_f32((float)zr[c]) * inv * w[c0 + c]);
 }
 
+/* BF16 with parts of a multiple of 8 up to 8192 and 16-byte aligned rows: the part stays in registers */
+__global__ void __launch_bounds__(256)
+gd_gated_group_norm_vec_kernel(const gd_bf16 *__restrict__ y, const gd_bf16 *__restrict__ z, uint32_t ldz,
+                               const float *__restrict__ w, gd_bf16 *__restrict__ out, uint32_t part, uint32_t inner,
+                               float eps)
+{
+    __shared__ float red[4];
+    const uint32_t c0 = blockIdx.y * part;
+    const gd_bf16 *yr = y + (size_t)blockIdx.x * inner + c0, *zr = z + (size_t)blockIdx.x * ldz + c0;
+    constexpr int KEEP = 4;
+    gd_bf16x8 yv[KEEP], zv[KEEP];
+    float v[KEEP][8], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        const uint32_t c = (threadIdx.x + 256u * i) * 8u;
+        if (c >= part) continue;
+        yv[i] = *reinterpret_cast<const gd_bf16x8 *>(yr + c);
+        zv[i] = *reinterpret_cast<const gd_bf16x8 *>(zr + c);
+    }
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        if ((threadIdx.x + 256u * i) * 8u >= part) continue;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            v[i][e] = (float)yv[i][e] * gd_silu_f32((float)zv[i][e]);
+            ss = fmaf(v[i][e], v[i][e], ss);
+        }
+    }
+    ss = gd_block_sum<4>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)part + eps);
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        const uint32_t c = (threadIdx.x + 256u * i) * 8u;
+        if (c >= part) continue;
+        gd_bf16x8 o;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = (gd_bf16)(v[i][e] * inv * w[c0 + c + e]);
+        *reinterpret_cast<gd_bf16x8 *>(out + (size_t)blockIdx.x * inner + c0 + c) = o;
+    }
+}
+
 extern "C" int gd_hip_launch_gated_group_norm(hipStream_t stream, const void *y, const void *z, uint32_t ldz,
                                               const float *w, void *out, uint32_t rows, uint32_t inner, uint32_t groups,
-                                              float eps, int is_f32)
+                                              float eps, int is_f32, int aligned16)
 {
     const dim3 grid(rows, groups);
     if (rows == 0u) return (int)hipSuccess;
+    if (!is_f32 && aligned16 && (inner / groups) % 8u == 0u && inner / groups <= 8192u) {
+        gd_gated_group_norm_vec_kernel<<<grid, 256, 0, stream>>>((const gd_bf16 *)y, (const gd_bf16 *)z, ldz, w, (gd_bf16 *)out, inner / groups, inner, eps);
+        return (int)hipGetLastError();
+    }
     if (is_f32)
         gd_gated_group_norm_kernel<float><<<grid, 256, 0, stream>>>((const float *)y, (const float *)z, ldz, w, (float *)out, inner / groups, inner, eps);
     else

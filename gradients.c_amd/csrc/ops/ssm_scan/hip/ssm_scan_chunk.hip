@@ -52,12 +52,14 @@ struct gd_sc_layout {
     static constexpr uint32_t BC = NP * 2u + 16u; /* bytes per token row of B and C; per column row of S^T */
     static constexpr uint32_t XS = PT * 2u + 16u; /* per token row of X */
     static constexpr uint32_t MS = GD_SC_L * 2u + 16u;
-    static constexpr uint32_t b = 0u, c = b + GD_SC_L * BC, x = c + GD_SC_L * BC, mh = x + GD_SC_L * XS, ml = mh + GD_SC_L * MS,
-                              sh = ml + GD_SC_L * MS, sl = sh + PT * BC, end = sl + PT * BC;
+    /* M takes the place of C, which is used up when M is written */
+    static constexpr uint32_t CM = BC > 2u * MS ? GD_SC_L * BC : GD_SC_L * 2u * MS;
+    static constexpr uint32_t b = 0u, c = b + GD_SC_L * BC, mh = c, ml = mh + GD_SC_L * MS, x = c + CM, sh = x + GD_SC_L * XS,
+                              sl = sh + PT * BC, end = sl + PT * BC;
 };
 
 template <int NP>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, NP <= 128 ? 2 : 1)
 gd_ssm_scan_chunk_kernel(const gd_bf16 *__restrict__ xbc, const gd_bf16 *__restrict__ dt_raw,
                          const float *__restrict__ dt_bias, const float *__restrict__ a_log,
                          const float *__restrict__ d_skip, float *__restrict__ states, gd_bf16 *__restrict__ y,
@@ -67,7 +69,7 @@ gd_ssm_scan_chunk_kernel(const gd_bf16 *__restrict__ xbc, const gd_bf16 *__restr
     constexpr int TILES = NP / 32 * 2, TPW = (TILES + 3) / 4; /* 32 x 32 tiles of the state, per wavefront */
     constexpr int NCH = NP / 8;                               /* 16-byte chunks per token of B and C */
     extern __shared__ __align__(16) unsigned char sm[];
-    __shared__ float s_cs[GD_SC_L], s_dt[GD_SC_L], s_w[GD_SC_L];
+    __shared__ __align__(16) float s_cs[GD_SC_L], s_dt[GD_SC_L], s_w[GD_SC_L]; /* cs in the exp2 domain */
     const uint32_t tid = threadIdx.x, lane = tid & 63u, lc = lane & 31u, hh = lane >> 5;
     const uint32_t wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const uint32_t p0 = blockIdx.x * L::PT, h = blockIdx.y, N = m.state, P = m.vdim, inner = m.heads * P;
@@ -75,7 +77,7 @@ gd_ssm_scan_chunk_kernel(const gd_bf16 *__restrict__ xbc, const gd_bf16 *__restr
     int32_t first, n, start, slot;
     if (!gd_seq_span(q, blockIdx.z, &first, &n, &start, &slot)) return;
     float *st = states + ((size_t)slot * m.heads + h) * N * P + p0;
-    const float rate = expf(a_log[h]), bias = dt_bias[h], skip = d_skip[h];
+    const float rate = expf(a_log[h]) * 1.4426950408889634f, bias = dt_bias[h], skip = d_skip[h];
 
     /* the state: tile t of this wavefront covers rows 32 * nb, columns 32 * pb */
     gd_float16 S[TPW];
@@ -139,7 +141,7 @@ gd_ssm_scan_chunk_kernel(const gd_bf16 *__restrict__ xbc, const gd_bf16 *__restr
             }
             s_cs[lane] = cs;
             s_dt[lane] = dt;
-            s_w[lane] = expf(__shfl(cs, 63, 64) - cs) * dt;
+            s_w[lane] = __builtin_amdgcn_exp2f(__shfl(cs, 63, 64) - cs) * dt;
         }
         /* the state in front of the chunk as S^T, in two parts */
 #pragma unroll
@@ -164,55 +166,51 @@ gd_ssm_scan_chunk_kernel(const gd_bf16 *__restrict__ xbc, const gd_bf16 *__restr
         if (t0 + (int32_t)GD_SC_L < n) request(t0 + (int32_t)GD_SC_L);
         __syncthreads();
 
-        /* M^T quadrants: G^T = B C^T keeps a lane's registers along j, four consecutive ones per store of M[i][j] */
-        const uint32_t ib = wave >> 1, jb = wave & 1u;
-        if (jb <= ib) {
-            gd_float16 acc;
+        /* G^T = B C^T keeps a lane's registers along j, four consecutive ones per store of M[i][j]; Y^T: rows p (columns
+         * 32 * pb of the slice), columns i (row block ib): a lane holds one token */
+        const uint32_t ib = wave >> 1, jb = wave & 1u, pb = jb, i = 32u * ib + lc;
+        gd_float16 gm, ys;
 #pragma unroll
-            for (int e = 0; e < 16; ++e) acc[e] = 0.f;
+        for (int e = 0; e < 16; ++e) gm[e] = ys[e] = 0.f;
 #pragma unroll
-            for (int ks = 0; ks < NP / 16; ++ks) {
-                const uint32_t c = (16u * ks + 8u * hh) * 2u;
+        for (int ks = 0; ks < NP / 16; ++ks) {
+            const uint32_t c = (16u * ks + 8u * hh) * 2u;
+            const gd_bf16x8 cv = *reinterpret_cast<const gd_bf16x8 *>(sm + L::c + i * L::BC + c);
+            const gd_bf16x8 ah = *reinterpret_cast<const gd_bf16x8 *>(sm + L::sh + (32u * pb + lc) * L::BC + c);
+            const gd_bf16x8 al = *reinterpret_cast<const gd_bf16x8 *>(sm + L::sl + (32u * pb + lc) * L::BC + c);
+            if (jb <= ib) {
                 const gd_bf16x8 bv = *reinterpret_cast<const gd_bf16x8 *>(sm + L::b + (32u * jb + lc) * L::BC + c);
-                const gd_bf16x8 cv = *reinterpret_cast<const gd_bf16x8 *>(sm + L::c + (32u * ib + lc) * L::BC + c);
-                acc = GD_MFMA(bv, cv, acc);
+                gm = GD_MFMA(bv, cv, gm);
             }
-            const uint32_t i = 32u * ib + lc;
-            const float ci = s_cs[i];
+            ys = GD_MFMA(ah, cv, ys);
+            ys = GD_MFMA(al, cv, ys);
+        }
+        const float ci = s_cs[i];
+        __syncthreads(); /* C is used up: M takes its place */
+        if (jb <= ib) {
 #pragma unroll
             for (int a = 0; a < 4; ++a) {
+                const uint32_t j0 = 32u * jb + 8u * (uint32_t)a + 4u * hh;
+                const gd_float4 cj = *reinterpret_cast<const gd_float4 *>(&s_cs[j0]);
+                const gd_float4 dj = *reinterpret_cast<const gd_float4 *>(&s_dt[j0]);
                 gd_bf16x4 vh, vl;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const uint32_t j = 32u * jb + 8u * (uint32_t)a + 4u * hh + (uint32_t)r;
-                    const float v = j <= i ? acc[4 * a + r] * expf(ci - s_cs[j]) * s_dt[j] : 0.f;
+                    const float v = j0 + (uint32_t)r <= i ? gm[4 * a + r] * __builtin_amdgcn_exp2f(ci - cj[r]) * dj[r] : 0.f;
                     gd_bf16 hi, lo;
                     gd_sc_split(v, &hi, &lo);
                     vh[r] = hi;
                     vl[r] = lo;
                 }
-                const uint32_t at = i * L::MS + (32u * jb + 8u * (uint32_t)a + 4u * hh) * 2u;
-                *reinterpret_cast<gd_bf16x4 *>(sm + L::mh + at) = vh;
-                *reinterpret_cast<gd_bf16x4 *>(sm + L::ml + at) = vl;
+                *reinterpret_cast<gd_bf16x4 *>(sm + L::mh + i * L::MS + j0 * 2u) = vh;
+                *reinterpret_cast<gd_bf16x4 *>(sm + L::ml + i * L::MS + j0 * 2u) = vl;
             }
         }
         __syncthreads();
-
-        /* Y^T tile: rows p (columns 32 * pb of the slice), columns i (row block ib): a lane holds one token */
         {
-            const uint32_t pb = wave & 1u, i = 32u * ib + lc;
-            gd_float16 ys, ym;
+            const float ei = __builtin_amdgcn_exp2f(ci);
 #pragma unroll
-            for (int e = 0; e < 16; ++e) ys[e] = ym[e] = 0.f;
-#pragma unroll
-            for (int ks = 0; ks < NP / 16; ++ks) { /* S^T C */
-                const uint32_t c = (16u * ks + 8u * hh) * 2u;
-                const gd_bf16x8 cv = *reinterpret_cast<const gd_bf16x8 *>(sm + L::c + i * L::BC + c);
-                const gd_bf16x8 ah = *reinterpret_cast<const gd_bf16x8 *>(sm + L::sh + (32u * pb + lc) * L::BC + c);
-                const gd_bf16x8 al = *reinterpret_cast<const gd_bf16x8 *>(sm + L::sl + (32u * pb + lc) * L::BC + c);
-                ys = GD_MFMA(ah, cv, ys);
-                ys = GD_MFMA(al, cv, ys);
-            }
+            for (int e = 0; e < 16; ++e) ys[e] *= ei;
 #pragma unroll
             for (int ks = 0; ks < 4; ++ks) { /* X^T M^T over j <= i: the second half only for the lower rows */
                 if (16u * ks >= 32u * (ib + 1u)) continue;
@@ -220,10 +218,9 @@ gd_ssm_scan_chunk_kernel(const gd_bf16 *__restrict__ xbc, const gd_bf16 *__restr
                 const gd_bf16x8 xv = gd_sc_turned(sm + L::x, L::XS, 16u * (uint32_t)ks, 32u * pb, lane);
                 const gd_bf16x8 mh = *reinterpret_cast<const gd_bf16x8 *>(sm + L::mh + i * L::MS + j);
                 const gd_bf16x8 ml = *reinterpret_cast<const gd_bf16x8 *>(sm + L::ml + i * L::MS + j);
-                ym = GD_MFMA(xv, mh, ym);
-                ym = GD_MFMA(xv, ml, ym);
+                ys = GD_MFMA(xv, mh, ys);
+                ys = GD_MFMA(xv, ml, ys);
             }
-            const float ei = expf(s_cs[i]);
             if (i < nt) {
                 gd_bf16 *yr = y + (size_t)(first + t0 + (int32_t)i) * inner + h * P + p0 + 32u * pb;
 #pragma unroll
@@ -233,34 +230,41 @@ gd_ssm_scan_chunk_kernel(const gd_bf16 *__restrict__ xbc, const gd_bf16 *__restr
                     const gd_bf16x4 xv = *reinterpret_cast<const gd_bf16x4 *>(sm + L::x + i * L::XS + (32u * pb + p) * 2u);
                     gd_bf16x4 o;
 #pragma unroll
-                    for (int r = 0; r < 4; ++r)
-                        o[r] = (gd_bf16)(ym[4 * a + r] + ei * ys[4 * a + r] + skip * (float)xv[r]);
+                    for (int r = 0; r < 4; ++r) o[r] = (gd_bf16)(ys[4 * a + r] + skip * (float)xv[r]);
                     *reinterpret_cast<gd_bf16x4 *>(yr + p) = o;
                 }
             }
         }
         /* state behind the chunk */
-        const float decay = expf(s_cs[GD_SC_L - 1u]);
+        const float decay = __builtin_amdgcn_exp2f(s_cs[GD_SC_L - 1u]);
+        constexpr int PB = TPW < 2 ? TPW : 2; /* tiles of one row block that lie with this wavefront */
 #pragma unroll
-        for (int t = 0; t < TPW; ++t) {
-            const uint32_t ti = wave * (uint32_t)TPW + (uint32_t)t, nb = ti / 2u, pb = ti % 2u;
-            if (ti >= (uint32_t)TILES) continue;
+        for (int t = 0; t < TPW; ++t)
 #pragma unroll
             for (int e = 0; e < 16; ++e) S[t][e] *= decay;
 #pragma unroll
+        for (int tb = 0; tb < TPW; tb += PB) {
+            const uint32_t ti = wave * (uint32_t)TPW + (uint32_t)tb, nb = ti / 2u;
+            if (ti >= (uint32_t)TILES) continue;
+#pragma unroll
             for (int ks = 0; ks < 4; ++ks) {
                 const gd_bf16x8 bv = gd_sc_turned(sm + L::b, L::BC, 16u * (uint32_t)ks, 32u * nb, lane);
-                const gd_bf16x8 xv = gd_sc_turned(sm + L::x, L::XS, 16u * (uint32_t)ks, 32u * pb, lane);
+                const gd_float4 w0 = *reinterpret_cast<const gd_float4 *>(&s_w[16 * ks + 8 * (int)hh]);
+                const gd_float4 w1 = *reinterpret_cast<const gd_float4 *>(&s_w[16 * ks + 8 * (int)hh + 4]);
                 gd_bf16x8 bh, bl;
 #pragma unroll
                 for (int e = 0; e < 8; ++e) {
                     gd_bf16 hi, lo;
-                    gd_sc_split((float)bv[e] * s_w[16 * ks + 8 * (int)hh + e], &hi, &lo);
+                    gd_sc_split((float)bv[e] * (e < 4 ? w0[e & 3] : w1[e & 3]), &hi, &lo);
                     bh[e] = hi;
                     bl[e] = lo;
                 }
-                S[t] = GD_MFMA(bh, xv, S[t]);
-                S[t] = GD_MFMA(bl, xv, S[t]);
+#pragma unroll
+                for (int u = 0; u < PB; ++u) {
+                    const gd_bf16x8 xv = gd_sc_turned(sm + L::x, L::XS, 16u * (uint32_t)ks, 32u * ((ti + (uint32_t)u) % 2u), lane);
+                    S[tb + u] = GD_MFMA(bh, xv, S[tb + u]);
+                    S[tb + u] = GD_MFMA(bl, xv, S[tb + u]);
+                }
             }
         }
     }
