@@ -197,6 +197,8 @@ _SIGNATURES = {
     "gd_backend_residual_norm_rows": [_vp, _TV, _TV, _TV, _TV, C.c_float],
     "gd_backend_causal_conv_silu": [_vp, _MV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs)],
     "gd_backend_ssm_scan": [_vp, _TV, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(SsmArgs)],
+    "gd_backend_conv_ssm_step": [_vp, _MV, _TV, _TV, _TV, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs),
+                                 C.POINTER(SsmArgs)],
     "gd_backend_gated_group_norm": [_vp, _TV, _MV, _TV, _TV, C.c_uint32, C.c_float],
     "gd_backend_latent_prepare": [_vp, _MV, _TV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(LatentArgs)],
     "gd_backend_latent_attend": [_vp, _TV, _TV, _TV, _MV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs),

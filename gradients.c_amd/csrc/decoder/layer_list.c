@@ -499,14 +499,18 @@ static gd_status mamba2(forward *f, const layer_config *l, layer_weights *w)
     tview(&w->conv, &taps);
     tview(&w->conv_b, &cb);
     tview(&w->ring, &ring);
-    view2(&f->a, f->type, f->rows, ch, &conv);
-    TRY(gd_backend_causal_conv_silu(f->be, &u, &taps, &cb, &ring, &conv, &f->seqs));
     tview(&w->dt_bias, &dtb);
     tview(&w->a_log, &al);
     tview(&w->d_skip, &dk);
     tview(&w->states, &st);
     view2(&f->b, f->type, f->rows, inner, &y);
-    TRY(gd_backend_ssm_scan(f->be, &conv, &dt, &dtb, &al, &dk, &st, &y, &f->seqs, &l->ssm));
+    if (f->seqs.max_new == 1U) {
+        TRY(gd_backend_conv_ssm_step(f->be, &u, &taps, &cb, &ring, &dt, &dtb, &al, &dk, &st, &y, &f->seqs, &l->ssm));
+    } else {
+        view2(&f->a, f->type, f->rows, ch, &conv);
+        TRY(gd_backend_causal_conv_silu(f->be, &u, &taps, &cb, &ring, &conv, &f->seqs));
+        TRY(gd_backend_ssm_scan(f->be, &conv, &dt, &dtb, &al, &dk, &st, &y, &f->seqs, &l->ssm));
+    }
     tview(&w->gnorm, &gn);
     view2(&f->a, f->type, f->rows, inner, &out);
     TRY(gd_backend_gated_group_norm(f->be, &y, &z, &gn, &out, (uint32_t)l->norm_groups, f->ll->c.eps));

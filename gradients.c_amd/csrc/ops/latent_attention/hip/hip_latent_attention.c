@@ -54,7 +54,7 @@ static bool params(const gd_backend_latent_args *a, gd_hip_latent_params *m)
 static bool decode_sizes(const gd_hip_latent_params *m, uint32_t dtype)
 {
     return dtype == GD_BACKEND_DTYPE_BF16 && (m->dim % 8u) == 0u && (m->rot_dim % 8u) == 0u && (m->kv_rank % 16u) == 0u &&
-           m->kv_rank <= 1024u && m->pitch <= 1088u;
+           m->pitch <= 1088u;
 }
 
 static bool prefill_sizes(const gd_hip_latent_params *m, uint32_t dtype)

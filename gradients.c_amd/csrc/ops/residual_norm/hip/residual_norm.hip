@@ -61,6 +61,17 @@ gd_residual_embed_kernel(const T *__restrict__ table, const int32_t *__restrict_
     const int32_t id = ids[blockIdx.x];
     const bool ok = id >= 0 && (uint32_t)id < vocab;
     const T *row = table + (size_t)(ok ? id : 0) * cols;
+    if (ok && copy != nullptr && (cols % 8u) == 0u && ((reinterpret_cast<uintptr_t>(table) | reinterpret_cast<uintptr_t>(copy)) & 15u) == 0u) {
+        for (uint32_t c = threadIdx.x * 8u; c < cols; c += GD_RN_THREADS * 8u) {
+            float v[8];
+            gd_rn_vec<T>::load(row + c, v);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] *= scale;
+            gd_rn_vec<float>::store(x + (size_t)blockIdx.x * cols + c, v);
+            gd_rn_vec<T>::store(copy + (size_t)blockIdx.x * cols + c, v);
+        }
+        return;
+    }
     for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS) {
         const float v = ok ? (float)row[c] * scale : __builtin_nanf("");
         x[(size_t)blockIdx.x * cols + c] = v;
@@ -77,13 +88,18 @@ gd_residual_norm_add_kernel(const T *__restrict__ u, const float *__restrict__ w
     const size_t base = (size_t)blockIdx.x * cols;
     float ss = 0.f;
     if (VEC) {
-        float uv[GD_RN_CHUNKS][8], xv[GD_RN_CHUNKS][8];
+        float uv[GD_RN_CHUNKS][8], xv[GD_RN_CHUNKS][8], wv[GD_RN_CHUNKS][8]; /* all requested in front of the sum */
 #pragma unroll
         for (int i = 0; i < GD_RN_CHUNKS; ++i) {
             const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
             if (c >= cols) continue;
             gd_rn_vec<T>::load(u + base + c, uv[i]);
             gd_rn_vec<float>::load(x + base + c, xv[i]);
+            gd_rn_vec<float>::load(w + c, wv[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+            if ((threadIdx.x + i * GD_RN_THREADS) * 8u >= cols) continue;
 #pragma unroll
             for (int e = 0; e < 8; ++e) ss = fmaf(uv[i][e], uv[i][e], ss);
         }
@@ -93,10 +109,8 @@ gd_residual_norm_add_kernel(const T *__restrict__ u, const float *__restrict__ w
         for (int i = 0; i < GD_RN_CHUNKS; ++i) {
             const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
             if (c >= cols) continue;
-            float wv[8];
-            gd_rn_vec<float>::load(w + c, wv);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) xv[i][e] += mult * (uv[i][e] * inv * wv[e]);
+            for (int e = 0; e < 8; ++e) xv[i][e] += mult * (uv[i][e] * inv * wv[i][e]);
             gd_rn_vec<float>::store(x + base + c, xv[i]);
             if (copy != nullptr) gd_rn_vec<T>::store(copy + base + c, xv[i]);
         }

@@ -20,11 +20,29 @@
 
 __device__ __forceinline__ float gd_softplus(float v) { return fmaxf(v, 0.0f) + log1pf(expf(-fabsf(v))); }
 
-template <typename T, int NR>
+/* silu of the causal convolution of channel c at position pos, rounded to T as the separate operator stores it; keep:
+ * this workgroup is the one that stores the channel's new input */
+template <typename T>
+__device__ __forceinline__ float gd_ssm_conv_at(const gd_hip_ssm_conv &cv, const T *__restrict__ u, T *__restrict__ rg,
+                                                uint32_t c, int32_t pos, bool keep)
+{
+    const float *w = cv.taps + (size_t)c * cv.K;
+    const T now = u[c];
+    float acc = fmaf(w[cv.K - 1u], (float)now, cv.bias[c]);
+    for (uint32_t k = 1u; k < cv.K && (int32_t)k <= pos; ++k)
+        acc = fmaf(w[cv.K - 1u - k], (float)rg[(size_t)((uint32_t)(pos - (int32_t)k) % cv.K) * cv.C + c], acc);
+    if (keep) rg[(size_t)((uint32_t)pos % cv.K) * cv.C + c] = now;
+    return (float)(T)gd_silu_f32(acc);
+}
+
+/* CONV: xbc holds the inputs of the convolution (row pitch ld_xbc) and every sequence brings one token: the channels a
+ * workgroup needs are convolved here.  B and C are convolved by every workgroup of their group; the places of the
+ * ring that are read (positions in front of the token) and written (its own) differ, so they do not race. */
+template <typename T, int NR, bool CONV>
 __global__ void __launch_bounds__(256)
 gd_ssm_scan_kernel(const T *__restrict__ xbc, const T *__restrict__ dt_raw, const float *__restrict__ dt_bias,
                    const float *__restrict__ a_log, const float *__restrict__ d_skip, float *__restrict__ states,
-                   T *__restrict__ y, gd_hip_ssm_params m, gd_hip_seqs q)
+                   T *__restrict__ y, gd_hip_ssm_params m, gd_hip_ssm_conv cv, gd_hip_seqs q)
 {
     __shared__ float sb[GD_SSM_BATCH][NR * 32], sc[GD_SSM_BATCH][NR * 32], sx[GD_SSM_BATCH][GD_SSM_COLS];
     __shared__ float part[GD_SSM_BATCH][4][GD_SSM_COLS], sdt[GD_SSM_BATCH], sdec[GD_SSM_BATCH];
@@ -51,6 +69,20 @@ gd_ssm_scan_kernel(const T *__restrict__ xbc, const T *__restrict__ dt_raw, cons
     for (int32_t t0 = 0; t0 < n; t0 += GD_SSM_BATCH) {
         const uint32_t nb = min((uint32_t)(n - t0), (uint32_t)GD_SSM_BATCH);
         const T *rows = xbc + (size_t)(first + t0) * m.ld_xbc;
+        if (CONV) {
+            T *rg = (T *)cv.ring + (size_t)slot * cv.K * cv.C;
+            const bool own = blockIdx.x == 0u && h % (m.heads / m.groups) == 0u; /* of B and C of the group */
+            for (uint32_t i = threadIdx.x; i < 2u * NR * 32u + GD_SSM_COLS; i += 256u) {
+                const uint32_t k = i % (NR * 32u), part = i / (NR * 32u);
+                if (part < 2u) {
+                    float *dst = part == 0u ? &sb[0][k] : &sc[0][k];
+                    *dst = k < N ? gd_ssm_conv_at<T>(cv, rows, rg, inner + (part * m.groups + g) * N + k, start, own) : 0.f;
+                } else {
+                    const uint32_t c = i - 2u * NR * 32u;
+                    sx[0][c] = c < cols ? gd_ssm_conv_at<T>(cv, rows, rg, h * P + p0 + c, start, true) : 0.f;
+                }
+            }
+        } else {
         for (uint32_t i = threadIdx.x; i < nb * (NR * 32u); i += 256u) {
             const uint32_t t = i / (NR * 32u), k = i % (NR * 32u);
             const T *b = rows + (size_t)t * m.ld_xbc + inner + g * N;
@@ -60,6 +92,7 @@ gd_ssm_scan_kernel(const T *__restrict__ xbc, const T *__restrict__ dt_raw, cons
         for (uint32_t i = threadIdx.x; i < nb * GD_SSM_COLS; i += 256u) {
             const uint32_t t = i / GD_SSM_COLS, c = i % GD_SSM_COLS;
             sx[t][c] = c < cols ? (float)rows[(size_t)t * m.ld_xbc + h * P + p0 + c] : 0.f;
+        }
         }
         if (threadIdx.x < nb) {
             const float dt = gd_softplus((float)dt_raw[(size_t)(first + t0 + (int32_t)threadIdx.x) * m.ld_dt + h] + bias);
@@ -110,21 +143,27 @@ gd_ssm_scan_kernel(const T *__restrict__ xbc, const T *__restrict__ dt_raw, cons
 
 extern "C" int gd_hip_launch_ssm_scan(hipStream_t stream, const void *xbc, const void *dt_raw, const float *dt_bias,
                                       const float *a_log, const float *d_skip, float *states, void *y,
-                                      const gd_hip_ssm_params *m, const gd_hip_seqs *q, int is_f32)
+                                      const gd_hip_ssm_params *m, const gd_hip_ssm_conv *cv, const gd_hip_seqs *q,
+                                      int is_f32)
 {
     const dim3 grid((m->vdim + GD_SSM_COLS - 1u) / GD_SSM_COLS, m->heads, q->seqs);
     if (q->rows == 0u || q->seqs == 0u) return (int)hipSuccess;
     if (m->state > GD_SSM_STATE_MAX) return (int)hipErrorInvalidValue;
-#define GD_GO(T, NR) gd_ssm_scan_kernel<T, NR><<<grid, 256, 0, stream>>>((const T *)xbc, (const T *)dt_raw, dt_bias, a_log, d_skip, states, (T *)y, *m, *q)
-#define GD_PICK(T)                          \
-    do {                                    \
-        if (m->state <= 32u) GD_GO(T, 1);   \
-        else if (m->state <= 64u) GD_GO(T, 2);  \
-        else if (m->state <= 128u) GD_GO(T, 4); \
-        else if (m->state <= 256u) GD_GO(T, 8); \
-        else GD_GO(T, 16);                  \
+    const gd_hip_ssm_conv none = {nullptr, nullptr, nullptr, 0u, 0u};
+#define GD_GO(T, NR, CONV) gd_ssm_scan_kernel<T, NR, CONV><<<grid, 256, 0, stream>>>((const T *)xbc, (const T *)dt_raw, dt_bias, a_log, d_skip, states, (T *)y, *m, CONV ? *cv : none, *q)
+#define GD_PICK(T, CONV)                              \
+    do {                                              \
+        if (m->state <= 32u) GD_GO(T, 1, CONV);       \
+        else if (m->state <= 64u) GD_GO(T, 2, CONV);  \
+        else if (m->state <= 128u) GD_GO(T, 4, CONV); \
+        else if (m->state <= 256u) GD_GO(T, 8, CONV); \
+        else GD_GO(T, 16, CONV);                      \
     } while (0)
-    if (is_f32) GD_PICK(float); else GD_PICK(gd_bf16);
+    if (cv != nullptr) {
+        if (is_f32) GD_PICK(float, true); else GD_PICK(gd_bf16, true);
+    } else {
+        if (is_f32) GD_PICK(float, false); else GD_PICK(gd_bf16, false);
+    }
 #undef GD_PICK
 #undef GD_GO
     return (int)hipGetLastError();
@@ -174,6 +213,7 @@ gd_gated_group_norm_vec_kernel(const gd_bf16 *__restrict__ y, const gd_bf16 *__r
     const gd_bf16 *yr = y + (size_t)blockIdx.x * inner + c0, *zr = z + (size_t)blockIdx.x * ldz + c0;
     constexpr int KEEP = 4;
     gd_bf16x8 yv[KEEP], zv[KEEP];
+    gd_float4 wv[KEEP][2]; /* requested with the rest: behind the sum they would be one more round trip */
     float v[KEEP][8], ss = 0.f;
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
@@ -181,6 +221,8 @@ gd_gated_group_norm_vec_kernel(const gd_bf16 *__restrict__ y, const gd_bf16 *__r
         if (c >= part) continue;
         yv[i] = *reinterpret_cast<const gd_bf16x8 *>(yr + c);
         zv[i] = *reinterpret_cast<const gd_bf16x8 *>(zr + c);
+        wv[i][0] = *reinterpret_cast<const gd_float4 *>(w + c0 + c);
+        wv[i][1] = *reinterpret_cast<const gd_float4 *>(w + c0 + c + 4u);
     }
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
@@ -199,7 +241,7 @@ gd_gated_group_norm_vec_kernel(const gd_bf16 *__restrict__ y, const gd_bf16 *__r
         if (c >= part) continue;
         gd_bf16x8 o;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = (gd_bf16)(v[i][e] * inv * w[c0 + c + e]);
+        for (int e = 0; e < 8; ++e) o[e] = (gd_bf16)(v[i][e] * inv * wv[i][e >> 2][e & 3]);
         *reinterpret_cast<gd_bf16x8 *>(out + (size_t)blockIdx.x * inner + c0 + c) = o;
     }
 }

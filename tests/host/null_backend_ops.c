@@ -16,6 +16,7 @@ GD_NULL_OP(gd_backend_argmax_advance)
 GD_NULL_OP(gd_backend_argmax_rows)
 GD_NULL_OP(gd_backend_causal_conv_silu)
 GD_NULL_OP(gd_backend_concat_to_full)
+GD_NULL_OP(gd_backend_conv_ssm_step)
 GD_NULL_OP(gd_backend_decode_advance)
 GD_NULL_OP(gd_backend_embedding_forward)
 GD_NULL_OP(gd_backend_fused_linear)

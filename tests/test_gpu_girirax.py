@@ -267,6 +267,35 @@ def test_recurrence_carries_one_early_token_through_chunks(backend, gda, arena, 
 
 
 @TYPES
+@pytest.mark.parametrize("H,P,N,Gn,K", [(4, 16, 16, 2, 4), (3, 20, 40, 3, 3), (2, 64, 128, 1, 4), (5, 7, 9, 5, 1), (2, 40, 300, 1, 7)])
+def test_fused_convolution_and_recurrence_step(backend, gda, arena, dtype, H, P, N, Gn, K):
+    """One launch of a decode step against the two operators: same results, rings and states, from the first token on."""
+    rng = np.random.default_rng(N)
+    ch, B = H * P + 2 * Gn * N, 3
+    small = [_put(arena, F32, v)[0] for v in (rng.uniform(-3, -1, H), rng.uniform(-1, 1, H), rng.standard_normal(H))]
+    taps, bias = _put(arena, F32, rng.standard_normal((ch, K)) * 0.5)[0], _put(arena, F32, rng.standard_normal(ch) * 0.1)[0]
+    args = gda.SsmArgs(H, P, N, Gn)
+    junk = rng.standard_normal((4, K, ch)) * 9, rng.standard_normal((4, H, N, P)) * 9
+    sides = [(_put(arena, dtype, junk[0])[0], _put(arena, F32, junk[1])[0], arena.alloc((B, H * P), dtype)) for _ in range(2)]
+    conv = arena.alloc((B, ch), dtype)
+    for t in range(6):
+        start = [t, t + 1 if t else 0, 0]
+        sq = Seqs(gda, arena, [(2, start[0], 1), (0, t, 1), (3, start[2], 1)])
+        x = _put(arena, dtype, rng.standard_normal((B, ch + H)))[0]
+        xm, dt = x.matrix(cols=ch), x.matrix(cols=H)
+        dt.offset += ch * x.itemsize
+        rest = [v.view() for v in small]
+        ring, st, y = sides[0]
+        _ok(backend.call("gd_backend_causal_conv_silu", xm, taps.view(), bias.view(), ring.view(), conv.view(), sq.ref()))
+        _ok(backend.call("gd_backend_ssm_scan", conv.view(), dt, *rest, st.view(), y.view(), sq.ref(), C.byref(args)))
+        ring, st, y = sides[1]
+        _ok(backend.call("gd_backend_conv_ssm_step", xm, taps.view(), bias.view(), ring.view(), dt, *rest, st.view(), y.view(),
+                         sq.ref(), C.byref(args)))
+        for a, b in zip(*sides):
+            _near(a.read_float(), b.read_float(), dtype)
+
+
+@TYPES
 @pytest.mark.parametrize("inner,parts", [(64, 1), (96, 4), (4096, 2), (30, 3), (5000, 1)])
 def test_gate_then_group_norm(backend, gda, arena, L, dtype, inner, parts):
     rng = np.random.default_rng(inner)
