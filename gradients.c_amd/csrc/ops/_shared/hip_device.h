@@ -60,6 +60,12 @@ __device__ __forceinline__ float gd_sigmoid_f32(float z)
     const float e = __expf(-fabsf(z)), inv = 1.0f / (1.0f + e);
     return z >= 0.0f ? inv : e * inv;
 }
+/* for results that are rounded to 16 bits: the reciprocal instruction instead of a division */
+__device__ __forceinline__ float gd_sigmoid_fast(float z)
+{
+    const float e = __expf(-fabsf(z)), inv = __builtin_amdgcn_rcpf(1.0f + e);
+    return z >= 0.0f ? inv : e * inv;
+}
 __device__ __forceinline__ float gd_silu_f32(float z) { return z * gd_sigmoid_f32(z); }
 /* 0.5 z (1 + tanh(u)) = z sigmoid(2 u) with u = sqrt(2/pi) (z + 0.044715 z^3) */
 __device__ __forceinline__ float gd_gelu_tanh_f32(float z)

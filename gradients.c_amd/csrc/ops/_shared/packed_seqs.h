@@ -18,6 +18,13 @@ typedef struct gd_hip_seqs {
 __device__ __forceinline__ bool gd_seq_of_row(const gd_hip_seqs &q, uint32_t row, int32_t *seq, int32_t *pos,
                                               int32_t *slot)
 {
+    if (q.max_new == 1u && q.rows == q.seqs) { /* one row each, in order: one round trip to memory less */
+        const int32_t st = q.start[row], sl = q.slot[row];
+        *seq = (int32_t)row;
+        *slot = sl;
+        *pos = st;
+        return st >= 0 && sl >= 0 && (uint32_t)sl < q.slots;
+    }
     const int32_t s = q.row_seq[row];
     if (s < 0 || (uint32_t)s >= q.seqs) return false;
     const int32_t st = q.start[s], sl = q.slot[s], first = q.cu[s];

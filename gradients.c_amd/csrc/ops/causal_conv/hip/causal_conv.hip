@@ -82,7 +82,7 @@ gd_causal_conv_silu_vec_kernel(const gd_bf16 *__restrict__ u, uint32_t ldu, cons
             float acc = fmaf(taps[K - 1][e], (float)win[0][e], b[e]);
 #pragma unroll
             for (int k = 1; k < K; ++k) acc = fmaf(taps[K - 1 - k][e], (float)win[k][e], acc);
-            o[e] = (gd_bf16)gd_silu_f32(acc);
+            o[e] = (gd_bf16)(acc * gd_sigmoid_fast(acc));
         }
         *reinterpret_cast<gd_bf16x8 *>(out + (size_t)row * C + c) = o;
         if (store_ring) *reinterpret_cast<gd_bf16x8 *>(rg + (size_t)((uint32_t)pos % K) * C) = win[0];

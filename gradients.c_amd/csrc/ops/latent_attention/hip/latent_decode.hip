@@ -155,12 +155,15 @@ gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__re
     typedef short gd_short4 __attribute__((ext_vector_type(4)));
 
     issue(k_begin, 0u);
+    if (k_begin + GD_LD_TILE < k_end) issue(k_begin + GD_LD_TILE, 1u);
     uint32_t it = 0u;
     for (uint32_t k0 = k_begin; k0 < k_end; k0 += GD_LD_TILE, ++it) {
         const unsigned char *tile = gd_ld_smem + (it & 1u) * STAGE;
-        __builtin_amdgcn_s_waitcnt(0x0F70); /* vmcnt(0): this wavefront's share of the tile is in LDS */
-        __syncthreads();                    /* everyone's share is, and the other stage is no longer read */
-        if (k0 + GD_LD_TILE < k_end) issue(k0 + GD_LD_TILE, (it + 1u) & 1u);
+        /* this wavefront's share of the tile is in LDS; the second tile was requested with the first */
+        if (it == 0u && k0 + GD_LD_TILE < k_end) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(NL) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads(); /* everyone's share is, and the other stage is no longer read */
+        if (it != 0u && k0 + GD_LD_TILE < k_end) issue(k0 + GD_LD_TILE, (it + 1u) & 1u);
         gd_float4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int s = 0; s < HS; ++s) {

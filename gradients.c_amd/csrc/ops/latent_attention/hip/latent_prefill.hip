@@ -282,7 +282,7 @@ gd_latent_prefill_kernel(const gd_bf16 *__restrict__ q_rows, const gd_bf16 *__re
                     for (int r = 0; r < 4; ++r) gv[r] = gr[c + (uint32_t)r];
             }
 #pragma unroll
-            for (int r = 0; r < 4; ++r) hv[r] = (gd_bf16)(o[dt][4 * a + r] * inv * gd_sigmoid_f32((float)gv[r]));
+            for (int r = 0; r < 4; ++r) hv[r] = (gd_bf16)(o[dt][4 * a + r] * inv * gd_sigmoid_fast((float)gv[r]));
             *reinterpret_cast<gd_bf16x4 *>(sO + lq * OS + c) = hv;
         }
     }

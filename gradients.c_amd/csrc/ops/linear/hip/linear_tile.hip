@@ -925,7 +925,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
 }
 
 template <int WM, int WN, bool W_NK, int PRO>
-static int launch_tile_one(hipStream_t stream, const gd_elem *x, const gd_elem *w, const gd_elem *bias,
+int gd_linear_tile_launch_one(hipStream_t stream, const gd_elem *x, const gd_elem *w, const gd_elem *bias,
                            const gd_elem *residual, const gd_elem *norm_w, gd_elem *y, const gd_hip_linear_params &p,
                            uint32_t vector_store, uint32_t workgroups)
 {
@@ -948,12 +948,39 @@ static int launch_tile_one(hipStream_t stream, const gd_elem *x, const gd_elem *
     return (int)hipGetLastError();
 }
 
+/* The F16 instantiations take minutes to compile; they are spread over translation units of their own
+ * (linear_tile_part*.hip define GD_LINEAR_TILE_PART and include this file) and only declared here. */
+#define GD_TILE_FORM(WORD, WM, WN, NK, PRO)                                                                              \
+    WORD template int gd_linear_tile_launch_one<WM, WN, NK, PRO>(hipStream_t, const gd_elem *, const gd_elem *,          \
+                                                                 const gd_elem *, const gd_elem *, const gd_elem *,      \
+                                                                 gd_elem *, const gd_hip_linear_params &, uint32_t, uint32_t);
+#define GD_TILE_PROLOGUES(WORD, WM, WN, NK)            \
+    GD_TILE_FORM(WORD, WM, WN, NK, GD_HIP_PRO_NONE)    \
+    GD_TILE_FORM(WORD, WM, WN, NK, GD_HIP_PRO_SWIGLU)  \
+    GD_TILE_FORM(WORD, WM, WN, NK, GD_HIP_PRO_RMS_NORM)
+#if defined(GD_LINEAR_TILE_PART) && GD_LINEAR_TILE_PART == 1
+GD_TILE_PROLOGUES(, 4, 4, true)
+#elif defined(GD_LINEAR_TILE_PART) && GD_LINEAR_TILE_PART == 2
+GD_TILE_PROLOGUES(, 4, 4, false)
+#elif defined(GD_LINEAR_TILE_PART) && GD_LINEAR_TILE_PART == 3
+GD_TILE_PROLOGUES(, 2, 2, true)
+GD_TILE_PROLOGUES(, 2, 2, false)
+GD_TILE_FORM(, 3, 4, true, GD_HIP_PRO_NONE)
+#else
+#if !GD_LINEAR_IS_BF16
+GD_TILE_PROLOGUES(extern, 4, 4, true)
+GD_TILE_PROLOGUES(extern, 4, 4, false)
+GD_TILE_PROLOGUES(extern, 2, 2, true)
+GD_TILE_PROLOGUES(extern, 2, 2, false)
+GD_TILE_FORM(extern, 3, 4, true, GD_HIP_PRO_NONE)
+#endif
+
 template <int WM, int WN>
 static int launch_tile(hipStream_t stream, const gd_elem *x, const gd_elem *w, const gd_elem *bias,
                        const gd_elem *residual, const gd_elem *norm_w, gd_elem *y, const gd_hip_linear_params &p,
                        uint32_t vector_store, uint32_t workgroups)
 {
-#define GD_GO(NK, PRO) return launch_tile_one<WM, WN, NK, PRO>(stream, x, w, bias, residual, norm_w, y, p, vector_store, workgroups)
+#define GD_GO(NK, PRO) return gd_linear_tile_launch_one<WM, WN, NK, PRO>(stream, x, w, bias, residual, norm_w, y, p, vector_store, workgroups)
 #if GD_LINEAR_IS_BF16
     GD_GO(true, GD_HIP_PRO_NONE);
 #else
@@ -1022,7 +1049,7 @@ extern "C" int GD_LINEAR_FN(gd_hip_launch_linear_tile)(hipStream_t stream, const
                 if (mid_tiles) {
                     const uint32_t first = p.M - mid_rows;
                     tail.M = mid_rows;
-                    return launch_tile_one<3, 4, true, GD_HIP_PRO_NONE>(
+                    return gd_linear_tile_launch_one<3, 4, true, GD_HIP_PRO_NONE>(
                         stream, xp + (size_t)first * p.ldx, (const gd_elem *)w, (const gd_elem *)bias,
                         rp != nullptr ? rp + (size_t)first * p.ldr : nullptr, (const gd_elem *)norm_w,
                         yp + (size_t)first * p.ldy, tail, (uint32_t)vector_store, units);
@@ -1095,3 +1122,4 @@ extern "C" uint32_t GD_LINEAR_FN(gd_hip_linear_tile_rope_head_rows)(uint32_t M, 
     return head_m * 256u;
 }
 #endif
+#endif /* GD_LINEAR_TILE_PART */

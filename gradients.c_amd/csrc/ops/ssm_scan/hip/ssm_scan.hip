@@ -29,6 +29,17 @@ __device__ __forceinline__ float gd_ssm_conv_at(const gd_hip_ssm_conv &cv, const
     const float *w = cv.taps + (size_t)c * cv.K;
     const T now = u[c];
     float acc = fmaf(w[cv.K - 1u], (float)now, cv.bias[c]);
+    if (cv.K <= 4u) { /* the places of the ring in one batch of loads */
+        float v[4], wv[4];
+#pragma unroll
+        for (uint32_t k = 1u; k < 4u; ++k) {
+            const bool ok = k < cv.K && (int32_t)k <= pos;
+            v[k] = ok ? (float)rg[(size_t)((uint32_t)(pos - (int32_t)k) % cv.K) * cv.C + c] : 0.f;
+            wv[k] = ok ? w[cv.K - 1u - k] : 0.f;
+        }
+#pragma unroll
+        for (uint32_t k = 1u; k < 4u; ++k) acc = fmaf(wv[k], v[k], acc);
+    } else
     for (uint32_t k = 1u; k < cv.K && (int32_t)k <= pos; ++k)
         acc = fmaf(w[cv.K - 1u - k], (float)rg[(size_t)((uint32_t)(pos - (int32_t)k) % cv.K) * cv.C + c], acc);
     if (keep) rg[(size_t)((uint32_t)pos % cv.K) * cv.C + c] = now;
@@ -229,7 +240,7 @@ gd_gated_group_norm_vec_kernel(const gd_bf16 *__restrict__ y, const gd_bf16 *__r
         if ((threadIdx.x + 256u * i) * 8u >= part) continue;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-            v[i][e] = (float)yv[i][e] * gd_silu_f32((float)zv[i][e]);
+            v[i][e] = (float)yv[i][e] * (float)zv[i][e] * gd_sigmoid_fast((float)zv[i][e]);
             ss = fmaf(v[i][e], v[i][e], ss);
         }
     }
