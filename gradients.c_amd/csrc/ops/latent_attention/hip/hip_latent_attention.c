@@ -63,11 +63,11 @@ static bool prefill_sizes(const gd_hip_latent_params *m, uint32_t dtype)
            (m->kv_rank % 8u) == 0u && m->dim + m->rot_dim <= 256u && m->vdim <= 128u;
 }
 
-/* keys per piece of the decode form: two workgroups per compute unit over the longest sequences, whole tiles of 64,
+/* keys per piece of the decode form: two workgroups (of up to 32 heads) per compute unit over the longest sequences, whole tiles of 64,
  * pieces of at least 128 keys */
 static void cut(gd_hip_latent_params *m, uint32_t rows, uint32_t units)
 {
-    const uint64_t groups = (uint64_t)rows * ((m->heads + 15u) / 16u);
+    const uint64_t groups = (uint64_t)rows * ((m->pitch > 576u ? (m->heads + 15u) / 16u : (m->heads + 31u) / 32u));
     uint64_t want = (2u * (uint64_t)units + groups - 1u) / groups, len;
     if (want > GD_HIP_LATENT_PIECES_MAX) want = GD_HIP_LATENT_PIECES_MAX;
     len = ((m->tmax + want - 1u) / want + 63u) & ~63ull;

@@ -3,7 +3,7 @@
  * heads of a token share one "key", the cache row, and one "value", its latent part.
  *
  *   absorb  q_lat[h] = W_uk[h]^T q[h] per 16 rows, head and 64 latent columns, and the rotated query part behind it
- *   attend  a workgroup of 4 wavefronts takes 16 heads of one token over a piece of its keys: a cache row is read from
+ *   attend  a workgroup of 4 wavefronts takes 16 or 32 heads of one token over a piece of its keys: a cache row is read from
  *           memory once for all of them.  HBM-bound on the cache rows.
  *   merge   the pieces of a token and head into one latent vector
  *   value   16 tokens and one head: the value up-projection and the output gate
@@ -93,9 +93,10 @@ __device__ __forceinline__ uint32_t gd_ld_swizzle(uint32_t r)
     return ((r & 2u) << 1) | ((r & 4u) >> 1) | ((r & 8u) >> 3);
 }
 
-/* STEPS: 32-wide steps that cover a cache row (pitch <= 32 * STEPS, STEPS even).  grid (pieces, ceil(heads / 16), rows).
+/* STEPS: 32-wide steps that cover a cache row (pitch <= 32 * STEPS, STEPS even); HG: groups of 16 heads per workgroup,
+ * which share every fragment read from LDS.  grid (pieces, ceil(heads / (16 * HG)), rows).
  * o_part F32 [rows, pieces, heads, kv_rank], ml F32 [rows, pieces, heads, 2] (reference point in the exp2 domain, sum) */
-template <int STEPS>
+template <int STEPS, int HG>
 __global__ void __launch_bounds__(256, STEPS <= 18 ? 2 : 1)
 gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__restrict__ cache, float *__restrict__ o_part,
                              float *__restrict__ ml, gd_hip_latent_params m, gd_hip_seqs q)
@@ -104,10 +105,10 @@ gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__re
     constexpr int NL = STEPS / 2, HS = STEPS / 2; /* wavefront loads per tile; steps of a wavefront's half */
     constexpr int CT = (2 * STEPS + 3) / 4;       /* 16-wide latent column tiles per wavefront */
     extern __shared__ __align__(16) unsigned char gd_ld_smem[]; /* [2][32] key rows */
-    __shared__ __align__(16) float s_part[4][64][4];
+    __shared__ __align__(16) float s_part[HG][4][64][4];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, li = lane & 15u, lg = lane >> 4;
     const uint32_t wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const uint32_t row = blockIdx.z, h0 = blockIdx.y * 16u, kg = wave & 1u, hf = wave >> 1;
+    const uint32_t row = blockIdx.z, h0 = blockIdx.y * (16u * HG), kg = wave & 1u, hf = wave >> 1;
     int32_t seq, pos, slot;
     if (!gd_seq_of_row(q, row, &seq, &pos, &slot)) return;
     const uint32_t keys = min((uint32_t)pos + 1u, m.tmax);
@@ -132,22 +133,27 @@ gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__re
             gd_ld_load_lds16(rows + (size_t)min(k0 + ld_row[t], k_end - 1u) * m.pitch + ld_off[t],
                              lds_base + stage * STAGE + (wave * (uint32_t)NL + (uint32_t)t) * 1024u);
     };
-    /* query fragments of head h0 + li, this wavefront's half of the row: loads the kernel does not wait for below with
-     * the tiles', so they come first */
-    gd_bf16x8 qf[HS];
+    /* query fragments of heads h0 + 16 n + li, this wavefront's half of the row */
+    gd_bf16x8 qf[HG][HS];
     const gd_bf16x8 zero = (gd_bf16x8)(gd_bf16)0.f;
-    {
-        const gd_bf16 *qr = ql + ((size_t)row * m.heads + min(h0 + li, m.heads - 1u)) * m.pitch;
+#pragma unroll
+    for (int n = 0; n < HG; ++n) {
+        const gd_bf16 *qr = ql + ((size_t)row * m.heads + min(h0 + 16u * (uint32_t)n + li, m.heads - 1u)) * m.pitch;
 #pragma unroll
         for (int s = 0; s < HS; ++s) {
             const uint32_t c = 4u * (hf * (uint32_t)HS + (uint32_t)s) + lg;
-            qf[s] = c < chunks ? *reinterpret_cast<const gd_bf16x8 *>(qr + c * 8u) : zero;
+            qf[n][s] = c < chunks ? *reinterpret_cast<const gd_bf16x8 *>(qr + c * 8u) : zero;
         }
     }
-    gd_float4 o[CT];
+    gd_float4 o[HG][CT];
+    float mref[HG], sum[HG]; /* of head h0 + 16 n + li; sum: the keys of this lane group */
 #pragma unroll
-    for (int t = 0; t < CT; ++t) o[t] = (gd_float4){0.f, 0.f, 0.f, 0.f};
-    float mref = -INFINITY, sum = 0.f; /* of head h0 + li; sum: the keys of this lane group */
+    for (int n = 0; n < HG; ++n) {
+        mref[n] = -INFINITY;
+        sum[n] = 0.f;
+#pragma unroll
+        for (int t = 0; t < CT; ++t) o[n][t] = (gd_float4){0.f, 0.f, 0.f, 0.f};
+    }
     const float scale2 = m.scale * 1.4426950408889634f;
     const uint32_t k_row = 16u * kg + li, k_swz = gd_ld_swizzle(k_row);
     const uint32_t tr_q = lane & 3u, tr_e = (lane >> 2) & 3u, v_row = 4u * lg + tr_e;
@@ -164,49 +170,53 @@ gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__re
         else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads(); /* everyone's share is, and the other stage is no longer read */
         if (it != 0u && k0 + GD_LD_TILE < k_end) issue(k0 + GD_LD_TILE, (it + 1u) & 1u);
-        gd_float4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+        gd_float4 sp[HG];
+#pragma unroll
+        for (int n = 0; n < HG; ++n) sp[n] = (gd_float4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int s = 0; s < HS; ++s) {
             const uint32_t c = 4u * (hf * (uint32_t)HS + (uint32_t)s) + lg;
             const gd_bf16x8 a = *reinterpret_cast<const gd_bf16x8 *>(tile + k_row * ROW + (c ^ k_swz) * 16u);
-            if (s & 1) s1 = GD_MFMA(a, qf[s], s1);
-            else s0 = GD_MFMA(a, qf[s], s0);
+#pragma unroll
+            for (int n = 0; n < HG; ++n) sp[n] = GD_MFMA(a, qf[n][s], sp[n]);
         }
 #pragma unroll
-        for (int r = 0; r < 4; ++r) s0[r] += s1[r];
-        *reinterpret_cast<gd_float4 *>(&s_part[wave][lane][0]) = s0;
+        for (int n = 0; n < HG; ++n) *reinterpret_cast<gd_float4 *>(&s_part[n][wave][lane][0]) = sp[n];
         __syncthreads();
-        float sc[8], mx = -INFINITY; /* keys 4 lg + r and 16 + 4 lg + r */
+        gd_bf16x8 ph[HG], pl[HG];
 #pragma unroll
-        for (int g = 0; g < 2; ++g) {
-            const gd_float4 a = *reinterpret_cast<const gd_float4 *>(&s_part[g][lane][0]);
-            const gd_float4 b = *reinterpret_cast<const gd_float4 *>(&s_part[2 + g][lane][0]);
+        for (int n = 0; n < HG; ++n) {
+            float sc[8], mx = -INFINITY; /* keys 4 lg + r and 16 + 4 lg + r */
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const uint32_t key = k0 + 16u * (uint32_t)g + 4u * lg + (uint32_t)r;
-                sc[4 * g + r] = key < k_end ? (a[r] + b[r]) * scale2 : -INFINITY;
-                mx = fmaxf(mx, sc[4 * g + r]);
+            for (int g = 0; g < 2; ++g) {
+                const gd_float4 a = *reinterpret_cast<const gd_float4 *>(&s_part[n][g][lane][0]);
+                const gd_float4 b = *reinterpret_cast<const gd_float4 *>(&s_part[n][2 + g][lane][0]);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const uint32_t key = k0 + 16u * (uint32_t)g + 4u * lg + (uint32_t)r;
+                    sc[4 * g + r] = key < k_end ? (a[r] + b[r]) * scale2 : -INFINITY;
+                    mx = fmaxf(mx, sc[4 * g + r]);
+                }
             }
-        }
-        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-        /* the tile holds at least one live key, so mx is finite (or NaN) */
-        if (__builtin_amdgcn_ballot_w64(!(mx <= mref + 8.f)) != 0ull) {
-            const float next = fmaxf(mref, mx), keep = __builtin_amdgcn_exp2f(mref - next);
-            mref = next;
-            sum *= keep;
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            /* the tile holds at least one live key, so mx is finite (or NaN) */
+            if (__builtin_amdgcn_ballot_w64(!(mx <= mref[n] + 8.f)) != 0ull) {
+                const float next = fmaxf(mref[n], mx), keep = __builtin_amdgcn_exp2f(mref[n] - next);
+                mref[n] = next;
+                sum[n] *= keep;
 #pragma unroll
-            for (int t = 0; t < CT; ++t)
+                for (int t = 0; t < CT; ++t)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) o[t][r] *= keep;
-        }
-        gd_bf16x8 ph, pl;
+                    for (int r = 0; r < 4; ++r) o[n][t][r] *= keep;
+            }
 #pragma unroll
-        for (int r = 0; r < 8; ++r) {
-            const float p = __builtin_amdgcn_exp2f(sc[r] - mref);
-            sum += p;
-            ph[r] = (gd_bf16)p;
-            pl[r] = (gd_bf16)(p - (float)ph[r]);
+            for (int r = 0; r < 8; ++r) {
+                const float p = __builtin_amdgcn_exp2f(sc[r] - mref[n]);
+                sum[n] += p;
+                ph[n][r] = (gd_bf16)p;
+                pl[n][r] = (gd_bf16)(p - (float)ph[n][r]);
+            }
         }
 #pragma unroll
         for (int t = 0; t < CT; ++t) {
@@ -218,23 +228,29 @@ gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__re
                 tile + v_row * ROW + (c ^ v_swz0) * 16u + w8));
             u.s[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) gd_short4 *)(
                 tile + (16u + v_row) * ROW + (c ^ v_swz1) * 16u + w8));
-            o[t] = GD_MFMA(u.v, ph, o[t]);
-            o[t] = GD_MFMA(u.v, pl, o[t]);
+#pragma unroll
+            for (int n = 0; n < HG; ++n) {
+                o[n][t] = GD_MFMA(u.v, ph[n], o[n][t]);
+                o[n][t] = GD_MFMA(u.v, pl[n], o[n][t]);
+            }
         }
     }
-    sum += __shfl_xor(sum, 16, 64);
-    sum += __shfl_xor(sum, 32, 64);
-    const uint32_t h = h0 + li;
-    if (h >= m.heads) return;
-    const size_t part = ((size_t)row * m.pieces + blockIdx.x) * m.heads + h;
-    if (wave == 0u && lg == 0u) {
-        ml[part * 2u] = mref;
-        ml[part * 2u + 1u] = sum;
-    }
 #pragma unroll
-    for (int t = 0; t < CT; ++t) {
-        const uint32_t col = (wave * (uint32_t)CT + (uint32_t)t) * 16u + 4u * lg;
-        if (col < m.kv_rank) *reinterpret_cast<gd_float4 *>(o_part + part * m.kv_rank + col) = o[t];
+    for (int n = 0; n < HG; ++n) {
+        sum[n] += __shfl_xor(sum[n], 16, 64);
+        sum[n] += __shfl_xor(sum[n], 32, 64);
+        const uint32_t h = h0 + 16u * (uint32_t)n + li;
+        if (h >= m.heads) continue;
+        const size_t part = ((size_t)row * m.pieces + blockIdx.x) * m.heads + h;
+        if (wave == 0u && lg == 0u) {
+            ml[part * 2u] = mref[n];
+            ml[part * 2u + 1u] = sum[n];
+        }
+#pragma unroll
+        for (int t = 0; t < CT; ++t) {
+            const uint32_t col = (wave * (uint32_t)CT + (uint32_t)t) * 16u + 4u * lg;
+            if (col < m.kv_rank) *reinterpret_cast<gd_float4 *>(o_part + part * m.kv_rank + col) = o[n][t];
+        }
     }
 }
 
@@ -329,19 +345,19 @@ gd_latent_value_mfma_kernel(const gd_bf16 *__restrict__ merged, const gd_bf16 *_
     }
 }
 
-template <int STEPS>
+template <int STEPS, int HG>
 static int launch_attend(hipStream_t stream, const gd_bf16 *ql, const gd_bf16 *cache, float *o_part, float *ml,
                          const gd_hip_latent_params &m, const gd_hip_seqs &q)
 {
     constexpr size_t lds = (size_t)2u * GD_LD_TILE * STEPS * 64u;
     static bool configured = false;
     if (!configured && lds > 48u * 1024u) {
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(gd_latent_attend_mfma_kernel<STEPS>),
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(gd_latent_attend_mfma_kernel<STEPS, HG>),
                                                  hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return (int)e;
         configured = true;
     }
-    gd_latent_attend_mfma_kernel<STEPS><<<dim3(m.pieces, (m.heads + 15u) / 16u, q.rows), 256, lds, stream>>>(ql, cache, o_part, ml, m, q);
+    gd_latent_attend_mfma_kernel<STEPS, HG><<<dim3(m.pieces, (m.heads + 16u * HG - 1u) / (16u * HG), q.rows), 256, lds, stream>>>(ql, cache, o_part, ml, m, q);
     return (int)hipGetLastError();
 }
 
@@ -360,11 +376,13 @@ extern "C" int gd_hip_launch_latent_decode(hipStream_t stream, const void *qv, c
         (const gd_bf16 *)qv, (const gd_bf16 *)w_ukt, angles, (gd_bf16 *)ql, m, q.rows);
     e = (int)hipGetLastError();
     if (e != 0) return e;
-    if (steps <= 6u) e = launch_attend<6>(stream, qlp, cp, o_part, ml, m, q);
-    else if (steps <= 10u) e = launch_attend<10>(stream, qlp, cp, o_part, ml, m, q);
-    else if (steps <= 18u) e = launch_attend<18>(stream, qlp, cp, o_part, ml, m, q);
-    else if (steps <= 34u) e = launch_attend<34>(stream, qlp, cp, o_part, ml, m, q);
+#define GD_GO(S) e = m.heads > 16u ? launch_attend<S, 2>(stream, qlp, cp, o_part, ml, m, q) : launch_attend<S, 1>(stream, qlp, cp, o_part, ml, m, q)
+    if (steps <= 6u) GD_GO(6);
+    else if (steps <= 10u) GD_GO(10);
+    else if (steps <= 18u) GD_GO(18);
+    else if (steps <= 34u) e = launch_attend<34, 1>(stream, qlp, cp, o_part, ml, m, q);
     else return (int)hipErrorInvalidValue;
+#undef GD_GO
     if (e != 0) return e;
     /* the queries are used up: their place takes the merged latents (kv_rank <= pitch) */
     gd_latent_merge_kernel<<<dim3(q.rows, m.heads), 256, 0, stream>>>(o_part, ml, (gd_bf16 *)ql, m, q);

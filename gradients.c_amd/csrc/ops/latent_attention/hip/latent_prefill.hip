@@ -21,26 +21,37 @@
 
 #define GD_LP_NEG_INF (-__builtin_inff())
 
-/* cache rows [slot, 0 .. start + n) of every sequence, packed; a thread per 16-byte piece; kv_cu [seqs + 1] */
+/* cache rows [slot, 0 .. start + n) of every sequence, packed, 16 rows per workgroup; kv_cu [seqs + 1] */
 __global__ void __launch_bounds__(256)
 gd_latent_gather_kernel(const gd_bf16 *__restrict__ cache, const int32_t *__restrict__ kv_cu, gd_bf16 *__restrict__ packed,
                         uint32_t total, gd_hip_latent_params m, gd_hip_seqs q)
 {
-    const uint32_t chunks = m.pitch / 8u;
-    const uint64_t g = (uint64_t)blockIdx.x * 256u + threadIdx.x;
-    const uint32_t r = (uint32_t)(g / chunks), c = (uint32_t)(g % chunks);
-    if (r >= total) return;
-    uint32_t lo = 0u, hi = q.seqs; /* the sequence whose range holds r */
-    while (hi - lo > 1u) {
-        const uint32_t mid = (lo + hi) / 2u;
-        if ((uint32_t)kv_cu[mid] <= r) lo = mid;
-        else hi = mid;
+    __shared__ long long s_src[16]; /* first element of the cache row; -1: none */
+    const uint32_t r0 = blockIdx.x * 16u, chunks = m.pitch / 8u;
+    if (threadIdx.x < 16u) {
+        const uint32_t r = r0 + threadIdx.x;
+        long long src = -1;
+        if (r < total) {
+            uint32_t lo = 0u, hi = q.seqs; /* the sequence whose range holds r */
+            while (hi - lo > 1u) {
+                const uint32_t mid = (lo + hi) / 2u;
+                if ((uint32_t)kv_cu[mid] <= r) lo = mid;
+                else hi = mid;
+            }
+            const int32_t slot = q.slot[lo];
+            const uint32_t at = r - (uint32_t)kv_cu[lo];
+            if (slot >= 0 && (uint32_t)slot < q.slots && at < m.tmax) src = (long long)(((size_t)slot * m.tmax + at) * m.pitch);
+        }
+        s_src[threadIdx.x] = src;
     }
-    const int32_t slot = q.slot[lo];
-    const uint32_t at = r - (uint32_t)kv_cu[lo];
-    if (slot < 0 || (uint32_t)slot >= q.slots || at >= m.tmax) return;
-    reinterpret_cast<gd_bf16x8 *>(packed + (size_t)r * m.pitch)[c] =
-        reinterpret_cast<const gd_bf16x8 *>(cache + ((size_t)slot * m.tmax + at) * m.pitch)[c];
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < 16u * chunks; i += 256u) {
+        const uint32_t r = i / chunks, c = i % chunks;
+        const long long src = s_src[r];
+        if (src >= 0)
+            reinterpret_cast<gd_bf16x8 *>(packed + (size_t)(r0 + r) * m.pitch)[c] =
+                reinterpret_cast<const gd_bf16x8 *>(cache + src)[c];
+    }
 }
 
 /* 16 bytes per lane from global memory straight into LDS (lane l's data lands at lds_address + 16*l); the kernel
@@ -299,7 +310,7 @@ gd_latent_prefill_kernel(const gd_bf16 *__restrict__ q_rows, const gd_bf16 *__re
 extern "C" int gd_hip_launch_latent_gather(hipStream_t stream, const void *cache, const int32_t *kv_cu, void *packed,
                                            uint32_t total, const gd_hip_latent_params *m, const gd_hip_seqs *q)
 {
-    gd_latent_gather_kernel<<<(unsigned)(((uint64_t)total * (m->pitch / 8u) + 255u) / 256u), 256, 0, stream>>>((const gd_bf16 *)cache, kv_cu, (gd_bf16 *)packed, total, *m, *q);
+    gd_latent_gather_kernel<<<(total + 15u) / 16u, 256, 0, stream>>>((const gd_bf16 *)cache, kv_cu, (gd_bf16 *)packed, total, *m, *q);
     return (int)hipGetLastError();
 }
 

@@ -378,7 +378,8 @@ class Latent:
 
 
 LATENT_SIZES = [(4, 24, 8, 16, 48), (3, 64, 16, 64, 128), (16, 128, 64, 128, 512), (17, 32, 16, 40, 64), (2, 20, 6, 10, 21),
-                (1, 8, 2, 8, 16), (20, 128, 32, 96, 256), (5, 192, 64, 128, 192), (1, 1, 2, 1, 1)]
+                (1, 8, 2, 8, 16), (20, 128, 32, 96, 256), (5, 192, 64, 128, 192), (1, 1, 2, 1, 1),
+                (40, 16, 8, 8, 32), (18, 16, 16, 16, 640)]
 
 
 @TYPES
