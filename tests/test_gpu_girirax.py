@@ -615,6 +615,40 @@ def test_greedy_generation_through_the_entry_point(D, L, models):
 
 
 @DTYPES
+def test_the_inference_program_opens_a_model_folder(D, models, compute):
+    folder, tokens, _, _, _ = models("mixed")
+    prompt = tokens[0][:11]
+    exe = os.path.join(ROOT, "gradients.c_amd", "gpt_lm_infer")
+
+    def run(*args):
+        r = subprocess.run([exe, "--checkpoint", folder, "--dtype", compute, *args], capture_output=True, timeout=60)
+        return r.returncode, r.stdout.decode(), r.stderr.decode()
+    ids = ",".join(str(int(t)) for t in prompt)
+    d = _decoder(D, folder, compute, max_seq=40, batch=1)
+    try:
+        greedy = d.generate(prompt, [0, len(prompt)], 12)[0].tolist()
+        sampled = d.generate(prompt, [0, len(prompt)], 12, 0.9, 0.02, 1.2, 0.0, -1,
+                             D.lib().gd_gpt_generation_rng(5, 1, 0))[0].tolist()
+    finally:
+        d.close()
+    line = lambda out: [int(v) for v in next(l for l in out.splitlines() if l.startswith("ids:"))[4:].split()]
+    rc, out, err = run("--token-ids", ids, "--max-new-tokens", "12")
+    assert rc == 0, (rc, err)
+    assert line(out) == greedy and "architecture=Girirax" in out and "prompt_tokens=11" in out
+    rc, out, err = run("--token-ids", ids, "--max-new-tokens", "12", "--temperature", "0.9", "--min-p", "0.02",
+                       "--repetition-penalty", "1.2", "--seed", "5")
+    assert rc == 0 and line(out) == sampled
+    stop = greedy[5]
+    rc, out, err = run("--token-ids", ids, "--max-new-tokens", "12", "--stop-token", str(stop))
+    assert rc == 0 and line(out) == greedy[:greedy.index(stop)]
+    rc, out, err = run("--token-ids", "1,2,1000000")
+    assert rc == 1 and "vocabulary" in err
+    rc, out, err = run("--token-ids", "1,two")
+    assert rc == 1 and "list" in err
+    assert run("--token-ids", "1", "--prompt", "x")[0] == 2
+
+
+@DTYPES
 def test_long_decoding(D, L, tmp_path, compute):
     """Hundreds of single tokens behind a short prompt: the state is carried, the cache grows over several pieces."""
     cfg = G.config([G.mamba(), G.latent()], vocab=64, width=48, ff=64)
