@@ -142,7 +142,7 @@ gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__re
 #pragma unroll
         for (int s = 0; s < HS; ++s) {
             const uint32_t c = 4u * (hf * (uint32_t)HS + (uint32_t)s) + lg;
-            qf[n][s] = c < chunks ? *reinterpret_cast<const gd_bf16x8 *>(qr + c * 8u) : zero;
+            qf[n][s] = *reinterpret_cast<const gd_bf16x8 *>(qr + (c < chunks ? c * 8u : 0u));
         }
     }
     gd_float4 o[HG][CT];
@@ -162,12 +162,20 @@ gd_latent_attend_mfma_kernel(const gd_bf16 *__restrict__ ql, const gd_bf16 *__re
 
     issue(k_begin, 0u);
     if (k_begin + GD_LD_TILE < k_end) issue(k_begin + GD_LD_TILE, 1u);
+    /* The query rows are complete from here on.  Without this use of them the compiler, which does not count the loads
+     * into LDS, would wait for all memory at their first use in every pass of the loop: right behind the request for
+     * the next tile. */
+#pragma unroll
+    for (int n = 0; n < HG; ++n)
+#pragma unroll
+        for (int s = 0; s < HS; ++s) {
+            qf[n][s] = 4u * (hf * (uint32_t)HS + (uint32_t)s) + lg < chunks ? qf[n][s] : zero;
+            asm volatile("" : "+v"(qf[n][s]));
+        }
     uint32_t it = 0u;
     for (uint32_t k0 = k_begin; k0 < k_end; k0 += GD_LD_TILE, ++it) {
         const unsigned char *tile = gd_ld_smem + (it & 1u) * STAGE;
-        /* this wavefront's share of the tile is in LDS; the second tile was requested with the first */
-        if (it == 0u && k0 + GD_LD_TILE < k_end) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(NL) : "memory");
-        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); /* this wavefront's share of the tile is in LDS */
         __syncthreads(); /* everyone's share is, and the other stage is no longer read */
         if (it != 0u && k0 + GD_LD_TILE < k_end) issue(k0 + GD_LD_TILE, (it + 1u) & 1u);
         gd_float4 sp[HG];

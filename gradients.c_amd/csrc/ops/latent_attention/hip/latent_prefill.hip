@@ -128,10 +128,26 @@ gd_latent_prefill_kernel(const gd_bf16 *__restrict__ q_rows, const gd_bf16 *__re
 #pragma unroll
         for (int ks = 0; ks < KSTEPS; ++ks) {
             const uint32_t e0 = 16u * ks + 8u * hh;
-            qf[ks] = (gd_bf16x8)(gd_bf16)0.f;
-            if (!row_live || e0 >= qd) continue;
-            qf[ks] = *reinterpret_cast<const gd_bf16x8 *>(qp + e0);
-            if (e0 >= m.dim) {
+            qf[ks] = *reinterpret_cast<const gd_bf16x8 *>(qp + (e0 < qd ? e0 : 0u)); /* rows behind the end: the last */
+        }
+#pragma unroll
+        for (int ks = 0; ks < KSTEPS; ++ks) {
+            const uint32_t e0 = 16u * ks + 8u * hh;
+            if (e0 >= qd) {
+                qf[ks] = (gd_bf16x8)(gd_bf16)0.f;
+            } else if (e0 >= m.dim && half % 8u == 0u) { /* the 8 elements lie in one half */
+                const uint32_t r0 = e0 - m.dim, p0 = r0 < half ? r0 : r0 - half;
+                const gd_bf16x8 other = *reinterpret_cast<const gd_bf16x8 *>(qp + m.dim + (r0 < half ? r0 + half : p0));
+                const gd_float4 c4[2] = {*reinterpret_cast<const gd_float4 *>(ang + p0),
+                                         *reinterpret_cast<const gd_float4 *>(ang + p0 + 4u)};
+                const gd_float4 s4[2] = {*reinterpret_cast<const gd_float4 *>(ang + half + p0),
+                                         *reinterpret_cast<const gd_float4 *>(ang + half + p0 + 4u)};
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const float c = c4[e >> 2][e & 3], s = s4[e >> 2][e & 3], own = (float)qf[ks][e], far = (float)other[e];
+                    qf[ks][e] = (gd_bf16)(r0 < half ? own * c - far * s : own * c + far * s);
+                }
+            } else if (e0 >= m.dim) {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) {
                     const uint32_t r = e0 + (uint32_t)e - m.dim, p = r < half ? r : r - half;
@@ -274,26 +290,40 @@ gd_latent_prefill_kernel(const gd_bf16 *__restrict__ q_rows, const gd_bf16 *__re
     }
 
     /* normalise and gate in registers, then through LDS so that rows leave in whole pieces */
+    const gd_bf16 *gr = gate + qrow * ldg + head * m.vdim;
+    gd_bf16x4 gv[DTILES][4]; /* requested together */
+    if (((reinterpret_cast<uintptr_t>(gate) | (ldg * 2u)) & 7u) == 0u) {
+#pragma unroll
+        for (int dt = 0; dt < DTILES; ++dt)
+#pragma unroll
+            for (int a = 0; a < 4; ++a) {
+                const uint32_t c = 32u * dt + 8u * a + 4u * hh;
+                gv[dt][a] = *reinterpret_cast<const gd_bf16x4 *>(gr + (c < m.vdim ? c : 0u));
+            }
+    } else {
+#pragma unroll
+        for (int dt = 0; dt < DTILES; ++dt)
+#pragma unroll
+            for (int a = 0; a < 4; ++a)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const uint32_t c = 32u * dt + 8u * a + 4u * hh;
+                    gv[dt][a][r] = gr[(c < m.vdim ? c : 0u) + (uint32_t)r];
+                }
+    }
     l += __shfl_xor(l, 32, 64);
     const float inv = l > 0.f ? 1.f / l : 0.f;
     constexpr uint32_t OS = 32u * DTILES + 8u; /* elements per row of the LDS block */
     __syncthreads(); /* all fragment reads of the last block are done */
     gd_bf16 *sO = reinterpret_cast<gd_bf16 *>(gd_lp_smem) + (size_t)wave * 32u * OS;
-    const gd_bf16 *gr = gate + qrow * ldg + head * m.vdim;
-    const bool g8 = ((reinterpret_cast<uintptr_t>(gate) | (ldg * 2u) | (m.vdim * 2u)) & 7u) == 0u;
 #pragma unroll
     for (int dt = 0; dt < DTILES; ++dt) {
 #pragma unroll
         for (int a = 0; a < 4; ++a) {
             const uint32_t c = 32u * dt + 8u * a + 4u * hh;
-            gd_bf16x4 hv = (gd_bf16x4)(gd_bf16)0.f, gv = hv;
-            if (c < m.vdim) {
-                if (g8) gv = *reinterpret_cast<const gd_bf16x4 *>(gr + c);
-                else
-                    for (int r = 0; r < 4; ++r) gv[r] = gr[c + (uint32_t)r];
-            }
+            gd_bf16x4 hv;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) hv[r] = (gd_bf16)(o[dt][4 * a + r] * inv * gd_sigmoid_fast((float)gv[r]));
+            for (int r = 0; r < 4; ++r) hv[r] = (gd_bf16)(o[dt][4 * a + r] * inv * gd_sigmoid_fast((float)gv[dt][a][r]));
             *reinterpret_cast<gd_bf16x4 *>(sO + lq * OS + c) = hv;
         }
     }
