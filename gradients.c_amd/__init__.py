@@ -86,7 +86,7 @@ class SdpaDecodeArgs(C.Structure):
 
 class FusedLinearArgs(C.Structure):
     _fields_ = [("w_is_nk", C.c_uint32), ("bias_mode", C.c_uint32), ("prologue", C.c_uint32), ("eps", C.c_float),
-                ("epilogue", C.c_uint32)]
+                ("epilogue", C.c_uint32), ("gate_limit", C.c_float), ("gate_alpha", C.c_float)]
 
 
 class MinimaxArgs(C.Structure):  # gd_backend_minimax_m3_sparse_args
@@ -117,6 +117,33 @@ class SsmArgs(C.Structure):  # gd_backend_ssm_args
 class LatentArgs(C.Structure):  # gd_backend_latent_args
     _fields_ = [(n, C.c_uint32) for n in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank")] + \
                [("scale", C.c_float), ("eps", C.c_float)]
+
+
+class GroupedArgs(C.Structure):  # gd_backend_grouped_args
+    _fields_ = [(n, C.c_uint32) for n in ("heads", "kv_heads", "dim", "vdim", "rot_dims", "chunk")] + \
+               [("scale", C.c_float), ("rot_mult", C.c_float)]
+
+
+class RoutedRows(C.Structure):  # gd_backend_routed_rows
+    _fields_ = [("rows", C.POINTER(TensorView)), ("place", C.POINTER(TensorView)), ("top", C.c_uint32),
+                ("weight", C.c_float)]
+
+
+class RoutedArgs(C.Structure):  # gd_backend_routed_args
+    _fields_ = [(n, C.c_uint32) for n in ("experts", "top", "width", "ff")] + \
+               [(n, C.c_float) for n in ("gate_limit", "gate_alpha", "weight")]
+
+
+class RouteJob(C.Structure):  # gd_backend_route_job
+    _fields_ = [(n, C.POINTER(TensorView)) for n in ("table", "place", "first", "tiles")] + \
+               [("args", C.POINTER(RoutedArgs))]
+
+
+class Routes(C.Structure):  # gd_backend_routes
+    _fields_ = [("first", C.POINTER(TensorView)), ("tiles", C.POINTER(TensorView)), ("rows", C.c_uint32)]
+
+
+ROUTED_PAD = 256  # GD_BACKEND_ROUTED_PAD
 
 
 class ConcatArgs(C.Structure):
@@ -194,6 +221,10 @@ _SIGNATURES = {
     "gd_backend_minimax_m3_sparse_attention": [_vp, _TV, _TV, _TV, _TV, _TV, _TV, C.POINTER(MinimaxArgs)],
     "gd_backend_residual_embed": [_vp, _TV, _TV, _TV, _TV, C.c_float],
     "gd_backend_residual_norm_add": [_vp, _TV, _TV, _TV, _TV, C.c_float, C.c_float],
+    "gd_backend_residual_add_norm": [_vp, _TV, C.POINTER(RoutedRows), _TV, _TV, _TV, C.POINTER(RoutedRows), C.c_float],
+    "gd_backend_grouped_attend": [_vp, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(GroupedArgs)],
+    "gd_backend_route_by_tables": [_vp, C.POINTER(RouteJob), C.c_uint32, _TV, C.c_uint32],
+    "gd_backend_routed_mlp": [_vp, _TV, _TV, _TV, _TV, _TV, C.POINTER(Routes), C.POINTER(RoutedArgs)],
     "gd_backend_residual_norm_rows": [_vp, _TV, _TV, _TV, _TV, C.c_float],
     "gd_backend_causal_conv_silu": [_vp, _MV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs)],
     "gd_backend_ssm_scan": [_vp, _TV, _MV, _TV, _TV, _TV, _TV, _TV, C.POINTER(PackedSeqs), C.POINTER(SsmArgs)],
@@ -232,6 +263,8 @@ _OTHER_RESTYPE = {
     "gd_backend_sample_work_count": (C.c_size_t, [C.c_uint32, C.c_uint32]),
     "gd_backend_latent_pitch": (C.c_uint32, [C.c_uint32, C.c_uint32]),
     "gd_backend_latent_work_bytes": (C.c_size_t, [_vp, C.POINTER(LatentArgs)] + [C.c_uint32] * 5),
+    "gd_backend_grouped_work_bytes": (C.c_size_t, [_vp, C.POINTER(GroupedArgs)] + [C.c_uint32] * 4),
+    "gd_backend_route_tiles": (C.c_uint32, [C.POINTER(RoutedArgs), C.c_uint32, C.c_uint32]),
     "gd_backend_graph_destroy": (None, [_vp]),
 }
 EXPORTED_SYMBOLS = sorted(list(_SIGNATURES) + list(_OTHER_RESTYPE))
@@ -499,8 +532,9 @@ class Backend:
         _check(self.call("gd_backend_swiglu_split_linear", x12.matrix(), w.matrix(),
                          bias.vector() if bias else None, y.matrix()), "gd_backend_swiglu_split_linear")
 
-    def fused_linear(self, x, w, bias, residual, norm_weight, y, w_is_nk, bias_mode, prologue, eps=0.0, epilogue=0):
-        a = FusedLinearArgs(int(w_is_nk), bias_mode, prologue, eps, epilogue)
+    def fused_linear(self, x, w, bias, residual, norm_weight, y, w_is_nk, bias_mode, prologue, eps=0.0, epilogue=0,
+                     gate_limit=0.0, gate_alpha=0.0):
+        a = FusedLinearArgs(int(w_is_nk), bias_mode, prologue, eps, epilogue, gate_limit, gate_alpha)
         _check(self.call("gd_backend_fused_linear", x.matrix(), w.matrix(), bias.vector() if bias else None,
                          residual.matrix() if residual else None, norm_weight.vector() if norm_weight else None,
                          y.matrix(), C.byref(a)), "gd_backend_fused_linear")

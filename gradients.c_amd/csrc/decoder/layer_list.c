@@ -1,317 +1,113 @@
 /*
- * The decoder whose layers are listed in a configuration (layer_list.h): weights, caches and states, and one forward
- * over packed new tokens that serves prompts, portions of prompts and decode steps alike.
+ * The decoder whose layers are listed in a configuration (layer_list.h): caches, states, and one forward over packed new
+ * tokens that serves prompts, portions of prompts and decode steps alike.
  *
- * Per layer, with an F32 residual stream x and its copy h in the projections' type:
- *   mixer   mamba2            in -> causal conv + silu -> recurrence -> gate, group norm -> out
- *           latent_attention  [dq | dkv | g] -> norms, rotation, cache append -> uq -> attention, output gate -> out
- *   x += m * norm1(mixer(h));  h = x
- *   feed-forward  gelu(gate) * up with biases -> down;  x += m * norm2(ff(h));  h = x
+ * The residual stream x is F32; h is what a sublayer reads, in the projections' type.
+ *   mixer   mamba2              in -> causal conv + silu -> recurrence -> gate, group norm -> out
+ *           latent_attention    [dq | dkv | g] -> norms, rotation, cache append -> uq -> attention, output gate -> out
+ *           grouped attention   [q | k | v | g] -> rotation, attention, output gate, cache append -> out
+ *   feed-forward  gelu(gate) * up with biases -> down;  relu(up)^2 -> down;  routed experts and a shared one
+ * Norms on the outputs:  x += m * norm1(mixer(h)), h = x;  x += m * norm2(ff(h)), h = x.
+ * Norms first:  h = norm1(x), x += mixer(h);  h = norm2(x), x += ff(h): a sublayer's result is added together with the norm in
+ * front of the next one, so that the stream is read and written once per sublayer.
  * Projections that read the same input are one weight matrix.  What a sequence keeps: the convolution's last inputs and
- * the recurrent state (mamba2), the latent and the rotated key part of every token (latent_attention), each in the
- * place of its slot; positions decide what of it is read, so nothing is cleared when a slot is used again.
+ * the recurrent state (mamba2), the latent and the rotated key part of every token (latent_attention), rotated keys and
+ * values of every token, or with chunks of the current chunk's (grouped attention), each in the place of its slot;
+ * positions decide what of it is read, so nothing is cleared when a slot is used again.
  */
 #include <math.h>
 #include <stdio.h>
 
-#include "layer_list.h"
-
-#define MAX_PIECES 3
-
-typedef struct layer_weights {
-    gd_tensor norm1, norm2;
-    gd_tensor in, conv, conv_b, dt_bias, a_log, d_skip, gnorm; /* mamba2; in: also [dq | dkv | g] of latent attention */
-    gd_tensor dq_norm, dkv_norm, uq, ukv, ukt, freq; /* latent attention; ukv: [uk | uv]; ukt: uk turned per head */
-    gd_tensor out;
-    gd_tensor upgate, upgate_b, down, down_b; /* feed-forward; upgate: [up | gate] */
-    gd_tensor ring, states, cache;            /* per slot */
-} layer_weights;
-
-struct layer_list {
-    layer_list_config c;
-    gd_dtype type; /* of projections and activations */
-    int32_t max_step_tokens;
-    int32_t kv_rows; /* tokens whose keys and values a step may expand at once (latent attention) */
-    gd_tensor embed, final_norm;
-    layer_weights *layers;
-    gd_tensor rows_dev, cu_dev; /* 0 .. batch-1 and 0 .. batch: the tables of a decode step over every slot */
-};
-
-static int64_t conv_channels(const layer_config *l)
-{
-    return (int64_t)l->ssm.heads * l->ssm.vdim + 2 * (int64_t)l->ssm.groups * l->ssm.state;
-}
-static int64_t inner_size(const layer_config *l) { return (int64_t)l->ssm.heads * l->ssm.vdim; }
-static int64_t mixer_in(const layer_config *l)
-{
-    if (l->mixer == MIXER_MAMBA2) return inner_size(l) + conv_channels(l) + l->ssm.heads;
-    return (int64_t)l->latent.q_rank + l->latent.kv_rank + l->latent.rot_dim + (int64_t)l->latent.heads * l->latent.vdim;
-}
-static int64_t mixer_out(const layer_config *l)
-{
-    return l->mixer == MIXER_MAMBA2 ? inner_size(l) : (int64_t)l->latent.heads * l->latent.vdim;
-}
-static int64_t query_size(const layer_config *l)
-{
-    return (int64_t)l->latent.heads * (l->latent.dim + l->latent.rot_dim);
-}
-
-/* ---- weights ------------------------------------------------------------------------------------- */
-
-/* One weight of the decoder: where it goes, its type and shape, the tensors of the file that are stacked in it, and the
- * range of random weights. */
-typedef struct weight {
-    gd_tensor *dst;
-    gd_dtype type;
-    int64_t rows, cols; /* cols 0: a vector */
-    const char *piece[MAX_PIECES];
-    int64_t piece_rows[MAX_PIECES];
-    float lo, hi;
-} weight;
-
-typedef gd_status (*weight_fn)(void *user, const weight *w, int32_t layer);
-
-/* calls fn for every weight, the layers' in order (layer -1: the model's own); ll->layers NULL: destinations are NULL */
-static gd_status each_weight(const layer_list_config *c, gd_dtype type, struct layer_list *ll, weight_fn fn, void *user)
-{
-    int32_t i;
-#define AT(field) (ll != NULL ? &ll->field : NULL)
-#define ONE(dst_, type_, rows_, cols_, name_, lo_, hi_)                                                         \
-    do {                                                                                                        \
-        const weight w_ = {dst_, type_, rows_, cols_, {name_, NULL, NULL}, {rows_, 0, 0}, lo_, hi_};            \
-        TRY(fn(user, &w_, i));                                                                                  \
-    } while (0)
-    i = -1;
-    ONE(AT(embed), type, c->vocab, c->width, "embed", -0.05f, 0.05f);
-    ONE(AT(final_norm), GD_DTYPE_F32, c->width, 0, "final.norm", 1.0f, 1.0f);
-    for (i = 0; i < c->n_layers; ++i) {
-        const layer_config *l = &c->layers[i];
-        const float wide = 1.7f / sqrtf((float)c->width); /* uniform range whose products keep unit variance */
-        ONE(AT(layers[i].norm1), GD_DTYPE_F32, c->width, 0, "norm1", 1.0f, 1.0f);
-        if (l->mixer == MIXER_MAMBA2) {
-            const int64_t ch = conv_channels(l), H = l->ssm.heads;
-            ONE(AT(layers[i].in), type, mixer_in(l), c->width, "mix.in", -wide, wide);
-            ONE(AT(layers[i].conv), GD_DTYPE_F32, ch, l->taps, "mix.conv", -0.5f, 0.5f);
-            ONE(AT(layers[i].conv_b), GD_DTYPE_F32, ch, 0, "mix.conv.b", -0.1f, 0.1f);
-            ONE(AT(layers[i].dt_bias), GD_DTYPE_F32, H, 0, "mix.dt_bias", -4.6f, -2.3f);
-            ONE(AT(layers[i].a_log), GD_DTYPE_F32, H, 0, "mix.A_log", 0.0f, 2.7f);
-            ONE(AT(layers[i].d_skip), GD_DTYPE_F32, H, 0, "mix.D", 0.5f, 1.5f);
-            ONE(AT(layers[i].gnorm), GD_DTYPE_F32, inner_size(l), 0, "mix.norm", 1.0f, 1.0f);
-        } else {
-            const gd_backend_latent_args *a = &l->latent;
-            const int64_t H = a->heads;
-            const float qr = 1.7f / sqrtf((float)a->q_rank), kr = 1.7f / sqrtf((float)a->kv_rank);
-            const weight in = {AT(layers[i].in), type, mixer_in(l), c->width, {"mix.dq", "mix.dkv", "mix.g"},
-                               {a->q_rank, (int64_t)a->kv_rank + a->rot_dim, H * a->vdim}, -wide, wide};
-            const weight ukv = {AT(layers[i].ukv), type, H * ((int64_t)a->dim + a->vdim), a->kv_rank,
-                                {"mix.uk", "mix.uv", NULL}, {H * a->dim, H * a->vdim, 0}, -kr, kr};
-            TRY(fn(user, &in, i));
-            ONE(AT(layers[i].dq_norm), GD_DTYPE_F32, a->q_rank, 0, "mix.dq.norm", 1.0f, 1.0f);
-            ONE(AT(layers[i].dkv_norm), GD_DTYPE_F32, a->kv_rank, 0, "mix.dkv.norm", 1.0f, 1.0f);
-            ONE(AT(layers[i].uq), type, query_size(l), a->q_rank, "mix.uq", -qr, qr);
-            TRY(fn(user, &ukv, i));
-            ONE(AT(layers[i].ukt), type, H * a->kv_rank, a->dim, NULL, 0.0f, 0.0f); /* from ukv */
-            ONE(AT(layers[i].freq), GD_DTYPE_F32, a->rot_dim / 2, 0, NULL, 0.0f, 0.0f); /* computed, not stored */
-        }
-        ONE(AT(layers[i].out), type, c->width, mixer_out(l), "mix.o", -wide, wide);
-        if (l->ff > 0) {
-            const weight ug = {AT(layers[i].upgate), type, 2 * (int64_t)l->ff, c->width, {"mlp.up", "mlp.gate", NULL},
-                               {l->ff, l->ff, 0}, -wide, wide};
-            const weight ugb = {AT(layers[i].upgate_b), type, 2 * (int64_t)l->ff, 0, {"mlp.up.b", "mlp.gate.b", NULL},
-                                {l->ff, l->ff, 0}, -0.1f, 0.1f};
-            const float fr = 1.7f / sqrtf((float)l->ff);
-            TRY(fn(user, &ug, i));
-            TRY(fn(user, &ugb, i));
-            ONE(AT(layers[i].down), type, c->width, l->ff, "mlp.down", -fr, fr);
-            ONE(AT(layers[i].down_b), type, c->width, 0, "mlp.down.b", -0.1f, 0.1f);
-            ONE(AT(layers[i].norm2), GD_DTYPE_F32, c->width, 0, "norm2", 1.0f, 1.0f);
-        }
-    }
-#undef ONE
-#undef AT
-    return GD_OK;
-}
-
-static int64_t weight_count(const weight *w) { return w->rows * (w->cols > 0 ? w->cols : 1); }
-
-static gd_status add_bytes(void *user, const weight *w, int32_t layer)
-{
-    (void)layer;
-    *(size_t *)user += gd_pad256((size_t)weight_count(w) * gd_dtype_size(w->type));
-    return GD_OK;
-}
-
-typedef struct weight_load {
-    gd_context *ctx;
-    const layer_list_config *c;
-    gd_safetensors *file;
-    uint64_t seed;
-    unsigned char *raw, *turned; /* host staging of the largest weight */
-    gd_tensor *ukv;              /* the layer's, already filled */
-} weight_load;
-
-static gd_status allocate_weight(void *user, const weight *w, int32_t layer)
-{
-    const weight_load *wl = (const weight_load *)user;
-    int64_t dims[2] = {w->rows, w->cols};
-    (void)layer;
-    return gd_tensor_empty(wl->ctx, GD_ARENA_PARAMS, w->type, gd_shape_make(w->cols > 0 ? 2U : 1U, dims), 256U, w->dst);
-}
-
-static float bf16_value(uint16_t bits)
-{
-    const uint32_t u = (uint32_t)bits << 16;
-    float f;
-    memcpy(&f, &u, sizeof(f));
-    return f;
-}
-
-static uint16_t bf16_bits(float f) /* to nearest, ties to even */
-{
-    uint32_t u;
-    memcpy(&u, &f, sizeof(u));
-    if ((u & 0x7fffffffU) > 0x7f800000U) return (uint16_t)((u >> 16) | 0x40U); /* NaN stays NaN */
-    return (uint16_t)((u + 0x7fffU + ((u >> 16) & 1U)) >> 16);
-}
-
-/* n values of a file tensor into dst as type `to` */
-static void convert(const unsigned char *src, gd_dtype from, unsigned char *dst, gd_dtype to, int64_t n)
-{
-    int64_t i;
-    if (from == to) {
-        memcpy(dst, src, (size_t)n * gd_dtype_size(to));
-        return;
-    }
-#pragma omp parallel for schedule(static) if (n > 65536)
-    for (i = 0; i < n; ++i) {
-        const float f = from == GD_DTYPE_F32 ? ((const float *)src)[i] : bf16_value(((const uint16_t *)src)[i]);
-        if (to == GD_DTYPE_F32) ((float *)dst)[i] = f;
-        else ((uint16_t *)dst)[i] = bf16_bits(f);
-    }
-}
-
-static void tensor_name(char *out, size_t size, const char *piece, int32_t layer)
-{
-    if (layer < 0) (void)snprintf(out, size, "%s", piece);
-    else (void)snprintf(out, size, "l%d.%s", (int)layer, piece);
-}
-
-/* the file holds the piece in the right shape and a type that converts */
-static gd_status check_weight(void *user, const weight *w, int32_t layer)
-{
-    weight_load *wl = (weight_load *)user;
-    int p;
-    for (p = 0; p < MAX_PIECES && w->piece[p] != NULL; ++p) {
-        char name[64];
-        const gd_safetensor *t;
-        tensor_name(name, sizeof(name), w->piece[p], layer);
-        t = gd_safetensors_find(wl->file, name);
-        if (t == NULL || t->rank != (w->cols > 0 ? 2U : 1U) || t->shape[0] != w->piece_rows[p] ||
-            (w->cols > 0 && t->shape[1] != w->cols))
-            return GD_ERR_BAD_STATE;
-        if (t->dtype != GD_DTYPE_BF16 && t->dtype != GD_DTYPE_F32) return GD_ERR_UNSUPPORTED;
-    }
-    return GD_OK;
-}
-
-static gd_status fill_weight(void *user, const weight *w, int32_t layer)
-{
-    weight_load *wl = (weight_load *)user;
-    const int64_t n = weight_count(w);
-    int64_t done = 0;
-    int p;
-    if (w->piece[0] == NULL && w->cols > 0) { /* ukt [heads, kv_rank, dim] from the first part of ukv [heads, dim, kv_rank] */
-        const gd_backend_latent_args *a = &wl->c->layers[layer].latent;
-        const size_t es = gd_dtype_size(w->type);
-        const int64_t D = a->dim, R = a->kv_rank;
-        gd_tensor uk;
-        TRY(gd_tensor_slice(wl->ctx, wl->ukv, 0U, 0, (int64_t)a->heads * D, &uk));
-        TRY(gd_tensor_read(wl->ctx, &uk, wl->raw, (size_t)n * es));
-#pragma omp parallel for schedule(static)
-        for (done = 0; done < n; ++done) {
-            const int64_t h = done / (R * D), r = done / D % R, d = done % D;
-            memcpy(wl->turned + (size_t)done * es, wl->raw + (size_t)((h * D + d) * R + r) * es, es);
-        }
-        return gd_tensor_write(wl->ctx, w->dst, wl->turned, (size_t)n * es);
-    }
-    if (w->piece[0] != NULL && !strcmp(w->piece[0], "mix.uk")) wl->ukv = w->dst;
-    if (w->piece[0] == NULL) { /* rotation frequencies: base^(-2i/dims), in double, rounded once */
-        const layer_config *l = &wl->c->layers[layer];
-        float *f = (float *)wl->turned;
-        for (done = 0; done < n; ++done)
-            f[done] = (float)pow(l->rot_base, -2.0 * (double)done / (double)l->latent.rot_dim);
-        return gd_tensor_write(wl->ctx, w->dst, f, (size_t)n * sizeof(float));
-    }
-    if (wl->file == NULL) {
-        wl->seed = gd_splitmix64(wl->seed);
-        return gd_backend_rand_uniform(gd_context_backend(wl->ctx), (gd_backend_buffer *)w->dst->storage.buffer,
-                                       w->dst->storage.offset, (size_t)n, (uint32_t)w->type, wl->seed, w->lo, w->hi);
-    }
-    for (p = 0; p < MAX_PIECES && w->piece[p] != NULL; ++p) {
-        const int64_t m = w->piece_rows[p] * (w->cols > 0 ? w->cols : 1);
-        char name[64];
-        const gd_safetensor *t;
-        tensor_name(name, sizeof(name), w->piece[p], layer);
-        t = gd_safetensors_find(wl->file, name);
-        TRY(gd_safetensors_read(wl->file, t, wl->raw));
-        convert(wl->raw, t->dtype, wl->turned + (size_t)done * gd_dtype_size(w->type), w->type, m);
-        done += m;
-    }
-    return gd_tensor_write(wl->ctx, w->dst, wl->turned, (size_t)n * gd_dtype_size(w->type));
-}
-
-static gd_status largest_weight(void *user, const weight *w, int32_t layer)
-{
-    int64_t *most = (int64_t *)user;
-    (void)layer;
-    if (weight_count(w) > *most) *most = weight_count(w);
-    return GD_OK;
-}
-
-static gd_status load_weights(gd_context *ctx, struct layer_list *ll, gd_safetensors *file, uint64_t seed)
-{
-    weight_load wl = {ctx, &ll->c, file, seed, NULL, NULL, NULL};
-    int64_t most = 0;
-    gd_status st;
-    if (file != NULL) TRY(each_weight(&ll->c, ll->type, ll, check_weight, &wl)); /* before the first byte is written */
-    TRY(each_weight(&ll->c, ll->type, ll, allocate_weight, &wl));
-    TRY(each_weight(&ll->c, ll->type, ll, largest_weight, &most));
-    wl.raw = (unsigned char *)malloc((size_t)most * 4U);
-    wl.turned = (unsigned char *)malloc((size_t)most * 4U);
-    st = wl.raw == NULL || wl.turned == NULL ? GD_ERR_OUT_OF_MEMORY : each_weight(&ll->c, ll->type, ll, fill_weight, &wl);
-    free(wl.raw);
-    free(wl.turned);
-    return st;
-}
+#include "layer_list_internal.h"
 
 /* ---- caches and states ----------------------------------------------------------------------------- */
 
-static void state_dims(const layer_config *l, int64_t slots, int64_t max_seq, int64_t ring[3], int64_t states[4],
-                       int64_t cache[3])
+/* what a layer keeps: mamba2 its ring and states, latent attention its cache, grouped attention keys and values */
+typedef struct state_shapes {
+    int64_t ring[3], states[4], cache[3], k[4], v[4];
+} state_shapes;
+
+static state_shapes state_dims(const layer_config *l, int64_t slots, int64_t max_seq)
 {
-    ring[0] = states[0] = cache[0] = slots;
-    ring[1] = l->taps;
-    ring[2] = conv_channels(l);
-    states[1] = l->ssm.heads;
-    states[2] = l->ssm.state;
-    states[3] = l->ssm.vdim;
-    cache[1] = max_seq;
-    cache[2] = gd_backend_latent_pitch(l->latent.kv_rank, l->latent.rot_dim);
+    state_shapes s;
+    memset(&s, 0, sizeof(s));
+    s.ring[0] = s.states[0] = s.cache[0] = s.k[0] = s.v[0] = slots;
+    s.ring[1] = l->taps;
+    s.ring[2] = conv_channels(l);
+    s.states[1] = l->ssm.heads;
+    s.states[2] = l->ssm.state;
+    s.states[3] = l->ssm.vdim;
+    s.cache[1] = max_seq;
+    s.cache[2] = gd_backend_latent_pitch(l->latent.kv_rank, l->latent.rot_dim);
+    s.k[1] = s.v[1] = l->grouped.kv_heads;
+    s.k[2] = s.v[2] = l->grouped.chunk > 0U && l->grouped.chunk < max_seq ? l->grouped.chunk : max_seq;
+    s.k[3] = l->grouped.dim;
+    s.v[3] = l->grouped.vdim;
+    return s;
 }
 
-static size_t state_bytes(const layer_list_config *c, gd_dtype type, int64_t slots, int64_t max_seq)
+static size_t dims_bytes(const int64_t *dims, int rank, size_t es)
+{
+    int i;
+    for (i = 0; i < rank; ++i) es *= (size_t)dims[i];
+    return gd_pad256(es);
+}
+
+/* the tables of a routed layer for steps of up to `rows` tokens: place, first, tiles */
+static void route_dims(const layer_config *l, int64_t rows, int64_t dims[3])
+{
+    dims[0] = rows * l->routed.top;
+    dims[1] = (int64_t)l->routed.experts + 1;
+    dims[2] = 2 + 2 * (int64_t)gd_backend_route_tiles(&l->routed, (uint32_t)rows, 1U);
+}
+
+static size_t state_bytes(const layer_list_config *c, gd_dtype type, int64_t slots, int64_t max_seq, int64_t step_tokens)
 {
     const size_t es = gd_dtype_size(type);
     size_t total = 0U;
-    int32_t i;
+    int32_t i, t;
     for (i = 0; i < c->n_layers; ++i) {
-        int64_t r[3], s[4], k[3];
-        state_dims(&c->layers[i], slots, max_seq, r, s, k);
-        if (c->layers[i].mixer == MIXER_MAMBA2)
-            total += gd_pad256((size_t)(r[0] * r[1] * r[2]) * es) + gd_pad256((size_t)(s[0] * s[1] * s[2] * s[3]) * 4U);
-        else total += gd_pad256((size_t)(k[0] * k[1] * k[2]) * es);
+        const layer_config *l = &c->layers[i];
+        const state_shapes s = state_dims(l, slots, max_seq);
+        if (l->mixer == MIXER_MAMBA2) total += dims_bytes(s.ring, 3, es) + dims_bytes(s.states, 4, 4U);
+        else if (l->mixer == MIXER_LATENT_ATTENTION) total += dims_bytes(s.cache, 3, es);
+        else total += dims_bytes(s.k, 4, es) + dims_bytes(s.v, 4, es);
+        if (l->mlp == MLP_ROUTED && l->weights_of == i) {
+            int64_t r[3];
+            route_dims(l, step_tokens, r);
+            for (t = 0; t < 3; ++t) total += dims_bytes(&r[t], 1, 4U);
+        }
     }
     return total + 2U * gd_pad256((size_t)(slots + 1) * 4U);
+}
+
+static gd_status state_zeros(gd_context *ctx, gd_dtype type, uint32_t rank, int64_t *dims, gd_tensor *out)
+{
+    return gd_tensor_zeros(ctx, GD_ARENA_STATE, type, gd_shape_make(rank, dims), 256U, out);
+}
+
+static gd_status allocate_layer_state(gd_context *ctx, struct layer_list *ll, int32_t i, int64_t slots, int64_t max_seq)
+{
+    const layer_config *l = &ll->c.layers[i];
+    layer_weights *w = &ll->layers[i];
+    state_shapes s = state_dims(l, slots, max_seq);
+    if (l->mixer == MIXER_MAMBA2) {
+        TRY(state_zeros(ctx, ll->type, 3U, s.ring, &w->ring));
+        TRY(state_zeros(ctx, GD_DTYPE_F32, 4U, s.states, &w->states));
+    } else if (l->mixer == MIXER_LATENT_ATTENTION) {
+        TRY(state_zeros(ctx, ll->type, 3U, s.cache, &w->cache));
+    } else {
+        TRY(state_zeros(ctx, ll->type, 4U, s.k, &w->k_cache));
+        TRY(state_zeros(ctx, ll->type, 4U, s.v, &w->v_cache));
+    }
+    if (l->mlp == MLP_ROUTED && l->weights_of == i) {
+        int64_t r[3];
+        route_dims(l, ll->max_step_tokens, r);
+        TRY(state_zeros(ctx, GD_DTYPE_I32, 1U, &r[0], &w->place));
+        TRY(state_zeros(ctx, GD_DTYPE_I32, 1U, &r[1], &w->first));
+        TRY(state_zeros(ctx, GD_DTYPE_I32, 1U, &r[2], &w->tiles));
+    }
+    return GD_OK;
 }
 
 static gd_status allocate_states(gd_context *ctx, struct layer_list *ll, int64_t slots, int64_t max_seq)
@@ -320,17 +116,7 @@ static gd_status allocate_states(gd_context *ctx, struct layer_list *ll, int64_t
     int32_t *iota = (int32_t *)malloc((size_t)(slots + 1) * sizeof(int32_t));
     gd_status st = iota == NULL ? GD_ERR_OUT_OF_MEMORY : GD_OK;
     int32_t i;
-    for (i = 0; i < ll->c.n_layers && st == GD_OK; ++i) {
-        int64_t r[3], s[4], k[3];
-        state_dims(&ll->c.layers[i], slots, max_seq, r, s, k);
-        if (ll->c.layers[i].mixer == MIXER_MAMBA2) {
-            st = gd_tensor_zeros(ctx, GD_ARENA_STATE, ll->type, gd_shape_make(3U, r), 256U, &ll->layers[i].ring);
-            if (st == GD_OK)
-                st = gd_tensor_zeros(ctx, GD_ARENA_STATE, GD_DTYPE_F32, gd_shape_make(4U, s), 256U, &ll->layers[i].states);
-        } else {
-            st = gd_tensor_zeros(ctx, GD_ARENA_STATE, ll->type, gd_shape_make(3U, k), 256U, &ll->layers[i].cache);
-        }
-    }
+    for (i = 0; i < ll->c.n_layers && st == GD_OK; ++i) st = allocate_layer_state(ctx, ll, i, slots, max_seq);
     if (st == GD_OK) st = gd_tensor_empty(ctx, GD_ARENA_STATE, GD_DTYPE_I32, gd_shape_make(1U, bdim), 256U, &ll->rows_dev);
     if (st == GD_OK) st = gd_tensor_empty(ctx, GD_ARENA_STATE, GD_DTYPE_I32, gd_shape_make(1U, cdim), 256U, &ll->cu_dev);
     if (st == GD_OK) {
@@ -350,6 +136,7 @@ typedef struct scratch_sizes {
     int64_t proj, a, b, branch; /* elements per row */
     int64_t angles;             /* F32 values per row */
     size_t work;                /* bytes for the whole step */
+    int64_t packed, packed_ff;  /* elements for the whole step: packed rows of the routed experts, and their activations */
 } scratch_sizes;
 
 static int64_t max64(int64_t a, int64_t b) { return a > b ? a : b; }
@@ -357,14 +144,19 @@ static int64_t max64(int64_t a, int64_t b) { return a > b ? a : b; }
 static scratch_sizes sizes_of(const layer_list_config *c, gd_dtype type, int64_t rows, int64_t max_new, int64_t kv_total,
                               int64_t max_seq)
 {
-    scratch_sizes s = {0, c->width, 1, c->width, 1, 256U};
+    scratch_sizes s = {0, c->width, 1, c->width, 1, 256U, 1, 1};
     int32_t i;
     for (i = 0; i < c->n_layers; ++i) {
         const layer_config *l = &c->layers[i];
-        s.proj = max64(s.proj, mixer_in(l));
+        s.proj = max64(s.proj, mixer_pitch(l));
         if (l->mixer == MIXER_MAMBA2) {
             s.a = max64(s.a, max64(conv_channels(l), inner_size(l)));
             s.b = max64(s.b, inner_size(l));
+        } else if (l->mixer == MIXER_GROUPED_ATTENTION) {
+            const size_t w = gd_backend_grouped_work_bytes(NULL, &l->grouped, (uint32_t)rows, (uint32_t)max_new,
+                                                           (uint32_t)max_seq, (uint32_t)type);
+            s.a = max64(s.a, mixer_out(l));
+            if (w > s.work) s.work = w;
         } else {
             const size_t w = gd_backend_latent_work_bytes(NULL, &l->latent, (uint32_t)rows, (uint32_t)max_new, (uint32_t)kv_total,
                                                           (uint32_t)max_seq, (uint32_t)type);
@@ -373,7 +165,12 @@ static scratch_sizes sizes_of(const layer_list_config *c, gd_dtype type, int64_t
             s.b = max64(s.b, query_size(l));
             if (w > s.work) s.work = w;
         }
-        s.a = max64(s.a, l->ff);
+        s.a = max64(s.a, max64(l->ff, l->shared_ff));
+        if (l->mlp == MLP_ROUTED) {
+            const int64_t packed = rows * l->routed.top + GD_BACKEND_ROUTED_PAD;
+            s.packed = max64(s.packed, packed * c->width);
+            s.packed_ff = max64(s.packed_ff, packed * l->routed.ff);
+        }
     }
     return s;
 }
@@ -383,7 +180,8 @@ static size_t forward_bytes(const layer_list_config *c, const scratch_sizes *s, 
     const size_t es = gd_dtype_size(type), R = (size_t)rows;
     return gd_pad256(R * (size_t)c->width * 4U) + gd_pad256(R * (size_t)c->width * es) + gd_pad256(R * (size_t)s->proj * es) +
            gd_pad256(R * (size_t)s->a * es) + gd_pad256(R * (size_t)s->b * es) + gd_pad256(R * (size_t)s->branch * es) +
-           gd_pad256(R * (size_t)s->angles * 4U) + gd_pad256(s->work);
+           gd_pad256(R * (size_t)s->angles * 4U) + gd_pad256(s->work) + 2U * gd_pad256((size_t)s->packed * es) +
+           gd_pad256((size_t)s->packed_ff * es);
 }
 
 typedef struct forward {
@@ -394,7 +192,12 @@ typedef struct forward {
     int64_t rows;
     gd_backend_packed_seqs seqs;
     gd_backend_tensor_view row_seq, cu, slot, start, kv_cu, ids;
-    gd_tensor x, h, proj, a, b, branch, angles, work; /* h: the copy of x, or x itself when the projections are F32 */
+    gd_tensor x, h, proj, a, b, branch, angles, work; /* h: what a sublayer reads; x itself when that is an F32 copy */
+    gd_tensor packed, packed_act, packed_out;         /* of the routed experts */
+    /* norms first: what waits to be added to the stream */
+    bool branch_waits;
+    layer_weights *routed_waits;
+    const layer_config *routed_config;
 } forward;
 
 static void view2(const gd_tensor *t, uint32_t dtype, int64_t d0, int64_t d1, gd_backend_tensor_view *v)
@@ -449,29 +252,50 @@ static gd_status forward_begin(forward *f, gd_gpt_decoder *d, int64_t rows, int6
     f->seqs.kv_cu = kv_total > 0 ? &f->kv_cu : NULL;
     f->seqs.kv_total = (uint32_t)kv_total;
     TRY(scratch(d->ctx, GD_DTYPE_F32, rows, ll->c.width, &f->x));
-    if (ll->type == GD_DTYPE_F32) f->h = f->x;
+    if (ll->type == GD_DTYPE_F32 && !ll->c.norms_first) f->h = f->x;
     else TRY(scratch(d->ctx, ll->type, rows, ll->c.width, &f->h));
     TRY(scratch(d->ctx, ll->type, rows, s.proj, &f->proj));
     TRY(scratch(d->ctx, ll->type, rows, s.a, &f->a));
     TRY(scratch(d->ctx, ll->type, rows, s.b, &f->b));
     TRY(scratch(d->ctx, GD_DTYPE_F32, rows, s.angles, &f->angles));
     TRY(scratch(d->ctx, ll->type, rows, s.branch, &f->branch));
+    TRY(scratch(d->ctx, ll->type, 1, s.packed, &f->packed));
+    TRY(scratch(d->ctx, ll->type, 1, s.packed_ff, &f->packed_act));
+    TRY(scratch(d->ctx, ll->type, 1, s.packed, &f->packed_out));
+    f->branch_waits = false;
+    f->routed_waits = NULL;
     return gd_tensor_empty(d->ctx, GD_ARENA_SCRATCH, GD_DTYPE_U8, gd_shape_make(1U, wdim), 256U, &f->work);
 }
 
-/* y [rows, w rows] = x [rows, w cols] w^T (+ bias), buffers holding packed rows */
+static bool epilogue_gated(uint32_t epilogue)
+{
+    return epilogue != 0U && epilogue != GD_BACKEND_EPILOGUE_SQUARE_RELU;
+}
+
+/* y [rows, outputs] = x [rows, w cols] w^T (+ bias) with the epilogue of args, buffers holding rows `pitch` apart
+ * (0: packed) */
+static gd_status project_as(forward *f, const gd_tensor *x, const gd_tensor *w, const gd_tensor *bias,
+                            gd_backend_fused_linear_args args, int64_t pitch, gd_tensor *y)
+{
+    const int64_t outs = epilogue_gated(args.epilogue) ? w->shape[0] / 2 : w->shape[0];
+    gd_backend_matrix_view xm, wm, ym;
+    gd_backend_vector_view bv;
+    args.w_is_nk = 1U;
+    args.bias_mode = bias != NULL ? 1U : 0U;
+    columns(x, f->type, f->rows, w->shape[1], 0, w->shape[1], &xm);
+    mview(w, w->shape[0], w->shape[1], &wm);
+    columns(y, f->type, f->rows, pitch > 0 ? pitch : outs, 0, outs, &ym);
+    if (bias != NULL) vview(bias, &bv);
+    return gd_backend_fused_linear(f->be, &xm, &wm, bias != NULL ? &bv : NULL, NULL, NULL, &ym, &args);
+}
+
 static gd_status project(forward *f, const gd_tensor *x, const gd_tensor *w, const gd_tensor *bias, uint32_t epilogue,
                          gd_tensor *y)
 {
-    const gd_backend_fused_linear_args args = {1U, bias != NULL ? 1U : 0U, 0U, 0.0f, epilogue};
-    const int64_t outs = epilogue != 0U ? w->shape[0] / 2 : w->shape[0];
-    gd_backend_matrix_view xm, wm, ym;
-    gd_backend_vector_view bv;
-    columns(x, f->type, f->rows, w->shape[1], 0, w->shape[1], &xm);
-    mview(w, w->shape[0], w->shape[1], &wm);
-    columns(y, f->type, f->rows, outs, 0, outs, &ym);
-    if (bias != NULL) vview(bias, &bv);
-    return gd_backend_fused_linear(f->be, &xm, &wm, bias != NULL ? &bv : NULL, NULL, NULL, &ym, &args);
+    gd_backend_fused_linear_args args;
+    memset(&args, 0, sizeof(args));
+    args.epilogue = epilogue;
+    return project_as(f, x, w, bias, args, 0, y);
 }
 
 /* x += m * norm(branch), h = x */
@@ -543,25 +367,174 @@ static gd_status latent_attention(forward *f, const layer_config *l, layer_weigh
     return project(f, &f->a, &w->out, NULL, 0U, &f->branch);
 }
 
-/* every layer over the rows of f, from the token ids to the residual stream in f->x */
-static gd_status run_layers(forward *f)
+static gd_status grouped_attention(forward *f, const layer_config *l, layer_weights *w)
 {
-    const int64_t W = f->ll->c.width;
-    gd_backend_tensor_view ve, vx, vh;
+    const gd_backend_fused_linear_args plain = {0U, 0U, 0U, 0.0f, 0U, 0.0f, 0.0f};
+    gd_backend_matrix_view pm;
+    gd_backend_tensor_view freq, kc, vc, work, out;
+    TRY(project_as(f, &f->h, &w->in, NULL, plain, mixer_pitch(l), &f->proj));
+    columns(&f->proj, f->type, f->rows, mixer_pitch(l), 0, mixer_in(l), &pm);
+    tview(&w->freq, &freq);
+    tview(&w->k_cache, &kc);
+    tview(&w->v_cache, &vc);
+    tview(&f->work, &work);
+    view2(&f->a, f->type, f->rows, mixer_out(l), &out);
+    TRY(gd_backend_grouped_attend(f->be, &pm, &freq, &kc, &vc, &work, &out, &f->seqs, &l->grouped));
+    return project(f, &f->a, &w->out, NULL, 0U, &f->branch);
+}
+
+static gd_status mixer(forward *f, const layer_config *l, layer_weights *w)
+{
+    if (l->mixer == MIXER_MAMBA2) return mamba2(f, l, w);
+    if (l->mixer == MIXER_LATENT_ATTENTION) return latent_attention(f, l, w);
+    return grouped_attention(f, l, w);
+}
+
+/* the step's tables of a routed layer (its weights' owner holds them) and, packed by expert, a buffer's rows */
+static void routes_of(const forward *f, const layer_config *l, const layer_weights *w, gd_backend_tensor_view *place,
+                      gd_backend_tensor_view *first, gd_backend_tensor_view *tiles)
+{
+    tview(&w->place, place);
+    tview(&w->first, first);
+    tview(&w->tiles, tiles);
+    place->shape[0] = f->rows * l->routed.top;
+    place->count = (size_t)place->shape[0];
+}
+
+static void packed_rows(const forward *f, const layer_config *l, const gd_tensor *t, int64_t cols, gd_backend_tensor_view *v)
+{
+    view2(t, f->type, f->rows * l->routed.top + GD_BACKEND_ROUTED_PAD, cols, v);
+}
+
+/* which rows go to which expert, for every table of the model: the token ids alone decide */
+static gd_status route(forward *f)
+{
+    enum { BATCH = 64 };
+    gd_backend_route_job jobs[BATCH];
+    gd_backend_tensor_view table[BATCH], place[BATCH], first[BATCH], tiles[BATCH];
+    uint32_t n = 0U;
     int32_t i;
-    tview(&f->ll->embed, &ve);
-    view2(&f->x, GD_BACKEND_DTYPE_F32, f->rows, W, &vx);
-    view2(&f->h, f->type, f->rows, W, &vh);
-    TRY(gd_backend_residual_embed(f->be, &ve, &f->ids, &vx, f->ll->type == GD_DTYPE_F32 ? NULL : &vh,
-                                  f->ll->c.embedding_scale));
     for (i = 0; i < f->ll->c.n_layers; ++i) {
         const layer_config *l = &f->ll->c.layers[i];
         layer_weights *w = &f->ll->layers[i];
-        if (l->mixer == MIXER_MAMBA2) TRY(mamba2(f, l, w));
-        else TRY(latent_attention(f, l, w));
+        if (l->mlp != MLP_ROUTED || l->weights_of != i) continue;
+        tview(&w->table, &table[n]);
+        routes_of(f, l, w, &place[n], &first[n], &tiles[n]);
+        jobs[n].table = &table[n];
+        jobs[n].place = &place[n];
+        jobs[n].first = &first[n];
+        jobs[n].tiles = &tiles[n];
+        jobs[n].args = &l->routed;
+        if (++n < BATCH) continue;
+        TRY(gd_backend_route_by_tables(f->be, jobs, n, &f->ids, f->type));
+        n = 0U;
+    }
+    return n > 0U ? gd_backend_route_by_tables(f->be, jobs, n, &f->ids, f->type) : GD_OK;
+}
+
+/* x += what waits;  h = norm(x) * weight (NULL: only the sum);  rows of a routed feed-forward that follows are packed */
+static gd_status settle_stream(forward *f, const gd_tensor *norm, const layer_config *next, layer_weights *next_w,
+                               gd_tensor *h)
+{
+    const int64_t W = f->ll->c.width;
+    gd_backend_tensor_view vb, vn, vx, vh, place_in, place_out, first, tiles, rows_in, rows_out;
+    gd_backend_routed_rows in, out;
+    view2(&f->branch, f->type, f->rows, W, &vb);
+    view2(&f->x, GD_BACKEND_DTYPE_F32, f->rows, W, &vx);
+    view2(h, f->type, f->rows, W, &vh);
+    if (norm != NULL) tview(norm, &vn);
+    if (f->routed_waits != NULL) {
+        routes_of(f, f->routed_config, f->routed_waits, &place_in, &first, &tiles);
+        packed_rows(f, f->routed_config, &f->packed_out, W, &rows_in);
+        in.rows = &rows_in;
+        in.place = &place_in;
+        in.top = f->routed_config->routed.top;
+        in.weight = f->routed_config->routed.weight;
+    }
+    if (next != NULL) {
+        routes_of(f, next, next_w, &place_out, &first, &tiles);
+        packed_rows(f, next, &f->packed, W, &rows_out);
+        out.rows = &rows_out;
+        out.place = &place_out;
+        out.top = next->routed.top;
+        out.weight = 1.0f;
+    }
+    TRY(gd_backend_residual_add_norm(f->be, f->branch_waits ? &vb : NULL, f->routed_waits != NULL ? &in : NULL, &vx,
+                                     norm != NULL ? &vn : NULL, norm != NULL ? &vh : NULL, next != NULL ? &out : NULL,
+                                     f->ll->c.eps));
+    f->branch_waits = false;
+    f->routed_waits = NULL;
+    return GD_OK;
+}
+
+static gd_status square_relu(forward *f, layer_weights *w)
+{
+    TRY(project(f, &f->h, &w->upgate, NULL, GD_BACKEND_EPILOGUE_SQUARE_RELU, &f->a));
+    f->branch_waits = true;
+    return project(f, &f->a, &w->down, NULL, 0U, &f->branch);
+}
+
+/* the packed rows (settle_stream) through their experts, and all rows through the shared one */
+static gd_status routed(forward *f, const layer_config *l, layer_weights *w)
+{
+    gd_backend_tensor_view rows, act, out, up, down, place, first, tiles;
+    gd_backend_routes routes;
+    routes_of(f, l, w, &place, &first, &tiles);
+    packed_rows(f, l, &f->packed, l->routed.width, &rows);
+    packed_rows(f, l, &f->packed_act, l->routed.ff, &act);
+    packed_rows(f, l, &f->packed_out, l->routed.width, &out);
+    tview(&w->expert_upgate, &up);
+    tview(&w->expert_down, &down);
+    routes.first = &first;
+    routes.tiles = &tiles;
+    routes.rows = (uint32_t)f->rows;
+    TRY(gd_backend_routed_mlp(f->be, &rows, &up, &down, &act, &out, &routes, &l->routed));
+    f->routed_waits = w;
+    f->routed_config = l;
+    if (l->shared_ff > 0) {
+        const gd_backend_fused_linear_args gate = {0U, 0U, 0U, 0.0f, GD_BACKEND_EPILOGUE_CLAMPED_GATE, l->shared_limit,
+                                                   l->routed.gate_alpha};
+        TRY(project_as(f, &f->h, &w->upgate, NULL, gate, 0, &f->a));
+        TRY(project(f, &f->a, &w->down, NULL, 0U, &f->branch));
+        f->branch_waits = true;
+    }
+    return GD_OK;
+}
+
+/* Norms in front of the sublayers.  all_normed: the last norm of every row is left in f->h; otherwise only the stream
+ * is complete. */
+static gd_status run_norms_first(forward *f, bool all_normed)
+{
+    const layer_list_config *c = &f->ll->c;
+    int32_t i;
+    TRY(route(f));
+    TRY(settle_stream(f, &f->ll->layers[0].norm1, NULL, NULL, &f->h));
+    for (i = 0; i < c->n_layers; ++i) {
+        const layer_config *l = &c->layers[i];
+        layer_weights *w = &f->ll->layers[i], *owner = &f->ll->layers[l->weights_of];
+        const bool last = i + 1 == c->n_layers;
+        TRY(mixer(f, l, w));
+        f->branch_waits = true;
+        if (l->mlp != MLP_NONE) {
+            TRY(settle_stream(f, &w->norm2, l->mlp == MLP_ROUTED ? l : NULL, owner, &f->h));
+            if (l->mlp == MLP_ROUTED) TRY(routed(f, l, owner));
+            else TRY(square_relu(f, w));
+        }
+        TRY(settle_stream(f, !last ? &f->ll->layers[i + 1].norm1 : all_normed ? &f->ll->final_norm : NULL, NULL, NULL, &f->h));
+    }
+    return GD_OK;
+}
+
+static gd_status run_norms_behind(forward *f)
+{
+    int32_t i;
+    for (i = 0; i < f->ll->c.n_layers; ++i) {
+        const layer_config *l = &f->ll->c.layers[i];
+        layer_weights *w = &f->ll->layers[i];
+        TRY(mixer(f, l, w));
         TRY(add_branch(f, &w->norm1));
-        if (l->ff > 0) {
-            TRY(project(f, &f->h, &w->upgate, &w->upgate_b, 2U, &f->a));
+        if (l->mlp == MLP_GELU_GATED) {
+            TRY(project(f, &f->h, &w->upgate, &w->upgate_b, GD_BACKEND_EPILOGUE_GELU_GATE, &f->a));
             TRY(project(f, &f->a, &w->down, &w->down_b, 0U, &f->branch));
             TRY(add_branch(f, &w->norm2));
         }
@@ -569,21 +542,37 @@ static gd_status run_layers(forward *f)
     return GD_OK;
 }
 
-/* F32 logits of the picked rows (NULL: of all rows) */
-static gd_status head(forward *f, const gd_backend_tensor_view *rows, int64_t n, gd_tensor *logits)
+/* every layer over the rows of f, from the token ids to the residual stream in f->x (see run_norms_first) */
+static gd_status run_layers(forward *f, bool all_normed)
+{
+    const int64_t W = f->ll->c.width;
+    const bool copy = !f->ll->c.norms_first && f->ll->type != GD_DTYPE_F32;
+    gd_backend_tensor_view ve, vx, vh;
+    tview(&f->ll->embed, &ve);
+    view2(&f->x, GD_BACKEND_DTYPE_F32, f->rows, W, &vx);
+    view2(&f->h, f->type, f->rows, W, &vh);
+    TRY(gd_backend_residual_embed(f->be, &ve, &f->ids, &vx, copy ? &vh : NULL, f->ll->c.embedding_scale));
+    return f->ll->c.norms_first ? run_norms_first(f, all_normed) : run_norms_behind(f);
+}
+
+/* F32 logits of the picked rows (NULL: of all rows, whose last norm may already be in f->h) */
+static gd_status head(forward *f, const gd_backend_tensor_view *rows, int64_t n, bool normed, gd_tensor *logits)
 {
     const layer_list_config *c = &f->ll->c;
+    const gd_tensor *weight = c->own_head ? &f->ll->head : &f->ll->embed;
     gd_backend_tensor_view vx, vn, vo;
     gd_backend_matrix_view xm, wm, ym;
-    gd_tensor normed;
-    TRY(scratch(f->d->ctx, f->ll->type, n, c->width, &normed));
+    gd_tensor last = f->h;
     TRY(scratch(f->d->ctx, GD_DTYPE_F32, n, c->vocab, logits));
-    view2(&f->x, GD_BACKEND_DTYPE_F32, f->rows, c->width, &vx);
-    tview(&f->ll->final_norm, &vn);
-    tview(&normed, &vo);
-    TRY(gd_backend_residual_norm_rows(f->be, &vx, rows, &vn, &vo, c->eps));
-    mview(&normed, n, c->width, &xm);
-    mview(&f->ll->embed, c->vocab, c->width, &wm);
+    if (!normed) {
+        TRY(scratch(f->d->ctx, f->ll->type, n, c->width, &last));
+        view2(&f->x, GD_BACKEND_DTYPE_F32, f->rows, c->width, &vx);
+        tview(&f->ll->final_norm, &vn);
+        tview(&last, &vo);
+        TRY(gd_backend_residual_norm_rows(f->be, &vx, rows, &vn, &vo, c->eps));
+    }
+    mview(&last, n, c->width, &xm);
+    mview(weight, c->vocab, c->width, &wm);
     mview(logits, n, c->vocab, &ym);
     return gd_backend_matmul_nt(f->be, &xm, &wm, &ym);
 }
@@ -599,8 +588,8 @@ static gd_status layer_list_step(gd_gpt_decoder *d, const gd_tensor *ids, const 
     view1(&d->layers->rows_dev, &f.slot);
     view1(&d->layers->cu_dev, &f.cu);
     view1(positions, &f.start);
-    TRY(run_layers(&f));
-    return head(&f, NULL, f.rows, logits);
+    TRY(run_layers(&f, true));
+    return head(&f, NULL, f.rows, d->layers->c.norms_first, logits);
 }
 
 static gd_status layer_list_extend(gd_gpt_decoder *d, const gd_extend_rows *e, gd_tensor *logits)
@@ -646,10 +635,10 @@ static gd_status layer_list_extend(gd_gpt_decoder *d, const gd_extend_rows *e, g
     view1(&part[SLOT], &f.slot);
     view1(&part[START], &f.start);
     view1(&part[KV_CU], &f.kv_cu);
-    TRY(run_layers(&f));
+    TRY(run_layers(&f, false));
     if (e->n_want == 0) return GD_OK;
     view1(&part[WANT], &want);
-    return head(&f, &want, e->n_want, logits);
+    return head(&f, &want, e->n_want, false, logits);
 }
 
 static gd_status layer_list_prefill(gd_gpt_decoder *d, const int32_t *ids, const int32_t *cu, gd_tensor *logits)
@@ -698,10 +687,15 @@ static gd_tensor *layer_list_tensor(gd_gpt_decoder *d, const char *name, int32_t
     struct layer_list *ll = d->layers;
     layer_weights *w;
     if (!strcmp(name, "embed")) return &ll->embed;
+    if (!strcmp(name, "head") && ll->c.own_head) return &ll->head;
     if (!strcmp(name, "final_norm")) return &ll->final_norm;
     if (layer < 0 || layer >= ll->c.n_layers) return NULL;
     w = &ll->layers[layer];
     if (!strcmp(name, "cache") && ll->c.layers[layer].mixer == MIXER_LATENT_ATTENTION) return &w->cache;
+    if (ll->c.layers[layer].mixer == MIXER_GROUPED_ATTENTION) {
+        if (!strcmp(name, "k_cache")) return &w->k_cache;
+        if (!strcmp(name, "v_cache")) return &w->v_cache;
+    }
     if (!strcmp(name, "states") && ll->c.layers[layer].mixer == MIXER_MAMBA2) return &w->states;
     if (!strcmp(name, "conv_ring") && ll->c.layers[layer].mixer == MIXER_MAMBA2) return &w->ring;
     return NULL;
@@ -715,9 +709,19 @@ static void layer_list_destroy(gd_gpt_decoder *d)
     free(d->layers);
 }
 
-static const gd_decoder_model layer_list_model = {"Girirax", layer_list_prefill, layer_list_step, layer_list_extend,
-                                                  layer_list_can_fuse, layer_list_feeds_x0, layer_list_tensor,
-                                                  layer_list_destroy};
+#define LAYER_LIST_MODEL(name)                                                                                         \
+    {name, layer_list_prefill, layer_list_step, layer_list_extend, layer_list_can_fuse, layer_list_feeds_x0,           \
+     layer_list_tensor, layer_list_destroy}
+static const gd_decoder_model layer_list_models[] = {LAYER_LIST_MODEL("Girirax"), LAYER_LIST_MODEL("Bonatar")};
+
+static const gd_decoder_model *model_of(const layer_list_config *c)
+{
+    size_t i;
+    for (i = 0U; i < sizeof(layer_list_models) / sizeof(layer_list_models[0]); ++i) {
+        if (!strcmp(layer_list_models[i].architecture, c->architecture)) return &layer_list_models[i];
+    }
+    return NULL;
+}
 
 /* the options with their defaults filled in, and what the session keeps of the configuration */
 static gd_status settle(const layer_list_config *c, const gd_model_options *in, gd_model_options *o, gd_gpt_config *g)
@@ -738,7 +742,7 @@ static gd_status settle(const layer_list_config *c, const gd_model_options *in, 
     g->n_layers = c->n_layers;
     g->max_seq = o->max_seq;
     g->batch = o->batch;
-    g->tie_lm_head = 1;
+    g->tie_lm_head = c->own_head ? 0 : 1;
     return GD_OK;
 }
 
@@ -753,16 +757,15 @@ gd_status gd_layer_list_memory(const layer_list_config *c, const gd_model_option
 {
     gd_model_options o;
     gd_gpt_config g;
-    size_t params = 0U, rows, logit_rows, step;
+    size_t rows, logit_rows, step;
     scratch_sizes s;
     TRY(settle(c, in, &o, &g));
-    TRY(each_weight(c, o.compute, NULL, add_bytes, &params));
     rows = (size_t)o.max_step_tokens;
     logit_rows = ((size_t)1 << 30) / ((size_t)c->vocab * 4U);
     if (logit_rows > rows) logit_rows = rows;
     *out = gd_memory_config_default();
-    out->params_bytes = params + 4096U;
-    out->state_bytes = state_bytes(c, o.compute, o.batch, o.max_seq) + gd_decoder_session_bytes(&g, GD_DTYPE_F32, false) + 4096U;
+    out->params_bytes = gd_layer_list_weight_bytes(c, o.compute) + 4096U;
+    out->state_bytes = state_bytes(c, o.compute, o.batch, o.max_seq, o.max_step_tokens) + gd_decoder_session_bytes(&g, GD_DTYPE_F32, false) + 4096U;
     /* a resident session holds an eager step and a captured one, its records besides; logits of every row of a step,
      * up to 1 GiB of them */
     /* the largest step: every form attention may take with that many rows */
@@ -803,7 +806,8 @@ gd_status gd_layer_list_create(gd_context *ctx, const layer_list_config *c, cons
     gd_status st;
     *out = NULL;
     TRY(settle(c, in, &o, &g));
-    TRY(gd_decoder_session_create(ctx, &layer_list_model, &g, &d));
+    if (model_of(c) == NULL) return GD_ERR_UNSUPPORTED;
+    TRY(gd_decoder_session_create(ctx, model_of(c), &g, &d));
     d->layers = ll = (struct layer_list *)calloc(1, sizeof(*ll));
     st = ll == NULL ? GD_ERR_OUT_OF_MEMORY : copy_config(c, &ll->c);
     if (st == GD_OK) {
@@ -813,7 +817,7 @@ gd_status gd_layer_list_create(gd_context *ctx, const layer_list_config *c, cons
         ll->layers = (layer_weights *)calloc((size_t)c->n_layers, sizeof(layer_weights));
         if (ll->layers == NULL) st = GD_ERR_OUT_OF_MEMORY;
     }
-    if (st == GD_OK) st = load_weights(ctx, ll, weights, seed);
+    if (st == GD_OK) st = gd_layer_list_load(ctx, ll, weights, seed);
     if (st == GD_OK) st = allocate_states(ctx, ll, o.batch, o.max_seq);
     if (st == GD_OK) st = gd_decoder_session_allocate(d, GD_DTYPE_F32, false);
     if (st != GD_OK) {

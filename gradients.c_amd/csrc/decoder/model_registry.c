@@ -75,9 +75,14 @@ static gd_status gpt_create(gd_context *ctx, gd_model *m, const gd_model_options
 
 /* ---- layer lists ------------------------------------------------------------------------------------- */
 
-static gd_status layers_configure(gd_model *m, const gd_json *root, char *message, size_t size)
+static gd_status girirax_configure(gd_model *m, const gd_json *root, char *message, size_t size)
 {
-    return gd_layer_list_parse(root, &m->layers, message, size);
+    return gd_layer_list_parse_girirax(root, &m->layers, message, size);
+}
+
+static gd_status bonatar_configure(gd_model *m, const gd_json *root, char *message, size_t size)
+{
+    return gd_layer_list_parse_bonatar(root, &m->layers, message, size);
 }
 
 static gd_status layers_memory(const gd_model *m, const gd_model_options *o, gd_memory_config *out)
@@ -92,7 +97,8 @@ static gd_status layers_create(gd_context *ctx, gd_model *m, const gd_model_opti
 
 static const architecture architectures[] = {
     {"gpt_lm", NULL, gpt_memory, gpt_create},
-    {"Girirax", layers_configure, layers_memory, layers_create},
+    {"Girirax", girirax_configure, layers_memory, layers_create},
+    {"Bonatar", bonatar_configure, layers_memory, layers_create},
 };
 
 /* ---- opening ------------------------------------------------------------------------------------------- */

@@ -21,8 +21,10 @@ int gd_hip_launch_linear_f32(hipStream_t stream, const void *x, const void *w, c
 static gd_status project_full(gd_backend *backend, const gd_backend_matrix_view *x, const gd_backend_matrix_view *w,
                               const gd_backend_vector_view *bias, const gd_backend_matrix_view *residual,
                               const gd_backend_vector_view *norm_w, float eps, const gd_backend_matrix_view *y,
-                              uint32_t w_is_nk, uint32_t epilogue, uint32_t prologue, uint32_t gated)
+                              uint32_t w_is_nk, uint32_t epilogue, uint32_t prologue, uint32_t activation,
+                              float gate_limit, float gate_alpha)
 {
+    const uint32_t gated = activation == GD_BACKEND_EPILOGUE_SQUARE_RELU ? 0u : activation;
     gd_hip_linear_params p;
     uint32_t K, es;
     int vec, kn_vec, store_vec, f16;
@@ -32,7 +34,7 @@ static gd_status project_full(gd_backend *backend, const gd_backend_matrix_view 
         return GD_ERR_INVALID_ARGUMENT;
     f16 = x->dtype == GD_BACKEND_DTYPE_F16;
     if ((!f16 && x->dtype != GD_BACKEND_DTYPE_BF16 && x->dtype != GD_BACKEND_DTYPE_F32) || w->dtype != x->dtype ||
-        (y->dtype != x->dtype && !(x->dtype == GD_BACKEND_DTYPE_BF16 && y->dtype == GD_BACKEND_DTYPE_F32 && !gated)) ||
+        (y->dtype != x->dtype && !(x->dtype == GD_BACKEND_DTYPE_BF16 && y->dtype == GD_BACKEND_DTYPE_F32 && activation == 0u)) ||
         (bias != NULL && bias->dtype != x->dtype) || (residual != NULL && residual->dtype != x->dtype) ||
         (norm_w != NULL && norm_w->dtype != x->dtype))
         return GD_ERR_UNSUPPORTED;
@@ -40,7 +42,7 @@ static gd_status project_full(gd_backend *backend, const gd_backend_matrix_view 
     if (!f16 && (!w_is_nk || prologue != GD_HIP_PRO_NONE || residual != NULL ||
                  (bias != NULL && epilogue != GD_HIP_EPI_BIAS_F32)))
         return GD_ERR_UNSUPPORTED;
-    if (f16 && gated > 1u) return GD_ERR_UNSUPPORTED;
+    if (f16 && activation > GD_BACKEND_EPILOGUE_SILU_GATE) return GD_ERR_UNSUPPORTED;
     es = (uint32_t)gd_hip_dtype_size(x->dtype);
     if (prologue == GD_HIP_PRO_SWIGLU) {
         if ((x->cols & 1u) != 0u) return GD_ERR_INVALID_ARGUMENT;
@@ -82,7 +84,13 @@ static gd_status project_full(gd_backend *backend, const gd_backend_matrix_view 
     p.force_waves = (uint16_t)backend->linear_waves;
     p.no_lds_stream = (uint16_t)(backend->linear_no_lds_stream != 0);
     p.flags = 0u;
-    if (gated == 2u) p.flags |= GD_HIP_LINEAR_GELU_GATE;
+    if (activation == GD_BACKEND_EPILOGUE_GELU_GATE) p.flags |= GD_HIP_LINEAR_GELU_GATE;
+    if (activation == GD_BACKEND_EPILOGUE_SQUARE_RELU) p.flags |= GD_HIP_LINEAR_SQUARE_RELU;
+    if (activation == GD_BACKEND_EPILOGUE_CLAMPED_GATE) {
+        p.flags |= GD_HIP_LINEAR_CLAMPED_GATE;
+        p.gate_limit = gate_limit;
+        p.gate_alpha = gate_alpha;
+    }
     if (y->dtype != x->dtype) p.flags |= GD_HIP_LINEAR_Y_F32;
     if (x->dtype == GD_BACKEND_DTYPE_F32) {
         backend->last_linear_family = GD_HIP_LINEAR_FAMILY_F32;
@@ -109,7 +117,7 @@ static gd_status project(gd_backend *backend, const gd_backend_matrix_view *x, c
                          uint32_t epilogue, uint32_t swiglu)
 {
     return project_full(backend, x, w, bias, NULL, NULL, 0.0f, y, w_is_nk, epilogue,
-                        swiglu ? GD_HIP_PRO_SWIGLU : GD_HIP_PRO_NONE, 0u);
+                        swiglu ? GD_HIP_PRO_SWIGLU : GD_HIP_PRO_NONE, 0u, 0.0f, 0.0f);
 }
 
 gd_status gd_backend_matmul(gd_backend *backend, const gd_backend_matrix_view *x, const gd_backend_matrix_view *w,
@@ -150,11 +158,11 @@ gd_status gd_backend_fused_linear(gd_backend *backend, const gd_backend_matrix_v
                                   const gd_backend_matrix_view *residual, const gd_backend_vector_view *norm_weight,
                                   const gd_backend_matrix_view *y, const gd_backend_fused_linear_args *args)
 {
-    if (args == NULL || args->bias_mode > 2u || args->prologue > 2u || args->epilogue > 2u ||
+    if (args == NULL || args->bias_mode > 2u || args->prologue > 2u || args->epilogue > 4u ||
         (args->bias_mode != 0u) != (bias != NULL))
         return GD_ERR_INVALID_ARGUMENT;
     return project_full(backend, x, w, bias, residual, norm_weight, args->eps, y, args->w_is_nk != 0u, args->bias_mode,
-                        args->prologue, args->epilogue);
+                        args->prologue, args->epilogue, args->gate_limit, args->gate_alpha);
 }
 
 #include <math.h>

@@ -15,6 +15,8 @@
 /* flags */
 #define GD_HIP_LINEAR_GELU_GATE 1u /* swiglu_cols: the gate function is gelu (tanh form) instead of silu */
 #define GD_HIP_LINEAR_Y_F32 2u     /* y is F32 (BF16 operands) */
+#define GD_HIP_LINEAR_CLAMPED_GATE 4u /* swiglu_cols: g sigmoid(gate_alpha g) (v + 1), both kept within gate_limit */
+#define GD_HIP_LINEAR_SQUARE_RELU 8u  /* not gated: y = max(u, 0)^2 */
 
 typedef struct gd_hip_linear_params {
     uint32_t M, N, K;
@@ -24,13 +26,19 @@ typedef struct gd_hip_linear_params {
     uint32_t prologue;
     uint32_t has_residual;  /* 1: y = half(epilogue(acc)) + residual, residual [M,N] pitch ldr */
     uint32_t ldr;
-    float eps;              /* rms_norm prologue */
+    union {
+        float eps;          /* rms_norm prologue */
+        float gate_limit;   /* GD_HIP_LINEAR_CLAMPED_GATE */
+    };
     uint32_t swiglu_cols;   /* 0, or H: w has 2H rows ([N,K] only); y [M,H] = half(u[:, :H] * silu(u[:, H:])) where u is
                              * the projection after the bias epilogue, rounded to F16 like a stored intermediate */
     /* rope + cache append epilogue (rope_head_dim != 0): the projection is the qkv projection of a decode step,
      * N = 3 * heads * head_dim; see gd_hip_rope_epilogue */
     uint32_t rope_heads, rope_head_dim, rope_tmax;
-    float rope_freq_scale;
+    union {
+        float rope_freq_scale;
+        float gate_alpha; /* GD_HIP_LINEAR_CLAMPED_GATE */
+    };
     /* The few-row kernel reads its arguments in one batch at entry: six pointers, this structure and the tile count
      * behind it fill exactly one 128-byte line of the argument segment.  Keep the structure at 76 bytes: with the
      * tile count on a second line every projection launch of a decode step took 0.06 us longer. */

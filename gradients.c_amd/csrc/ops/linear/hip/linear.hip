@@ -48,8 +48,9 @@ gd_linear_scalar_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict
             const gd_elem *gr = w + (size_t)(p.swiglu_cols + n) * p.ldw;
             for (uint32_t k = 0; k < p.K; ++k) g = fmaf((float)xr[k], (float)gr[k], g);
             if (p.epilogue == GD_HIP_EPI_BIAS_F32) g += (float)bias[p.swiglu_cols + n];
-            v = gd_lin_gated(v, g, p.flags);
+            v = gd_lin_gated(v, g, p);
         }
+        v = gd_lin_activated(v, p.flags);
         if (p.flags & GD_HIP_LINEAR_Y_F32) reinterpret_cast<float *>(y)[(size_t)m * p.ldy + n] = v;
         else y[(size_t)m * p.ldy + n] = (gd_elem)v;
         return;

@@ -5,7 +5,8 @@
  * layout, so nothing else differs, except that the BF16 build
  *   - instantiates only what its callers use: [N,K] weights, no prologue, no rotation epilogue;
  *   - keeps a gated projection in F32 up to the product with the gate (the F16 build rounds value and gate first,
- *     as the reference's separate operators do), and knows a second gate function (GD_HIP_LINEAR_GELU_GATE);
+ *     as the reference's separate operators do), and knows further gate functions (GD_HIP_LINEAR_GELU_GATE,
+ *     GD_HIP_LINEAR_CLAMPED_GATE) and the square of relu (GD_HIP_LINEAR_SQUARE_RELU);
  *   - can store F32 results (GD_HIP_LINEAR_Y_F32; few-row kernels only).
  */
 #ifndef GD_LINEAR_ELEM_H
@@ -31,11 +32,26 @@ typedef gd_half4 gd_elem4;
 #endif
 
 #if GD_LINEAR_IS_BF16
-/* value * gate function of a gated projection, both still F32 */
-__device__ __forceinline__ float gd_lin_gated(float value, float gate, uint32_t flags)
+/* g sigmoid(alpha g) (v + 1), g = min(gate, limit), v = value kept within +-limit; the result is rounded to 16 bits */
+__device__ __forceinline__ float gd_lin_clamped_gate(float value, float gate, float limit, float alpha)
 {
-    if (flags & GD_HIP_LINEAR_GELU_GATE) return value * gd_gelu_tanh_f32(gate);
+    const float g = fminf(gate, limit), v = fminf(fmaxf(value, -limit), limit);
+    return g * gd_sigmoid_fast(alpha * g) * (v + 1.0f);
+}
+
+/* value * gate function of a gated projection, both still F32 */
+__device__ __forceinline__ float gd_lin_gated(float value, float gate, const gd_hip_linear_params &p)
+{
+    if (p.flags & GD_HIP_LINEAR_CLAMPED_GATE) return gd_lin_clamped_gate(value, gate, p.gate_limit, p.gate_alpha);
+    if (p.flags & GD_HIP_LINEAR_GELU_GATE) return value * gd_gelu_tanh_f32(gate);
     return value * gd_silu_f32(gate);
+}
+
+/* what becomes of an output that is not gated */
+__device__ __forceinline__ float gd_lin_activated(float u, uint32_t flags)
+{
+    if (flags & GD_HIP_LINEAR_SQUARE_RELU) return u > 0.f ? u * u : 0.f;
+    return u;
 }
 #endif
 

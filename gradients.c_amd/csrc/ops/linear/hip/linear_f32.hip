@@ -52,10 +52,14 @@ gd_linear_f32_kernel(const float *__restrict__ x, const float *__restrict__ w, c
             if (GATED) {
                 const float g = acc[GATED ? 1 : 0][i][j] + (p.epilogue != GD_HIP_EPI_NONE ? bias[p.swiglu_cols + n] : 0.f);
                 /* the accurate functions: this path is held to 32-bit rounding */
-                if (p.flags & GD_HIP_LINEAR_GELU_GATE)
+                if (p.flags & GD_HIP_LINEAR_CLAMPED_GATE) {
+                    const float c = fminf(g, p.gate_limit);
+                    v = c / (1.0f + expf(-p.gate_alpha * c)) * (fminf(fmaxf(v, -p.gate_limit), p.gate_limit) + 1.0f);
+                } else if (p.flags & GD_HIP_LINEAR_GELU_GATE)
                     v *= 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
                 else v *= g / (1.0f + expf(-g));
             }
+            if (!GATED && (p.flags & GD_HIP_LINEAR_SQUARE_RELU)) v = v > 0.f ? v * v : 0.f;
             y[(size_t)m * p.ldy + n] = v;
         }
     }

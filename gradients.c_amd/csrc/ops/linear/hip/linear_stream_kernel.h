@@ -422,7 +422,7 @@ gd_linear_stream_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict
                     v1 += (float)pf_b1[i];
                     v2 += (float)pf_b2[i];
                 }
-                y[(size_t)row * p.ldy + col] = (gd_elem)gd_lin_gated(v1, v2, p.flags);
+                y[(size_t)row * p.ldy + col] = (gd_elem)gd_lin_gated(v1, v2, p);
                 continue;
 #endif
                 gd_elem h1, h2;
@@ -483,6 +483,11 @@ gd_linear_stream_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict
             if (p.flags & GD_HIP_LINEAR_Y_F32) {
                 if (p.epilogue == GD_HIP_EPI_BIAS_F32) v += (float)pf_b1[i];
                 reinterpret_cast<float *>(y)[(size_t)row * p.ldy + col] = v;
+                continue;
+            }
+            if (p.flags & GD_HIP_LINEAR_SQUARE_RELU) {
+                if (p.epilogue == GD_HIP_EPI_BIAS_F32) v += (float)pf_b1[i];
+                y[(size_t)row * p.ldy + col] = (gd_elem)gd_lin_activated(v, p.flags);
                 continue;
             }
 #endif

@@ -98,15 +98,17 @@ __device__ __forceinline__ float gd_tile_silu(float z)
     return z * (z >= 0.0f ? inv : e * inv);
 }
 
-__device__ __forceinline__ float gd_tile_gated(float value, float gate, uint32_t flags)
+__device__ __forceinline__ float gd_tile_gated(float value, float gate, const gd_hip_linear_params &p)
 {
 #if GD_LINEAR_IS_BF16
-    if (flags & GD_HIP_LINEAR_GELU_GATE) {
+    if (p.flags & GD_HIP_LINEAR_CLAMPED_GATE) return gd_lin_clamped_gate(value, gate, p.gate_limit, p.gate_alpha);
+    if (p.flags & GD_HIP_LINEAR_GELU_GATE) {
         const float u = 2.0f * 0.7978845608028654f * (gate + 0.044715f * gate * gate * gate);
         const float e = __expf(-fabsf(u)), inv = __builtin_amdgcn_rcpf(1.0f + e);
         return value * gate * (u >= 0.0f ? inv : e * inv);
     }
 #endif
+    (void)p;
     return value * gd_tile_silu(gate);
 }
 
@@ -491,6 +493,12 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const float v = a[4 * q + r];
+#if GD_LINEAR_IS_BF16
+            if (p.flags & GD_HIP_LINEAR_SQUARE_RELU) {
+                h[r] = (gd_elem)gd_lin_activated(MODE == GD_HIP_EPI_BIAS_F32 ? v + (float)bq[j][q][r] : v, p.flags);
+                continue;
+            }
+#endif
             if (MODE == GD_HIP_EPI_NONE) h[r] = (gd_elem)v;
             else if (MODE == GD_HIP_EPI_BIAS_F32) h[r] = (gd_elem)(v + (float)bq[j][q][r]);
             else h[r] = (gd_elem)v + bq[j][q][r];
@@ -536,7 +544,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
                 const gd_elem8 hv = read_chunk(er, cv), hg = read_chunk(er, cv + HW / 8u);
                 gd_elem8 h;
 #pragma unroll
-                for (int t = 0; t < 8; ++t) h[t] = (gd_elem)gd_tile_gated((float)hv[t], (float)hg[t], p.flags);
+                for (int t = 0; t < 8; ++t) h[t] = (gd_elem)gd_tile_gated((float)hv[t], (float)hg[t], p);
                 gd_elem *yr = y + (size_t)gr * p.ldy + gc;
                 if (vector_store && gc + 8u <= p.N) {
                     *reinterpret_cast<gd_elem8 *>(yr) = h;
@@ -677,7 +685,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
                                 fv += (float)bq[j][q][t];
                                 fg += (float)bq[j + WN / 2][q][t];
                             }
-                            o[s2][t] = (gd_elem)gd_tile_gated(fv, fg, p.flags);
+                            o[s2][t] = (gd_elem)gd_tile_gated(fv, fg, p);
                         }
 #else
                         const gd_elem4 hv = quad_f16(mode_tag, acc[I][j], j, 2 * pr + s2);

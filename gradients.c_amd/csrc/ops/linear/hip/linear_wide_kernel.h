@@ -321,6 +321,11 @@ gd_linear_wide_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
                 p.epilogue == GD_HIP_EPI_BIAS_F32 ? v1 + (float)pf_b1[i] : v1;
             continue;
         }
+        if (EPI == GD_WIDE_EPI_PLAIN && (p.flags & GD_HIP_LINEAR_SQUARE_RELU)) {
+            y[(size_t)row * p.ldy + col] =
+                (gd_elem)gd_lin_activated(p.epilogue == GD_HIP_EPI_BIAS_F32 ? v1 + (float)pf_b1[i] : v1, p.flags);
+            continue;
+        }
 #endif
         gd_elem h1, h2 = (gd_elem)0.f;
         if (p.epilogue == GD_HIP_EPI_BIAS_F32) {
@@ -497,6 +502,11 @@ gd_linear_wide_half_kernel(const gd_elem *__restrict__ x, const gd_elem *__restr
             if (p.flags & GD_HIP_LINEAR_Y_F32) {
                 reinterpret_cast<float *>(y)[(size_t)e_row * p.ldy + e_col] =
                     p.epilogue == GD_HIP_EPI_BIAS_F32 ? v + (float)pf_b : v;
+                return;
+            }
+            if (p.flags & GD_HIP_LINEAR_SQUARE_RELU) {
+                y[(size_t)e_row * p.ldy + e_col] =
+                    (gd_elem)gd_lin_activated(p.epilogue == GD_HIP_EPI_BIAS_F32 ? v + (float)pf_b : v, p.flags);
                 return;
             }
 #endif

@@ -1,7 +1,9 @@
 /*
- * F32 residual stream with norms on the sublayers' outputs (gfx950).  HBM-bound row kernels, one workgroup per row:
+ * F32 residual stream with norms on the sublayers' outputs or in front of the sublayers (gfx950).  HBM-bound row kernels, one workgroup per row:
  *   embed      x = table[id] * scale, and x once more in the type the projections read
  *   norm_add   x += mult * (u * w / rms(u)) for a sublayer's output u, and the copy
+ *   add_norm   x += a sublayer's output u and the outputs of the experts a row went through, then h = x * w / rms(x),
+ *              which the next sublayer reads, once more for every expert the row goes to
  *   norm_rows  out = x * w / rms(x) of picked rows (the model's last norm in front of the LM head)
  * Sums, norms and the residual itself are F32 whatever the element type.  Rows of up to 8 * 256 * 4 elements on
  * aligned pointers stay in registers between the sum of squares and the update; others are read twice.
@@ -13,6 +15,14 @@
 
 template <typename T>
 struct gd_rn_vec;
+/* gd_backend_routed_rows; top 0: none */
+template <typename T>
+struct gd_hip_routed_choice {
+    T *at;
+    const int32_t *place;
+    uint32_t rows, top;
+    float weight;
+};
 template <>
 struct gd_rn_vec<gd_bf16> {
     static __device__ __forceinline__ void load(const gd_bf16 *p, float (&v)[8])
@@ -129,6 +139,105 @@ gd_residual_norm_add_kernel(const T *__restrict__ u, const float *__restrict__ w
     }
 }
 
+/* u, w and out may be null; choices of a row: rows place[row * top + k] of the packed rows, negative: none.  VEC: rows of
+ * up to 8 * 256 * 4 elements in 16-byte pieces, in registers between the sum of squares and the stores. */
+template <typename T, bool VEC>
+__global__ void __launch_bounds__(GD_RN_THREADS)
+gd_residual_add_norm_kernel(const T *__restrict__ u, gd_hip_routed_choice<T> in, float *__restrict__ x,
+                            const float *__restrict__ w, T *__restrict__ out, gd_hip_routed_choice<T> to, uint32_t cols,
+                            float eps)
+{
+    __shared__ float red[GD_RN_THREADS / 64];
+    const uint32_t row = blockIdx.x;
+    const size_t base = (size_t)row * cols;
+    float ss = 0.f;
+    if (VEC) {
+        float uv[GD_RN_CHUNKS][8], xv[GD_RN_CHUNKS][8], wv[GD_RN_CHUNKS][8]; /* all requested in front of the sums */
+#pragma unroll
+        for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+            const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
+            if (c >= cols) continue;
+            if (u != nullptr) gd_rn_vec<T>::load(u + base + c, uv[i]);
+            gd_rn_vec<float>::load(x + base + c, xv[i]);
+            if (w != nullptr) gd_rn_vec<float>::load(w + c, wv[i]);
+        }
+        if (u != nullptr) {
+#pragma unroll
+            for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+                if ((threadIdx.x + i * GD_RN_THREADS) * 8u >= cols) continue;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) xv[i][e] += uv[i][e];
+            }
+        }
+        for (uint32_t k = 0; k < in.top; ++k) {
+            const int32_t at = in.place[row * in.top + k];
+            if (at < 0 || (uint32_t)at >= in.rows) continue;
+#pragma unroll
+            for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+                const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
+                if (c < cols) gd_rn_vec<T>::load(in.at + (size_t)at * cols + c, uv[i]);
+            }
+#pragma unroll
+            for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+                if ((threadIdx.x + i * GD_RN_THREADS) * 8u >= cols) continue;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) xv[i][e] = fmaf(in.weight, uv[i][e], xv[i][e]);
+            }
+        }
+        const bool changed = u != nullptr || in.top != 0u;
+#pragma unroll
+        for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+            const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
+            if (c >= cols) continue;
+            if (changed) gd_rn_vec<float>::store(x + base + c, xv[i]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss = fmaf(xv[i][e], xv[i][e], ss);
+        }
+        if (w == nullptr) return;
+        ss = gd_block_sum<GD_RN_THREADS / 64>(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)cols + eps);
+#pragma unroll
+        for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+            const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
+            if (c >= cols) continue;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) xv[i][e] = xv[i][e] * inv * wv[i][e];
+            gd_rn_vec<T>::store(out + base + c, xv[i]);
+        }
+        for (uint32_t k = 0; k < to.top; ++k) {
+            const int32_t at = to.place[row * to.top + k];
+            if (at < 0 || (uint32_t)at >= to.rows) continue;
+#pragma unroll
+            for (int i = 0; i < GD_RN_CHUNKS; ++i) {
+                const uint32_t c = (threadIdx.x + i * GD_RN_THREADS) * 8u;
+                if (c < cols) gd_rn_vec<T>::store(to.at + (size_t)at * cols + c, xv[i]);
+            }
+        }
+        return;
+    }
+    for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS) {
+        float v = x[base + c];
+        if (u != nullptr) v += (float)u[base + c];
+        for (uint32_t k = 0; k < in.top; ++k) {
+            const int32_t at = in.place[row * in.top + k];
+            if (at >= 0 && (uint32_t)at < in.rows) v = fmaf(in.weight, (float)in.at[(size_t)at * cols + c], v);
+        }
+        x[base + c] = v;
+        ss = fmaf(v, v, ss);
+    }
+    if (w == nullptr) return;
+    ss = gd_block_sum<GD_RN_THREADS / 64>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)cols + eps);
+    for (uint32_t c = threadIdx.x; c < cols; c += GD_RN_THREADS) { /* the columns this thread has just stored */
+        const T h = (T)(x[base + c] * inv * w[c]);
+        out[base + c] = h;
+        for (uint32_t k = 0; k < to.top; ++k) {
+            const int32_t at = to.place[row * to.top + k];
+            if (at >= 0 && (uint32_t)at < to.rows) to.at[(size_t)at * cols + c] = h;
+        }
+    }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(GD_RN_THREADS)
 gd_residual_norm_rows_kernel(const float *__restrict__ x, const int32_t *__restrict__ rows, uint32_t n_rows,
@@ -164,6 +273,24 @@ extern "C" int gd_hip_launch_residual_norm_add(hipStream_t stream, const void *u
     if (rows == 0u) return (int)hipSuccess;
     const bool vec = aligned16 && (cols % 8u) == 0u && cols <= 8u * GD_RN_THREADS * GD_RN_CHUNKS;
 #define GD_GO(T, V) gd_residual_norm_add_kernel<T, V><<<rows, GD_RN_THREADS, 0, stream>>>((const T *)u, w, x, (T *)copy, cols, eps, mult)
+    if (is_f32) { if (vec) GD_GO(float, true); else GD_GO(float, false); }
+    else { if (vec) GD_GO(gd_bf16, true); else GD_GO(gd_bf16, false); }
+#undef GD_GO
+    return (int)hipGetLastError();
+}
+
+extern "C" int gd_hip_launch_residual_add_norm(hipStream_t stream, const void *u, void *in, const int32_t *in_place,
+                                               uint32_t in_rows, uint32_t in_top, float in_weight, float *x, const float *w,
+                                               void *out, void *to, const int32_t *to_place, uint32_t to_rows,
+                                               uint32_t to_top, uint32_t rows, uint32_t cols, float eps, int is_f32,
+                                               int aligned16)
+{
+    if (rows == 0u) return (int)hipSuccess;
+    const bool vec = aligned16 && (cols % 8u) == 0u && cols <= 8u * GD_RN_THREADS * GD_RN_CHUNKS;
+#define GD_GO(T, V)                                                                                                    \
+    gd_residual_add_norm_kernel<T, V><<<rows, GD_RN_THREADS, 0, stream>>>(                                             \
+        (const T *)u, gd_hip_routed_choice<T>{(T *)in, in_place, in_rows, in_top, in_weight}, x, w, (T *)out,          \
+        gd_hip_routed_choice<T>{(T *)to, to_place, to_rows, to_top, 1.0f}, cols, eps)
     if (is_f32) { if (vec) GD_GO(float, true); else GD_GO(float, false); }
     else { if (vec) GD_GO(gd_bf16, true); else GD_GO(gd_bf16, false); }
 #undef GD_GO

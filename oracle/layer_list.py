@@ -1,9 +1,9 @@
-"""Plain NumPy model of the decoders whose layers are listed in config.json (architecture "Girirax").
+"""Plain NumPy models of the decoders whose layers are listed in config.json (architectures "Girirax" and "Bonatar").
 
 One function per mechanism, written for reading: a token loop for the recurrence, full score matrices for the
 attention, everything in the floating-point type the caller passes (float64 by default).  It is what
-tests/test_girirax.py and tests/test_gpu_girirax.py compare with; it shares nothing with the product: no kernels, no
-cache, no chunking.
+tests/test_girirax.py, tests/test_bonatar.py and their GPU counterparts compare with; it shares nothing with the
+product: no kernels, no cache, no portions.
 
 Notation: h [T, width] is what a sublayer reads, T the tokens of ONE sequence from position 0.
 """
@@ -117,6 +117,108 @@ def gated_mlp(h, w):
 
 
 MIXERS = {"mamba2": mamba2, "latent_attention": latent_attention}
+
+
+# ---- Bonatar: attention inside chunks with grouped heads, experts chosen by token id ----------------------------
+
+def yarn_frequencies(base, dims, scaling):
+    """Frequencies of the dims/2 rotation pairs, and the factor of cosine and sine.  scaling (factor, original, fast,
+    slow) or None: pairs that turn more than `fast` times over `original` positions keep their frequency, those that
+    turn less than `slow` times have it divided by factor, a ramp over the pairs lies between."""
+    i = np.arange(dims // 2)
+    f = np.float64(base) ** (-2.0 * i / dims)
+    if scaling is None:
+        return f, 1.0
+
+    def pair_that_turns(t):
+        return dims * np.log(scaling["original"] / (2 * np.pi * t)) / (2 * np.log(base))
+    lo = max(np.floor(pair_that_turns(scaling["fast"])), 0)
+    hi = min(np.ceil(pair_that_turns(scaling["slow"])), dims - 1)
+    ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0, 1)
+    return f / scaling["factor"] * ramp + f * (1 - ramp), 0.1 * np.log(scaling["factor"]) + 1
+
+
+def rotate_neighbours(x, positions, freq, mult):
+    """x [T, H, D]: pair (2i, 2i + 1) turned by position * freq[i], cosine and sine times mult; dimensions behind the
+    last pair stay."""
+    angle = (positions[:, None] * freq)[:, None, :]
+    cos, sin = (np.cos(angle) * mult).astype(x.dtype), (np.sin(angle) * mult).astype(x.dtype)
+    y = x.copy()
+    n = 2 * len(freq)
+    u, v = x[..., 0:n:2], x[..., 1:n:2]
+    y[..., 0:n:2] = u * cos - v * sin
+    y[..., 1:n:2] = v * cos + u * sin
+    return y
+
+
+def chunk_attention(q, k, v, scale, chunk):
+    """q [T, H, D], k [T, G, D], v [T, G, V]: query head h reads key/value head h // (H // G); position i sees j <= i
+    of its own chunk of `chunk` positions (None: of all)."""
+    T, H = q.shape[:2]
+    per = H // k.shape[1]
+    i = np.arange(T)
+    seen = i[:, None] >= i[None, :]
+    if chunk is not None:
+        seen &= (i[:, None] // chunk) == (i[None, :] // chunk)
+    out = np.zeros((T, H, v.shape[2]), q.dtype)
+    for h in range(H):
+        s = np.where(seen, (q[:, h] @ k[:, h // per].T) * scale, -np.inf)
+        s = np.exp(s - s.max(axis=1, keepdims=True))
+        out[:, h] = (s / s.sum(axis=1, keepdims=True)) @ v[:, h // per]
+    return out
+
+
+def gated_chunk_attention(h, w, m):
+    """m: sizes (heads, kv_heads, dim, vdim, scale, rot, mask.size); one gate number per head."""
+    T, H, G, D, V = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    freq, mult = yarn_frequencies(m["rot"]["base"], m["rot"]["dims"], m["rot"].get("scaling"))
+    turn = lambda x: rotate_neighbours(x, np.arange(T), freq, mult)
+    q, k = turn((h @ w["q"].T).reshape(T, H, D)), turn((h @ w["k"].T).reshape(T, G, D))
+    out = chunk_attention(q, k, (h @ w["v"].T).reshape(T, G, V), m["scale"], m["mask"]["size"])
+    return (out * sigmoid(h @ w["g"].T)[:, :, None]).reshape(T, H * V) @ w["o"].T
+
+
+def square_relu_mlp(h, w):
+    return np.maximum(h @ w["up"].T, 0) ** 2 @ w["down"].T
+
+
+def clamped_expert(h, w, prefix, limit):
+    g = np.minimum(h @ w[prefix + "gate"].T, limit)
+    u = np.clip(h @ w[prefix + "up"].T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1)) @ w[prefix + "down"].T
+
+
+def table_routed_mlp(h, w, tokens, m):
+    """Every token's experts are its row of the table, weighted equally; a shared expert runs for all."""
+    table = w["table"].astype(np.int64)
+    y = np.zeros_like(h)
+    for t, token in enumerate(tokens):
+        for e in table[token]:
+            y[t] += clamped_expert(h[t:t + 1], w, "e%d." % e, m["expert"]["limit"])[0] / m["router"]["top"]
+    if m.get("shared") is not None:
+        y += clamped_expert(h, w, "shared.", m["shared"]["limit"])
+    return y
+
+
+def forward_bonatar(config, tensors, tokens, dtype=np.float64, trace=None):
+    """Logits [T, vocab] of one sequence.  Norms stand in front of the sublayers, their weights around zero; a layer
+    with weights_of uses another layer's tensors."""
+    eps, tokens = config["norm"]["eps"], np.asarray(tokens)
+    norm = lambda x, name: rms_norm(x, 1 + tensors[name].astype(dtype), eps)
+    x = tensors["embed"].astype(dtype)[tokens] * dtype(config["embedding"]["scale"])
+    for i, layer in enumerate(config["layers"]):
+        while layer.get("weights_of") is not None:
+            i = layer["weights_of"]
+            layer = config["layers"][i]
+        p = "l%d." % i
+        x = x + gated_chunk_attention(norm(x, p + "norm1"), _short_names(tensors, p + "mix.", dtype), layer["mixer"])
+        m = layer["mlp"]
+        if m is not None:
+            h, w = norm(x, p + "norm2"), _short_names(tensors, p + "mlp.", dtype)
+            x = x + (square_relu_mlp(h, w) if m["kind"] == "dense" else table_routed_mlp(h, w, tokens, m))
+        if trace is not None:
+            trace.append(x.copy())
+    return norm(x, "final.norm") @ tensors["head"].astype(dtype).T
 
 
 def _short_names(tensors, prefix, dtype):

@@ -23,6 +23,7 @@ GD_NULL_OP(gd_backend_fused_linear)
 GD_NULL_OP(gd_backend_fused_qkv_rope_append)
 GD_NULL_OP(gd_backend_gated_group_norm)
 GD_NULL_OP(gd_backend_gather_rows)
+GD_NULL_OP(gd_backend_grouped_attend)
 GD_NULL_OP(gd_backend_kv_cache_append_at)
 GD_NULL_OP(gd_backend_kv_cache_append_packed)
 GD_NULL_OP(gd_backend_kv_cache_append_positions)
@@ -40,11 +41,14 @@ GD_NULL_OP(gd_backend_qkv_rope_append)
 GD_NULL_OP(gd_backend_qkv_rope_append_packed)
 GD_NULL_OP(gd_backend_qkv_split_rope_forward)
 GD_NULL_OP(gd_backend_rand_uniform)
+GD_NULL_OP(gd_backend_residual_add_norm)
 GD_NULL_OP(gd_backend_residual_embed)
 GD_NULL_OP(gd_backend_residual_norm_add)
 GD_NULL_OP(gd_backend_residual_norm_rows)
 GD_NULL_OP(gd_backend_rms_norm_forward)
 GD_NULL_OP(gd_backend_rope_table_packed)
+GD_NULL_OP(gd_backend_route_by_tables)
+GD_NULL_OP(gd_backend_routed_mlp)
 GD_NULL_OP(gd_backend_sample_advance)
 GD_NULL_OP(gd_backend_sdpa_decode)
 GD_NULL_OP(gd_backend_sdpa_decode_at)
@@ -63,3 +67,9 @@ __attribute__((visibility("default"))) uint32_t gd_backend_latent_pitch(uint32_t
     return (kv_rank + rot_dim + 7u) & ~7u;
 }
 __attribute__((visibility("default"))) uint64_t gd_backend_latent_work_bytes() { return 4096u; }
+__attribute__((visibility("default"))) uint64_t gd_backend_grouped_work_bytes() { return 4096u; }
+struct gd_backend_routed_args { uint32_t experts, top; };
+__attribute__((visibility("default"))) uint32_t gd_backend_route_tiles(const struct gd_backend_routed_args *args, uint32_t rows)
+{
+    return rows * args->top;
+}
