@@ -85,12 +85,12 @@ def planned_dispatches(a):
         parts["probe"] = {"sdpa_decode": 7 * 3 * (2 + 13) * 30, "few_row_linear": 3 * 10 * (2 + 13) * 24}.get(a.probe, 400)
     elif a.minimax_kernels:
         parts["minimax_kernels"] = 2 * (8 + 4 * (1 + 10 + 20))
-    elif a.girirax:
-        # at most 12 launches per layer and 16 weights; 24 layers in the deepest size
-        one = 16 * 24 + 2 * (12 * 24 + 8)
+    elif a.girirax or a.bonatar:
+        # at most 14 launches per layer and 16 weights; 24 layers in the deepest size
+        one = 16 * 24 + 2 * (14 * 24 + 8)
         steps = min(a.decode_steps, 128)
-        per_model = (0 if a.decode_only else one) + (0 if a.prefill_only else one + (2 + min(20, steps) + 3 * steps) * (12 * 24 + 8))
-        parts["girirax"] = per_model * (1 if a.model else 2) * (1 if a.size else 3)
+        per_model = (0 if a.decode_only else one) + (0 if a.prefill_only else one + (2 + min(20, steps) + 3 * steps) * (14 * 24 + 8))
+        parts["layer_lists"] = per_model * (1 if a.model else 2) * (1 if a.size else 3)
     elif a.workload != 2:
         parts[f"configs[{a.workload}]"] = long_context(a.workload, a.steps, a.warmup, (a.batches or 3) if a.workload == 3 else 1)
     elif a.sampled:
@@ -631,11 +631,13 @@ def build_parser():
                          "the BASELINE.json configurations, operands rotating through HBM; prints its own JSON line")
     ap.add_argument("--girirax", action="store_true",
                     help="prefill and decode throughput of Girirax decoders (random weights) beside gpt_lm at equal sizes "
-                         "(gradients.c_amd/perf_girirax.py); prints its own JSON line.  With --size, --model, "
+                         "(gradients.c_amd/perf_layer_lists.py); prints its own JSON line.  With --size, --model, "
                          "--prefill-only, --decode-only and --decode-steps for parts of it")
-    ap.add_argument("--size", type=int, choices=(1024, 2048, 4096), help="with --girirax: one width")
-    ap.add_argument("--model", choices=("girirax", "gpt_lm"), help="with --girirax: one of the two models")
-    ap.add_argument("--decode-only", action="store_true", help="with --girirax: no prefill timing")
+    ap.add_argument("--bonatar", action="store_true", help="the same for Bonatar decoders")
+    ap.add_argument("--size", type=int, choices=(1024, 2048, 4096), help="with --girirax or --bonatar: one width")
+    ap.add_argument("--model", choices=("girirax", "bonatar", "gpt_lm"),
+                    help="with --girirax or --bonatar: one of the two models")
+    ap.add_argument("--decode-only", action="store_true", help="with --girirax or --bonatar: no prefill timing")
     ap.add_argument("--kernel-only", action="store_true",
                     help="only launch sdpa_decode at the benchmark shape plus calibration copies (for --pmc runs)")
     return ap
@@ -653,7 +655,8 @@ def main():
     # nothing at the 24-layer decoders, -11 % on the batch-1 step.  --graph-replay runtime keeps the runtime's default.
     config0 = None
     if (a.graph_replay == "nodes" and a.workload == 2 and not profiler_attached() and
-            not (a.headline_only or a.config0_only or a.kernel_only or a.probe or a.minimax_kernels or a.sampled or a.girirax)):
+            not (a.headline_only or a.config0_only or a.kernel_only or a.probe or a.minimax_kernels or a.sampled or a.girirax or
+                 a.bonatar)):
         try:
             config0 = config0_in_a_process_of_its_own()
         except Exception as e:  # measured in this process instead, below
@@ -675,9 +678,9 @@ def main():
     if a.minimax_kernels:
         minimax_kernels(pkg)
         return
-    if a.girirax:
-        from gradients_c_amd import perf_girirax
-        perf_girirax.run(pkg, a.size, a.model, a.prefill_only, a.decode_only, min(a.decode_steps, 128))
+    if a.girirax or a.bonatar:
+        from gradients_c_amd import perf_layer_lists
+        perf_layer_lists.run(pkg, "girirax" if a.girirax else "bonatar", a.size, a.model, a.prefill_only, a.decode_only, min(a.decode_steps, 128))
         return
     from gradients_c_amd import decoder as D
     if a.config0_only:

@@ -124,13 +124,24 @@ __device__ __forceinline__ void gd_tile_load_lds16(const gd_elem *uniform_base, 
                  : "memory");
 }
 
-template <int WM, int WN, bool W_NK, int PRO, bool ROPE = false>
+/* GROUPED instantiation: the rows are packed by group (the experts of a routed feed-forward), and every group has its own
+ * weights, one behind the other.  tiles [0]: number of row tiles, then from [2] on (group, first row) of each, BM rows or
+ * up to the group's end first[group + 1].  x rows behind the last group's are read and must exist (up to BM - 1). */
+struct gd_tile_group {
+    const int32_t *first, *tiles;
+    uint32_t w_rows; /* weight rows of a group */
+};
+__device__ __forceinline__ const gd_tile_rope &gd_tile_rope_of(const gd_tile_rope &r) { return r; }
+__device__ __forceinline__ gd_tile_rope gd_tile_rope_of(const gd_tile_group &) { return gd_tile_rope{}; }
+
+template <int WM, int WN, bool W_NK, int PRO, bool ROPE = false, bool GROUPED = false>
 __global__ void __launch_bounds__(256)
 gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__ w, const gd_elem *__restrict__ bias,
                       const gd_elem *__restrict__ residual, const gd_elem *__restrict__ norm_w,
                       gd_elem *__restrict__ y, gd_hip_linear_params p, uint32_t tiles_m, uint32_t tiles_n,
-                      uint32_t vector_store, gd_tile_rope rp)
+                      uint32_t vector_store, std::conditional_t<GROUPED, gd_tile_group, gd_tile_rope> extra)
 {
+    auto &&rp = gd_tile_rope_of(extra);
     constexpr uint32_t BM = 64u * WM, BN = 64u * WN;
     constexpr int A_PER = BM / 32;                 /* 16-byte chunks of the activation tile per thread */
     constexpr int B_PER = W_NK ? (int)(BN / 32) : 8; /* weight chunks per thread */
@@ -141,7 +152,10 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
     unsigned char *epi = gd_tile_smem + STAGE_BYTES;           /* [64][BN] halfs */
     float *s_inv = reinterpret_cast<float *>(epi); /* [BM] row factors of rms_norm; live during the main loop only */
 
+    if constexpr (GROUPED) tiles_m = (uint32_t)__builtin_amdgcn_readfirstlane(extra.tiles[0]);
     const uint32_t total = tiles_m * tiles_n;
+    const gd_elem *wt = w;  /* GROUPED: the weights of the current tile's group */
+    uint32_t m_end = p.M;   /* GROUPED: one behind the last row of the group */
     constexpr bool DIRECT = PRO == GD_HIP_PRO_NONE;
     uint32_t m0 = 0u, n0 = 0u; /* origin of the current tile (rows, output columns) */
     /* swiglu epilogue ([N,K] weights of 2H rows, H = p.N output columns).  The BN weight rows of a tile are two
@@ -164,11 +178,19 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
         const uint32_t width = 8u * tiles_n;
         const uint32_t first_m = (pid / width) * 8u;
         const uint32_t gsz = min(tiles_m - first_m, 8u);
-        tm0 = (first_m + (pid % width) % gsz) * BM;
+        const uint32_t row_tile = first_m + (pid % width) % gsz;
         tn0 = ((pid % width) / gsz) * out_bn;
+        if constexpr (GROUPED) {
+            const uint32_t group = (uint32_t)__builtin_amdgcn_readfirstlane(extra.tiles[2u + 2u * row_tile]);
+            tm0 = (uint32_t)__builtin_amdgcn_readfirstlane(extra.tiles[3u + 2u * row_tile]);
+            wt = w + (size_t)group * extra.w_rows * p.ldw;
+            m_end = (uint32_t)__builtin_amdgcn_readfirstlane(extra.first[group + 1u]);
+        } else {
+            tm0 = row_tile * BM;
+        }
     };
     auto direct_ok = [&](uint32_t tm0, uint32_t tn0) __attribute__((always_inline)) {
-        return DIRECT && tm0 + BM <= p.M && tn0 + out_bn <= p.N && (p.K % 64u) == 0u && p.K >= 128u;
+        return DIRECT && (GROUPED || tm0 + BM <= p.M) && tn0 + out_bn <= p.N && (p.K % 64u) == 0u && p.K >= 128u;
     };
 
     uint32_t tid_opaque = threadIdx.x;
@@ -188,6 +210,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
     const uint32_t tid = tid_opaque, lane = tid & 63u, wave = tid >> 6;
     const uint32_t wm = wave >> 1, wn = wave & 1u;
     locate(tile, m0, n0);
+    const uint32_t row_end = GROUPED ? m_end : p.M; /* for the epilogue: m_end moves on with the next tile's loads */
 
     /* staging coordinates */
     const uint32_t a_c = tid & 7u, a_r = tid >> 3; /* activation: chunk a_c of rows a_r + 32*i */
@@ -213,7 +236,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
                 ra[i] = zero8;
                 if (PRO == GD_HIP_PRO_SWIGLU) rz[i] = zero8;
             }
-            if (!GUARDED || (kok && gm < p.M)) {
+            if (!GUARDED || (kok && gm < m_end)) {
                 const gd_elem *xr = x + (size_t)gm * p.ldx + k;
                 ra[i] = *reinterpret_cast<const gd_elem8 *>(xr);
                 if (PRO == GD_HIP_PRO_SWIGLU) rz[i] = *reinterpret_cast<const gd_elem8 *>(xr + p.K);
@@ -226,7 +249,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
                 const uint32_t gn = wrow(n0, a_r + 32u * (uint32_t)i);
                 if (GUARDED) rb[i] = zero8;
                 if (!GUARDED || (kok && wrow_ok(n0, a_r + 32u * (uint32_t)i)))
-                    rb[i] = *reinterpret_cast<const gd_elem8 *>(w + (size_t)gn * p.ldw + k);
+                    rb[i] = *reinterpret_cast<const gd_elem8 *>(wt + (size_t)gn * p.ldw + k);
             }
         } else {
             const uint32_t gn = n0 + kb_nc * 8u;
@@ -235,7 +258,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
                 const uint32_t gk = kt * GD_TILE_BK + kb_j * 8u + i;
                 if (GUARDED || !KB_ALL) rb[i] = zero8;
                 if ((KB_ALL || kb_active) && (!GUARDED || (gk < p.K && gn < p.N)))
-                    rb[i] = *reinterpret_cast<const gd_elem8 *>(w + (size_t)gk * p.ldw + gn);
+                    rb[i] = *reinterpret_cast<const gd_elem8 *>(wt + (size_t)gk * p.ldw + gn);
             }
         }
     };
@@ -308,7 +331,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
         } else if (W_NK) {
             const uint32_t tb = t - (uint32_t)A_DIRECT;
             const uint32_t row0 = wave_u * (BN / 4u) + tb * RW;
-            gd_tile_load_lds16(w + (size_t)wrow(tn0, row0) * p.ldw + kt * DBK, (tb & 1u) ? d_off_b1 : d_off_b,
+            gd_tile_load_lds16(wt + (size_t)wrow(tn0, row0) * p.ldw + kt * DBK, (tb & 1u) ? d_off_b1 : d_off_b,
                                lds_base + ((2u * BM + stage * BN) * CH + row0 * CH) * 16u);
         } else {
             /* k-rows kr0 .. kr0+RPL-1 of the tile; lane L fills position L%CPR of row kr0 + L/CPR */
@@ -316,7 +339,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
             const uint32_t kr0 = (wave_u * (uint32_t)B_DIRECT + tb) * RPL;
             const uint32_t row = (RPL >= 4u ? 0u : ((tb * RPL) & 3u)) + lane / CPR; /* row & 3 */
             const uint32_t chunk = (lane % CPR) ^ ((row & 3u) << 2);
-            gd_tile_load_lds16(w + (size_t)(kt * DBK + kr0) * p.ldw + tn0, d_off_b + chunk * 16u,
+            gd_tile_load_lds16(wt + (size_t)(kt * DBK + kr0) * p.ldw + tn0, d_off_b + chunk * 16u,
                                lds_base + ((2u * BM + stage * BN) * CH + kr0 * CPR) * 16u);
         }
     };
@@ -538,7 +561,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
                 const uint32_t idx = idx0 + tid;
                 const uint32_t er = idx / (CPRW / 2u), v = idx % (CPRW / 2u);
                 const uint32_t gr = m0 + (er >> 5) * (WM * 32u) + (uint32_t)I * 32u + (er & 31u), gc = n0 + v * 8u;
-                if (gr >= p.M || gc >= p.N) continue;
+                if (gr >= row_end || gc >= p.N) continue;
                 /* staged columns: wavefront column wc holds its HW value columns, then their gates */
                 const uint32_t cv = (v / (HW / 8u)) * (HW / 4u) + v % (HW / 8u);
                 const gd_elem8 hv = read_chunk(er, cv), hg = read_chunk(er, cv + HW / 8u);
@@ -558,7 +581,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
             const uint32_t idx = idx0 + tid;
             const uint32_t er = idx / CPRW, v = idx % CPRW;
             const uint32_t gr = m0 + (er >> 5) * (WM * 32u) + (uint32_t)I * 32u + (er & 31u), gc = n0 + v * 8u;
-            if (gr >= p.M || gc >= p.N) continue;
+            if (gr >= row_end || gc >= p.N) continue;
             gd_elem8 h = read_chunk(er, v);
             gd_elem *yr = y + (size_t)gr * p.ldy + gc;
             if (vector_store && gc + 8u <= p.N) {
@@ -838,7 +861,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
     };
 
         /* interior tile: every staged chunk is in range, so the main loop carries no guards */
-        const bool interior = m0 + BM <= p.M && n0 + out_bn <= p.N && (p.K % GD_TILE_BK) == 0u;
+        const bool interior = m0 + BM <= m_end && n0 + out_bn <= p.N && (p.K % GD_TILE_BK) == 0u;
 
         if (PRO == GD_HIP_PRO_RMS_NORM) {
             __syncthreads(); /* the previous tile's epilogue has left the buffer that holds the row factors */
@@ -890,7 +913,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
             const uint32_t next = tile + gridDim.x;
             if (next < total) {
                 uint32_t nm0, nn0;
-                locate(next, nm0, nn0);
+                locate(next, nm0, nn0); /* GROUPED: also the group of the next tile, whose loads are requested here */
                 if (direct_ok(nm0, nn0)) {
                     direct_loads(nm0, nn0, 0u);
                     direct_loads(nm0, nn0, 1u);
@@ -918,7 +941,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
         auto finish = [&](auto mode_tag) __attribute__((always_inline)) {
             if constexpr (ROPE) {
                 epilogue_own_rope(mode_tag);
-            } else if (WM >= 3 && WN == 4 && vector_store && m0 + BM <= p.M && n0 + out_bn <= p.N) {
+            } else if (WM >= 3 && WN == 4 && vector_store && m0 + BM <= row_end && n0 + out_bn <= p.N) {
                 if (gated) epilogue_own_gated(mode_tag);
                 else epilogue_own(mode_tag);
             } else {
@@ -932,6 +955,44 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
     }
 }
 
+#ifdef GD_LINEAR_TILE_GROUPED
+template <int WM, int WN>
+static int launch_tile_grouped(hipStream_t stream, const gd_elem *x, const gd_elem *w, gd_elem *y,
+                               const gd_hip_linear_params &p, const gd_tile_group &group, uint32_t max_tiles,
+                               uint32_t workgroups)
+{
+    constexpr uint32_t BM = 64u * WM, BN = 64u * WN;
+    constexpr size_t lds = (size_t)2u * (BM + BN) * 8u * 16u + (size_t)64u * BN * 2u;
+    static bool configured = false;
+    auto kernel = gd_linear_tile_kernel<WM, WN, true, GD_HIP_PRO_NONE, false, true>;
+    if (!configured) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel),
+                                                 hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return (int)e;
+        configured = true;
+    }
+    const uint32_t out_bn = p.swiglu_cols != 0u ? BN / 2u : BN, tiles_n = (p.N + out_bn - 1u) / out_bn;
+    const uint64_t all = (uint64_t)max_tiles * tiles_n;
+    kernel<<<(uint32_t)(all < workgroups ? all : workgroups), 256, lds, stream>>>(x, w, nullptr, nullptr, nullptr, y, p,
+                                                                                  max_tiles, tiles_n, 1u, group);
+    return (int)hipGetLastError();
+}
+
+/* y rows packed by group = x rows times the group's weights: p as for gd_hip_launch_linear_tile (M: packed rows; [N,K]
+ * weights, 16-byte aligned rows of x, w and y, no bias, no residual); max_tiles: upper bound of the row tiles, of 256
+ * (big_tiles) or 128 rows */
+extern "C" int gd_hip_launch_linear_tile_grouped_bf16(hipStream_t stream, const void *x, const void *w, void *y,
+                                                      const gd_hip_linear_params *p, const int32_t *first,
+                                                      const int32_t *tiles, uint32_t w_rows, uint32_t max_tiles,
+                                                      int big_tiles, int compute_units)
+{
+    const uint32_t units = ((uint32_t)(compute_units > 0 ? compute_units : 256) + 7u) & ~7u;
+    const gd_tile_group group = {first, tiles, w_rows};
+    if (big_tiles)
+        return launch_tile_grouped<4, 4>(stream, (const gd_elem *)x, (const gd_elem *)w, (gd_elem *)y, *p, group, max_tiles, units);
+    return launch_tile_grouped<2, 2>(stream, (const gd_elem *)x, (const gd_elem *)w, (gd_elem *)y, *p, group, max_tiles, 2u * units);
+}
+#else
 template <int WM, int WN, bool W_NK, int PRO>
 int gd_linear_tile_launch_one(hipStream_t stream, const gd_elem *x, const gd_elem *w, const gd_elem *bias,
                            const gd_elem *residual, const gd_elem *norm_w, gd_elem *y, const gd_hip_linear_params &p,
@@ -1131,3 +1192,4 @@ extern "C" uint32_t GD_LINEAR_FN(gd_hip_linear_tile_rope_head_rows)(uint32_t M, 
 }
 #endif
 #endif /* GD_LINEAR_TILE_PART */
+#endif /* GD_LINEAR_TILE_GROUPED */

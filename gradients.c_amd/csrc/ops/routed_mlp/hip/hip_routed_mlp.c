@@ -1,13 +1,25 @@
 /* Host dispatch of gd_backend_route_by_tables and gd_backend_routed_mlp. */
+#include <string.h>
+
 #include "../../_shared/packed_seqs_host.h"
+#include "../../linear/hip/hip_linear_types.h"
 #include "hip_routed_mlp_types.h"
 
 int gd_hip_launch_route(hipStream_t stream, const gd_hip_route_jobs *jobs, uint32_t n_jobs, const int32_t *ids, uint32_t rows);
 int gd_hip_launch_routed_project(hipStream_t stream, const void *x, const void *w, void *y, const int32_t *first,
                                  const int32_t *tiles, const gd_hip_routed_params *p, int is_f32);
 
-/* rows of a tile of the work list, by the kernels that will walk it */
-#define GD_ROUTED_ANY_ROWS 64u
+int gd_hip_launch_routed_stream(hipStream_t stream, const void *x, const void *w, void *y, const int32_t *first,
+                                const int32_t *tiles, const gd_hip_routed_params *p);
+int gd_hip_launch_linear_tile_grouped_bf16(hipStream_t stream, const void *x, const void *w, void *y,
+                                           const gd_hip_linear_params *p, const int32_t *first, const int32_t *tiles,
+                                           uint32_t w_rows, uint32_t max_tiles, int big_tiles, int compute_units);
+
+/* the kernels that walk the work list, by the rows of its tiles */
+#define GD_ROUTED_STREAM_ROWS 16u /* few rows per expert, BF16 */
+#define GD_ROUTED_ANY_ROWS 64u    /* any sizes and types */
+#define GD_ROUTED_TILE_ROWS 128u  /* many rows per expert, BF16 */
+#define GD_ROUTED_WIDE_ROWS 256u  /* very many */
 
 static bool args_ok(const gd_backend_routed_args *a)
 {
@@ -17,10 +29,10 @@ static bool args_ok(const gd_backend_routed_args *a)
 
 static uint32_t tile_rows_of(const gd_backend_routed_args *a, uint32_t rows, uint32_t dtype)
 {
-    (void)a;
-    (void)rows;
-    (void)dtype;
-    return GD_ROUTED_ANY_ROWS;
+    const uint64_t per_expert = (uint64_t)rows * a->top / a->experts;
+    if (dtype != GD_BACKEND_DTYPE_BF16 || (a->width % 8u) != 0u || (a->ff % 8u) != 0u) return GD_ROUTED_ANY_ROWS;
+    if (per_expert >= 768u) return GD_ROUTED_WIDE_ROWS;
+    return per_expert >= 24u ? GD_ROUTED_TILE_ROWS : GD_ROUTED_STREAM_ROWS;
 }
 
 /* every expert with rows has at most one tile that is not full */
@@ -79,6 +91,33 @@ static bool weight_ok(const gd_backend_tensor_view *v, uint64_t rows, uint32_t c
            (v->offset & 15u) == 0u;
 }
 
+/* y [packed, n] = x [packed, k] times the experts' weights */
+static int project(gd_backend *backend, const gd_backend_tensor_view *x, const gd_backend_tensor_view *w,
+                   const gd_backend_tensor_view *y, const int32_t *first, const int32_t *tiles, const gd_hip_routed_params *p,
+                   uint32_t dtype)
+{
+    const void *xp = gd_hip_view_ptr(x), *wp = gd_hip_view_ptr(w);
+    void *yp = gd_hip_view_ptr(y);
+    gd_hip_linear_params l;
+    if (p->tile_rows == GD_ROUTED_ANY_ROWS)
+        return gd_hip_launch_routed_project(backend->stream, xp, wp, yp, first, tiles, p, dtype == GD_BACKEND_DTYPE_F32);
+    if (p->tile_rows == GD_ROUTED_STREAM_ROWS)
+        return gd_hip_launch_routed_stream(backend->stream, xp, wp, yp, first, tiles, p);
+    memset(&l, 0, sizeof(l));
+    l.M = p->packed;
+    l.N = l.ldy = p->n;
+    l.K = l.ldx = l.ldw = p->k;
+    l.w_is_nk = 1u;
+    if (p->gated) {
+        l.swiglu_cols = p->n;
+        l.flags = GD_HIP_LINEAR_CLAMPED_GATE;
+        l.gate_limit = p->gate_limit;
+        l.gate_alpha = p->gate_alpha;
+    }
+    return gd_hip_launch_linear_tile_grouped_bf16(backend->stream, xp, wp, yp, &l, first, tiles, p->n * (p->gated ? 2u : 1u),
+                                                  p->max_tiles, p->tile_rows == GD_ROUTED_WIDE_ROWS, backend->compute_units);
+}
+
 gd_status gd_backend_routed_mlp(gd_backend *backend, const gd_backend_tensor_view *rows,
                                 const gd_backend_tensor_view *w_upgate, const gd_backend_tensor_view *w_down,
                                 const gd_backend_tensor_view *act, const gd_backend_tensor_view *out,
@@ -88,7 +127,7 @@ gd_status gd_backend_routed_mlp(gd_backend *backend, const gd_backend_tensor_vie
     uint64_t packed;
     uint32_t dtype, tile_rows;
     const int32_t *first, *tiles;
-    int e, f32;
+    int e;
     if (backend == NULL || !args_ok(args) || routes == NULL || routes->rows == 0u || !gd_hip_view_ok(rows))
         return GD_ERR_INVALID_ARGUMENT;
     packed = (uint64_t)routes->rows * args->top;
@@ -119,12 +158,8 @@ gd_status gd_backend_routed_mlp(gd_backend *backend, const gd_backend_tensor_vie
     down.n = args->width;
     down.k = args->ff;
     down.gated = 0u;
-    f32 = dtype == GD_BACKEND_DTYPE_F32;
     if (up.max_tiles > 65535u) return GD_ERR_UNSUPPORTED;
-    e = gd_hip_launch_routed_project(backend->stream, gd_hip_view_ptr(rows), gd_hip_view_ptr(w_upgate), gd_hip_view_ptr(act),
-                                     first, tiles, &up, f32);
-    if (e == 0)
-        e = gd_hip_launch_routed_project(backend->stream, gd_hip_view_ptr(act), gd_hip_view_ptr(w_down), gd_hip_view_ptr(out),
-                                         first, tiles, &down, f32);
+    e = project(backend, rows, w_upgate, act, first, tiles, &up, dtype);
+    if (e == 0) e = project(backend, act, w_down, out, first, tiles, &down, dtype);
     return gd_hip_finish_op(backend, e);
 }

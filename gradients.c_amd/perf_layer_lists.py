@@ -1,29 +1,34 @@
-"""Prefill and decode throughput of Girirax decoders at sizes that resemble real layers (random weights), beside the
-gpt_lm decoder of the same width, depth, feed-forward, vocabulary and batch.
+"""Prefill and decode throughput of the decoders whose layers are listed in config.json (Girirax, Bonatar) at sizes that
+resemble real layers (random weights), beside the gpt_lm decoder of the same width, depth, vocabulary and batch.
 
-    python bench.py --girirax                 every size, both models, one JSON line
-    python bench.py --girirax --size 2048     one size
-    python bench.py --girirax --size 2048 --model girirax --prefill-only     for kernel traces (one untimed pass, one timed)
-    python bench.py --girirax --size 2048 --model girirax --decode-steps 8   few steps, for kernel traces
+    python bench.py --girirax                 every size, Girirax and gpt_lm, one JSON line
+    python bench.py --bonatar                 every size, Bonatar and gpt_lm
+    python bench.py --bonatar --size 2048     one size
+    python bench.py --bonatar --size 2048 --model bonatar --prefill-only     for kernel traces (one untimed pass, one timed)
+    python bench.py --bonatar --size 2048 --model bonatar --decode-steps 8   few steps, for kernel traces
 
-Half of the layers are state-space recurrences, half latent attention; the projections of a layer hold about as many
-weights as those of the gpt_lm layer.  Prefill: packed prompts of mixed lengths.  Decode: greedy resident session over
-caches of 1024 .. 4095 tokens that a real prefill built, positions held, graph replays.
+Girirax: half of the layers are state-space recurrences, half latent attention; the projections of a layer hold about as
+many weights as those of the gpt_lm layer.  Bonatar: four query heads share keys and values; half of the layers have a
+square-relu feed-forward with as many weights as gpt_lm's, half a shared expert and two routed ones that together are as
+large for a token; the routed experts that a token does not use come on top.  Prefill: packed prompts of mixed lengths.
+Decode: greedy resident session over caches of 1024 .. 4095 tokens that a real prefill built, positions held, graph
+replays.
 """
 import json
 import time
 
 import numpy as np
 
-#        width: layers, feed-forward, vocabulary, gpt heads x size, recurrence, latent attention, decode batch
+#        width: layers, feed-forward, vocabulary, gpt heads x size, recurrence, latent attention, decode batch; Bonatar:
+#        key/value heads, chunk, number of experts
 SIZES = {
-    1024: dict(layers=12, ff=2816, vocab=32768, heads=8, head_dim=128, batch=64,
+    1024: dict(layers=12, ff=2816, vocab=32768, heads=8, head_dim=128, batch=64, kv_heads=2, chunk=8192, experts=16,
                ssm=dict(heads=32, vdim=64, state=128, groups=1, norm_groups=1, conv=4),
                latent=dict(heads=8, dim=128, rot_dim=64, vdim=128, q_rank=512, kv_rank=256)),
-    2048: dict(layers=24, ff=5632, vocab=32768, heads=16, head_dim=128, batch=16,
+    2048: dict(layers=24, ff=5632, vocab=32768, heads=16, head_dim=128, batch=16, kv_heads=4, chunk=2048, experts=16,
                ssm=dict(heads=64, vdim=64, state=128, groups=1, norm_groups=1, conv=4),
                latent=dict(heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512)),
-    4096: dict(layers=8, ff=11264, vocab=32768, heads=32, head_dim=128, batch=32,
+    4096: dict(layers=8, ff=11264, vocab=32768, heads=32, head_dim=128, batch=32, kv_heads=8, chunk=8192, experts=8,
                ssm=dict(heads=128, vdim=64, state=128, groups=8, norm_groups=8, conv=4),
                latent=dict(heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512)),
 }
@@ -41,6 +46,22 @@ def girirax_config(width):
                        for t, m in (mixers[i % 2] for i in range(s["layers"]))]}
 
 
+def bonatar_config(width):
+    s = SIZES[width]
+    D = s["head_dim"]
+    mixer = {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5,
+             "mask": {"size": s["chunk"]},
+             "rot": {"base": 500000.0, "dims": D, "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+    mlps = [{"kind": "dense", "ff": s["ff"] * 3 // 2},
+            {"kind": "moe", "router": {"experts": s["experts"], "top": 2}, "expert": {"ff": s["ff"] // 4, "limit": 7.0},
+             "shared": {"ff": s["ff"] // 2, "limit": 7.0}}]
+    return {"architecture": "Bonatar", "vocab": s["vocab"], "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 8.0},
+            "layers": [{"type": "attention", "mixer": mixer, "mlp": mlps[i % 2]} for i in range(s["layers"])]}
+
+
+CONFIGS = {"girirax": girirax_config, "bonatar": bonatar_config}
+
+
 def _prompts(which, batch):
     rng = np.random.default_rng(which)
     lens = rng.integers(64, 2049, batch) if which == 4 else rng.integers(1024, 4096, batch)
@@ -49,8 +70,8 @@ def _prompts(which, batch):
 
 def _open(D, model, width, batch, step_tokens):
     s = SIZES[width]
-    if model == "girirax":
-        m = D.Model(config_json=json.dumps(girirax_config(width)), seed=7)
+    if model in CONFIGS:
+        m = D.Model(config_json=json.dumps(CONFIGS[model](width)), seed=7)
         try:
             return m.decoder(max_seq=T, batch=batch, max_step_tokens=step_tokens)
         finally:
@@ -66,6 +87,9 @@ def _weights(model, width):
     mlp = 3 * width * s["ff"]
     if model == "gpt_lm":
         return s["layers"] * (4 * width * width + mlp)
+    if model == "bonatar":
+        qkvo = 2 * s["heads"] * s["head_dim"] + 2 * s["kv_heads"] * s["head_dim"] + s["heads"]
+        return s["layers"] * (width * qkvo + mlp)
     m, a = s["ssm"], s["latent"]
     inner = m["heads"] * m["vdim"]
     ssm = width * (3 * inner + 2 * m["groups"] * m["state"] + m["heads"])
@@ -112,16 +136,16 @@ def _decode(D, model, width, steps):
             "tokens_per_s": round(batch / s, 1)}
 
 
-def run(pkg, size=None, model=None, prefill_only=False, decode_only=False, steps=100):
+def run(pkg, architecture, size=None, model=None, prefill_only=False, decode_only=False, steps=100):
     from . import decoder as D
     out = {}
     for width in ([size] if size else sorted(SIZES)):
-        for m in ([model] if model else ["girirax", "gpt_lm"]):
+        for m in ([model] if model else [architecture, "gpt_lm"]):
             r = {"layer_weights": _weights(m, width)}
             if not decode_only:
                 r["prefill"] = _prefill(D, m, width)
             if not prefill_only:
                 r["decode"] = _decode(D, m, width, steps)
             out.setdefault("width %d, %d layers" % (width, SIZES[width]["layers"]), {})[m] = r
-    print(json.dumps({"girirax": out, "dtype": {"girirax": "bf16", "gpt_lm": "f16"}, "data": "synthetic",
+    print(json.dumps({architecture: out, "dtype": {architecture: "bf16", "gpt_lm": "f16"}, "data": "synthetic",
                       "weights": "random"}))
