@@ -165,6 +165,23 @@ extern "C" int GD_LINEAR_FN(gd_hip_launch_linear)(hipStream_t stream, const void
         const uint64_t big = (uint64_t)((p.M + 255u) / 256u) * ((p.N + out_cols - 1u) / out_cols);
         const uint32_t units = min_workgroups > 0 ? (uint32_t)min_workgroups / 2u : 256u;
         *family = GD_HIP_LINEAR_FAMILY_TILE;
+#if GD_LINEAR_IS_BF16
+        /* a last column tile of a few columns (gates, step sizes behind the large parts of a stacked projection) would
+         * take as long as a whole one, and off the direct staging path: the few-row kernel reads x once more instead */
+        const uint32_t narrow = p.N % 256u;
+        if (p.swiglu_cols == 0u && p.epilogue == GD_HIP_EPI_NONE && p.N > 256u && narrow != 0u && narrow <= 32u) {
+            gd_hip_linear_params rest = p, whole = p;
+            whole.N = p.N - narrow;
+            rest.N = narrow;
+            if (narrow <= 16u) launch_stream<1, 4>(stream, xp, wp + (size_t)whole.N * p.ldw, bp, rp, np, yp + whole.N, rest, rope);
+            else launch_stream<2, 4>(stream, xp, wp + (size_t)whole.N * p.ldw, bp, rp, np, yp + whole.N, rest, rope);
+            const int e = (int)hipGetLastError();
+            if (e != (int)hipSuccess) return e;
+            const uint64_t whole_tiles = (uint64_t)((p.M + 255u) / 256u) * (whole.N / 256u);
+            return GD_LINEAR_FN(gd_hip_launch_linear_tile)(stream, x, w, bias, residual, norm_w, y, &whole, whole_tiles >= units,
+                                                           store_vector_ok, (int)units);
+        }
+#endif
         return GD_LINEAR_FN(gd_hip_launch_linear_tile)(stream, x, w, bias, residual, norm_w, y, params, big >= units, store_vector_ok, (int)units);
     } else if (wide_mode != 0 && p.w_is_nk &&
                GD_LINEAR_FN(gd_hip_try_launch_linear_wide)(stream, x, w, bias, residual, norm_w, y, params, rope_epilogue,

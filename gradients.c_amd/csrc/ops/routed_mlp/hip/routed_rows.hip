@@ -9,6 +9,7 @@
 
 #define GD_ROUTE_THREADS 1024u
 #define GD_ROUTE_MAX_EXPERTS 4096u
+#define GD_ROUTE_BATCH 8u /* choices a thread looks up together */
 
 /* exclusive sums of v over the workgroup's threads; total receives the sum */
 __device__ __forceinline__ uint32_t gd_route_scan(uint32_t v, uint32_t *smem, uint32_t *total)
@@ -40,16 +41,31 @@ gd_route_kernel(gd_hip_route_jobs jobs, const int32_t *__restrict__ ids, uint32_
     const uint32_t pairs = rows * j.top, tid = threadIdx.x;
     for (uint32_t e = tid; e < j.experts; e += GD_ROUTE_THREADS) s_count[e] = 0u;
     __syncthreads();
-    auto expert_of = [&](uint32_t p) {
-        const int32_t id = ids[p / j.top];
-        const int32_t e = id >= 0 && (uint32_t)id < j.vocab ? j.table[(size_t)id * j.top + p % j.top] : -1;
-        return e >= 0 && (uint32_t)e < j.experts ? e : -1;
+    /* the experts of BATCH choices of this thread, p, p + threads, ..: all ids requested together, then all entries */
+    auto experts_of = [&](uint32_t p, int32_t (&e)[GD_ROUTE_BATCH]) __attribute__((always_inline)) {
+        int32_t id[GD_ROUTE_BATCH];
+#pragma unroll
+        for (uint32_t i = 0; i < GD_ROUTE_BATCH; ++i) {
+            const uint32_t at = p + i * GD_ROUTE_THREADS;
+            id[i] = at < pairs ? ids[at / j.top] : -1;
+        }
+#pragma unroll
+        for (uint32_t i = 0; i < GD_ROUTE_BATCH; ++i) {
+            const uint32_t at = p + i * GD_ROUTE_THREADS;
+            e[i] = id[i] >= 0 && (uint32_t)id[i] < j.vocab ? j.table[(size_t)id[i] * j.top + at % j.top] : -1;
+        }
+#pragma unroll
+        for (uint32_t i = 0; i < GD_ROUTE_BATCH; ++i) e[i] = (uint32_t)e[i] < j.experts ? e[i] : -1;
     };
     /* the choice's rank among those of its expert waits in place */
-#pragma unroll 4
-    for (uint32_t p = tid; p < pairs; p += GD_ROUTE_THREADS) {
-        const int32_t e = expert_of(p);
-        j.place[p] = e >= 0 ? (int32_t)atomicAdd(&s_count[e], 1u) : -1;
+    for (uint32_t p = tid; p < pairs; p += GD_ROUTE_BATCH * GD_ROUTE_THREADS) {
+        int32_t e[GD_ROUTE_BATCH];
+        experts_of(p, e);
+#pragma unroll
+        for (uint32_t i = 0; i < GD_ROUTE_BATCH; ++i) {
+            if (p + i * GD_ROUTE_THREADS < pairs)
+                j.place[p + i * GD_ROUTE_THREADS] = e[i] >= 0 ? (int32_t)atomicAdd(&s_count[e[i]], 1u) : -1;
+        }
     }
     __syncthreads();
     /* four neighbouring experts per thread */
@@ -80,10 +96,16 @@ gd_route_kernel(gd_hip_route_jobs jobs, const int32_t *__restrict__ ids, uint32_
         at += n[i];
     }
     __syncthreads();
-#pragma unroll 4
-    for (uint32_t p = tid; p < pairs; p += GD_ROUTE_THREADS) {
-        const int32_t e = expert_of(p);
-        if (e >= 0) j.place[p] += (int32_t)s_first[e];
+    for (uint32_t p = tid; p < pairs; p += GD_ROUTE_BATCH * GD_ROUTE_THREADS) {
+        int32_t e[GD_ROUTE_BATCH], rank[GD_ROUTE_BATCH];
+#pragma unroll
+        for (uint32_t i = 0; i < GD_ROUTE_BATCH; ++i)
+            rank[i] = p + i * GD_ROUTE_THREADS < pairs ? j.place[p + i * GD_ROUTE_THREADS] : -1;
+        experts_of(p, e);
+#pragma unroll
+        for (uint32_t i = 0; i < GD_ROUTE_BATCH; ++i) {
+            if (e[i] >= 0 && rank[i] >= 0) j.place[p + i * GD_ROUTE_THREADS] = rank[i] + (int32_t)s_first[e[i]];
+        }
     }
 }
 

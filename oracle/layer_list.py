@@ -151,16 +151,16 @@ def rotate_neighbours(x, positions, freq, mult):
     return y
 
 
-def chunk_attention(q, k, v, scale, chunk):
-    """q [T, H, D], k [T, G, D], v [T, G, V]: query head h reads key/value head h // (H // G); position i sees j <= i
-    of its own chunk of `chunk` positions (None: of all)."""
-    T, H = q.shape[:2]
+def chunk_attention(q, k, v, scale, chunk, first=0):
+    """q [N, H, D] of the positions from `first` on, k [T, G, D], v [T, G, V]: query head h reads key/value head
+    h // (H // G); position i sees j <= i of its own chunk of `chunk` positions (None: of all)."""
+    N, H = q.shape[:2]
     per = H // k.shape[1]
-    i = np.arange(T)
-    seen = i[:, None] >= i[None, :]
+    i, j = first + np.arange(N), np.arange(len(k))
+    seen = i[:, None] >= j[None, :]
     if chunk is not None:
-        seen &= (i[:, None] // chunk) == (i[None, :] // chunk)
-    out = np.zeros((T, H, v.shape[2]), q.dtype)
+        seen &= (i[:, None] // chunk) == (j[None, :] // chunk)
+    out = np.zeros((N, H, v.shape[2]), q.dtype)
     for h in range(H):
         s = np.where(seen, (q[:, h] @ k[:, h // per].T) * scale, -np.inf)
         s = np.exp(s - s.max(axis=1, keepdims=True))

@@ -84,14 +84,16 @@ def weights(cfg, seed):
 
 
 def save(folder, cfg, tensors):
-    """config.json and model.safetensors (BF16)."""
+    """config.json and model.safetensors (BF16; integer arrays as I32)."""
     os.makedirs(folder, exist_ok=True)
     with open(os.path.join(folder, "config.json"), "w") as f:
         json.dump(cfg, f)
     header, blob = {}, b""
     for name, a in tensors.items():
-        raw = _bf16(a).tobytes()
-        header[name] = {"dtype": "BF16", "shape": list(a.shape), "data_offsets": [len(blob), len(blob) + len(raw)]}
+        whole = np.issubdtype(np.asarray(a).dtype, np.integer)
+        raw = np.ascontiguousarray(a, np.int32).tobytes() if whole else _bf16(a).tobytes()
+        header[name] = {"dtype": "I32" if whole else "BF16", "shape": list(a.shape),
+                        "data_offsets": [len(blob), len(blob) + len(raw)]}
         blob += raw
     text = json.dumps(header).encode()
     with open(os.path.join(folder, "model.safetensors"), "wb") as f:
