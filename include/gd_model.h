@@ -2,14 +2,20 @@
  * gd_model.h - opening a stored model without knowing which one it is: a registry of the architectures this
  * library serves.  A path is either
  *   - a ".gdckpt" file of the reference's gpt_lm example (gd_checkpoint.h): "gpt_lm", or
- *   - a folder with config.json and model.safetensors, whose "architecture" names the model: "Girirax".
+ *   - a folder with config.json and model.safetensors, whose "architecture" names the model: "Girirax" or "Bonatar".
  * The decoder made from it is the one of gd_gpt_decoder.h: prefill, step, resident sessions, sampling and generation
  * are the same calls for every architecture.
  *
- * Configuration of a layer-list decoder ("Girirax"): vocab, width, norm.eps, residual_mult, embedding.scale and
- * layers[], every entry with its "type" and "mixer" sizes and its "mlp" ({"kind": "dense", "ff"} or null):
+ * Configuration of the layer-list decoders: vocab, width, norm.eps, embedding.scale and layers[], every entry with its
+ * "type" and "mixer" sizes and its "mlp" (or null).
+ * "Girirax": also residual_mult; mlp {"kind": "dense", "ff"}; types
  *   "mamba2"            heads, vdim, state, groups, norm_groups, conv (taps)
  *   "latent_attention"  heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, rot.base, rot.dims (= rot_dim)
+ * "Bonatar": a layer may name in "weights_of" another layer of the same sizes whose weights it uses; type
+ *   "attention"         heads, kv_heads, dim, vdim, scale, rot.base, rot.dims, rot.scaling {factor, original, fast, slow}
+ *                       (or none), mask.size (positions of a chunk; without mask: all)
+ *   mlp {"kind": "dense", "ff"}, or {"kind": "moe", "router": {experts, top}, "expert": {ff, limit},
+ *   "shared": {ff, limit} or null}
  */
 #ifndef GD_MODEL_H
 #define GD_MODEL_H

@@ -80,7 +80,8 @@ def test_forms_that_half_precision_does_not_have(backend, gda, arena):
 # ---- residual stream --------------------------------------------------------------------------------------
 
 @TYPES
-@pytest.mark.parametrize("N,W,top", [(1, 64, 1), (5, 36, 3), (9, 2048, 2), (3, 9000, 2), (2, 1, 1), (70, 200, 4)])
+@pytest.mark.parametrize("N,W,top", [(1, 64, 1), (5, 36, 3), (9, 2048, 2), (3, 9000, 2), (2, 1, 1), (70, 200, 4),
+                                     (1030, 512, 2), (1500, 2048, 1)])
 def test_add_and_norm(backend, gda, arena, dtype, N, W, top):
     """A branch, routed rows, both or neither; the norm for the next sublayer, packed for its experts or not."""
     rng = np.random.default_rng(N + W)
