@@ -169,6 +169,15 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
         const uint32_t wc = r / (BN / 2u), wr = r % (BN / 2u);
         return gated ? (wr < HW ? tn0 + wc * HW + wr : p.swiglu_cols + tn0 + wc * HW + (wr - HW)) : tn0 + r;
     };
+    /* first of 8 weight rows that a direct load of tile rows r .. r + 7 fetches.  GROUPED: a last column tile of fewer
+     * outputs (N % 8 == 0) takes the direct path too, with its last rows again in place of those behind them; what they
+     * give is not stored */
+    auto wrow_direct = [&](uint32_t tn0, uint32_t r) __attribute__((always_inline)) -> uint32_t {
+        if constexpr (!GROUPED) return wrow(tn0, r);
+        const uint32_t wc = r / (BN / 2u), wr = r % (BN / 2u);
+        if (!gated) return min(tn0 + r, p.N - 8u);
+        return (wr < HW ? 0u : p.swiglu_cols) + min(tn0 + wc * HW + wr % HW, p.N - 8u);
+    };
     auto wrow_ok = [&](uint32_t tn0, uint32_t r) __attribute__((always_inline)) {
         return (gated ? tn0 + (r / (BN / 2u)) * HW + r % HW : tn0 + r) < p.N;
     };
@@ -190,7 +199,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
         }
     };
     auto direct_ok = [&](uint32_t tm0, uint32_t tn0) __attribute__((always_inline)) {
-        return DIRECT && (GROUPED || tm0 + BM <= p.M) && tn0 + out_bn <= p.N && (p.K % 64u) == 0u && p.K >= 128u;
+        return DIRECT && (GROUPED || (tm0 + BM <= p.M && tn0 + out_bn <= p.N)) && (p.K % 64u) == 0u && p.K >= 128u;
     };
 
     uint32_t tid_opaque = threadIdx.x;
@@ -331,7 +340,7 @@ gd_linear_tile_kernel(const gd_elem *__restrict__ x, const gd_elem *__restrict__
         } else if (W_NK) {
             const uint32_t tb = t - (uint32_t)A_DIRECT;
             const uint32_t row0 = wave_u * (BN / 4u) + tb * RW;
-            gd_tile_load_lds16(wt + (size_t)wrow(tn0, row0) * p.ldw + kt * DBK, (tb & 1u) ? d_off_b1 : d_off_b,
+            gd_tile_load_lds16(wt + (size_t)wrow_direct(tn0, row0) * p.ldw + kt * DBK, (tb & 1u) ? d_off_b1 : d_off_b,
                                lds_base + ((2u * BM + stage * BN) * CH + row0 * CH) * 16u);
         } else {
             /* k-rows kr0 .. kr0+RPL-1 of the tile; lane L fills position L%CPR of row kr0 + L/CPR */
@@ -979,7 +988,7 @@ static int launch_tile_grouped(hipStream_t stream, const gd_elem *x, const gd_el
 }
 
 /* y rows packed by group = x rows times the group's weights: p as for gd_hip_launch_linear_tile (M: packed rows; [N,K]
- * weights, 16-byte aligned rows of x, w and y, no bias, no residual); max_tiles: upper bound of the row tiles, of 256
+ * weights, N % 8 == 0, 16-byte aligned rows of x, w and y, no bias, no residual); max_tiles: upper bound of the row tiles, of 256
  * (big_tiles) or 128 rows */
 extern "C" int gd_hip_launch_linear_tile_grouped_bf16(hipStream_t stream, const void *x, const void *w, void *y,
                                                       const gd_hip_linear_params *p, const int32_t *first,

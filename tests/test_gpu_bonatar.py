@@ -338,7 +338,7 @@ class Routed:
 @TYPES
 @pytest.mark.parametrize("E,K,W,F,N", [
     (5, 2, 64, 40, 3), (7, 1, 96, 24, 40), (3, 3, 30, 21, 11), (1, 1, 8, 8, 1), (16, 2, 256, 128, 33), (4, 2, 72, 8, 300),
-    (6, 2, 256, 128, 400), (3, 1, 192, 320, 500), (2, 2, 128, 256, 900), (3, 2, 256, 128, 1300), (2, 1, 512, 64, 1700), (300, 3, 64, 16, 70),
+    (6, 2, 256, 128, 400), (3, 1, 192, 320, 500), (2, 2, 128, 256, 900), (3, 2, 256, 128, 1300), (3, 2, 136, 200, 1200), (2, 1, 320, 192, 1600), (2, 1, 512, 64, 1700), (300, 3, 64, 16, 70),
     (9, 4, 128, 200, 260)])
 def test_routed_feed_forward(backend, gda, arena, dtype, E, K, W, F, N):
     """Few and many rows per expert, experts without rows, sizes on and off the tiles of every kernel."""
