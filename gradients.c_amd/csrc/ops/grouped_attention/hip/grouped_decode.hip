@@ -128,11 +128,7 @@ gd_grouped_decode_kernel(const gd_bf16 *__restrict__ proj, const float *__restri
     /* the angles of the position, while the first tiles are on their way */
     if (tid < STEPS * 16u) {
         float sn = 0.f, cs = 1.f;
-        if (tid < half) {
-            sincosf((float)pos * f, &sn, &cs);
-            sn *= m.rot_mult;
-            cs *= m.rot_mult;
-        }
+        if (tid < half) gd_grouped_angle(m, pos, f, &sn, &cs);
         s_cos[tid] = cs;
         s_sin[tid] = sn;
     }

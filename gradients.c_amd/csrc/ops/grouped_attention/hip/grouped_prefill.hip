@@ -35,11 +35,7 @@ gd_grouped_rotate_vec_kernel(gd_bf16 *__restrict__ proj, const float *__restrict
     for (uint32_t c = sub; c < m.half / 4u; c += lanes) {
         float cs[4], sn[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            sincosf((float)pos * freq[4u * c + (uint32_t)i], &sn[i], &cs[i]);
-            sn[i] *= m.rot_mult;
-            cs[i] *= m.rot_mult;
-        }
+        for (int i = 0; i < 4; ++i) gd_grouped_angle(m, pos, freq[4u * c + (uint32_t)i], &sn[i], &cs[i]);
         gd_bf16 *at = proj + (size_t)row * m.ld + c * 8u;
         for (uint32_t h0 = 0; h0 < heads; h0 += 4u) { /* the loads of four heads together */
             gd_bf16x8 v[4];

@@ -25,9 +25,7 @@ gd_grouped_rotate_kernel(T *__restrict__ proj, const float *__restrict__ freq, g
         const uint32_t h = i / m.half, p = i % m.half; /* the key heads follow the query heads */
         T *at = row + (size_t)h * m.dim + 2u * p;
         float s, c;
-        sincosf((float)pos * freq[p], &s, &c);
-        s *= m.rot_mult;
-        c *= m.rot_mult;
+        gd_grouped_angle(m, pos, freq[p], &s, &c);
         const float u = (float)at[0], v = (float)at[1];
         at[0] = (T)(u * c - v * s);
         at[1] = (T)(v * c + u * s);

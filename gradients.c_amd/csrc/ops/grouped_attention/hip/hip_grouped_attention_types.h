@@ -20,5 +20,16 @@ __device__ __forceinline__ int32_t gd_grouped_first(const gd_hip_grouped_params 
 {
     return m.chunk != 0u ? pos - pos % (int32_t)m.chunk : 0;
 }
+
+/* sine and cosine of pos * freq, times rot_mult.  What the product loses to rounding (for large angles more than the
+ * functions do) is put back to first order. */
+__device__ __forceinline__ void gd_grouped_angle(const gd_hip_grouped_params &m, int32_t pos, float freq, float *s, float *c)
+{
+    const float at = (float)pos, angle = at * freq, rest = fmaf(at, freq, -angle);
+    float sn, cs;
+    sincosf(angle, &sn, &cs);
+    *s = fmaf(cs, rest, sn) * m.rot_mult;
+    *c = fmaf(-sn, rest, cs) * m.rot_mult;
+}
 #endif
 #endif

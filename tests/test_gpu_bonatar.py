@@ -235,6 +235,16 @@ def test_a_key_is_seen_by_its_chunk_behind_it_and_by_no_other_row(backend, gda, 
         near(got, want, dtype, factor=2.5 if dtype == BF16 else 30)
 
 
+@TYPES
+def test_positions_far_from_the_start(backend, gda, arena, L, dtype):
+    """Angles of hundreds of thousands of turns, by portions and by steps, in the 50 places of a chunk."""
+    a = Grouped(gda, backend, arena, L, dtype, 4, 2, 16, 8, 16, 50, base=3.0)
+    start = 300000
+    a.k[1], a.v[1] = np.zeros((start, 2, 16)), np.zeros((start, 2, 8))
+    for runs in ([(1, start, 7)], [(1, start + 7, 1)], [(1, start + 8, 1)], [(1, start + 9, 60)], [(1, start + 69, 1)]):
+        near(*a.run(runs), dtype, **_tolerance(dtype))
+
+
 def test_slots_out_of_range_and_unfit_operands(backend, gda, arena, L):
     """Sequences with a slot or a start that does not exist leave the caches alone; operands that do not fit together
     are refused."""
